@@ -327,7 +327,7 @@ def qk_row_scales(proj, n_q_cols, n_k_cols, positions, bias=None, eps=None, temp
 
 def qkv_prepare(qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q_norm=None, k_norm=None, qk_eps=0.0,
                 rotation=None, value_norm_eps=None, value_rotation=None, k_cache=None, v_cache=None, slots=None, page_size=0,
-                bias=None, row_scales=None, norm_over_projection=False, values_from_keys=False):
+                bias=None, row_scales=None, norm_over_projection=False, values_from_keys=False, unweighted_norm=False):
     n = qkv.shape[0]
     x = qkv.to(torch.float32)
     if bias is not None:
@@ -344,6 +344,9 @@ def qkv_prepare(qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q
         q = q * q_norm.to(torch.float32).view(1, n_heads, head_dim)
         if n_kv:
             k = k * k_norm.to(torch.float32).view(1, n_kv, head_dim)
+    elif unweighted_norm:
+        q = q * torch.rsqrt((q * q).mean(-1, keepdim=True) + qk_eps)
+        k = k * torch.rsqrt((k * k).mean(-1, keepdim=True) + qk_eps)
     elif q_norm is not None:
         q = q * torch.rsqrt((q * q).mean(-1, keepdim=True) + qk_eps) * q_norm.to(torch.float32)
         k = k * torch.rsqrt((k * k).mean(-1, keepdim=True) + qk_eps) * k_norm.to(torch.float32)
@@ -366,7 +369,8 @@ def qkv_prepare(qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q
 
 
 def attention_masked(q, n_heads, n_kv, head_dim, value_dim, k_cache, v_cache, page_size, scale, ctx, group, window=0,
-                     keep_first=0, softcap=0.0, value_rotation=None, gate=None, gate_col=0, gate_elems=1, distance_bias=None, sink=None):
+                     keep_first=0, softcap=0.0, value_rotation=None, gate=None, gate_col=0, gate_elems=1, distance_bias=None, sink=None,
+                     chunked=False):
     n = q.shape[0]
     positions, token_seq = ctx.arrays["positions"], ctx.arrays["token_seq"]
     bt = ctx.arrays[f"block_table_g{group}"]
@@ -376,7 +380,9 @@ def attention_masked(q, n_heads, n_kv, head_dim, value_dim, k_cache, v_cache, pa
     for t in range(n):
         pos = int(positions[t])
         j = torch.arange(pos + 1, device=q.device)
-        if window:
+        if window and chunked:  # the query's own chunk of ``window`` positions
+            j = j[j >= pos - pos % window]
+        elif window:
             j = j[(pos - j < window) | (j < keep_first)]
         pages = bt[int(token_seq[t])][(j // page_size).long()].long()
         offs = (j % page_size).long()
@@ -612,8 +618,10 @@ def latent_attention(q_lat, pages, n_heads, kv_rank, rot_dim, scale, ctx, group,
 
 
 # ---------------------------------------------------------------- a matrix per head as the memory
-def causal_conv_act(x, weight, bias, state, ctx, act=None):
+def causal_conv_act(x, weight, bias, state, ctx, act=None, move_state=False):
     y = causal_conv(x, weight, bias, state, ctx)
+    if move_state and weight.shape[1] > 1:
+        conv_state_push(x, state, ctx)
     return y if act is None else activation(y, act, y.dtype)
 
 
@@ -626,7 +634,7 @@ def conv_state_push(x, state, ctx):
 
 
 def linear_state_scan(qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, unit_eps=None, decay=None, beta=None, columns=None,
-                      skip=None):
+                      skip=None, bonus=None):
     a = ctx.arrays
     n = qkv.shape[0]
     x = qkv.float()
@@ -642,6 +650,13 @@ def linear_state_scan(qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, un
         step = torch.nn.functional.softplus(src[:, col: col + n_heads].float() + dt_bias.float())
         g = torch.exp(-torch.exp(a_log.float()) * step)
         g = g[:, :, None].expand(n, n_heads, dim)
+    elif decay[0] == "channel_softplus":
+        _, src, col, a_log, dt_bias = decay
+        step = torch.nn.functional.softplus(src[:, col: col + n_heads * dim].float() + dt_bias.float()).view(n, n_heads, dim)
+        g = torch.exp(-torch.exp(a_log.float())[None, :, None] * step)
+    elif decay[0] == "channel_exp":
+        _, src, col, bias = decay
+        g = torch.exp(-torch.exp(src[:, col: col + n_heads * dim].float() + bias.float())).view(n, n_heads, dim)
     else:
         _, src, col, bias, tau = decay
         z = src[:, col: col + n_heads * dim].float() + bias.float()
@@ -657,6 +672,10 @@ def linear_state_scan(qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, un
             for h in range(n_heads):
                 kk, qq = k[t, h // per], q[t, h // per]
                 Sh = g[t, h][:, None] * S[h]
+                if bonus is not None:  # the memory as it was, and the token's own write weighed by the bonus
+                    out[t, h] = S[h].T @ qq + ((qq * bonus[h].float()) @ kk) * v[t, h]
+                    S[h] = Sh + torch.outer(kk, v[t, h])
+                    continue
                 u = v[t, h] if b is None else b[t, h] * (v[t, h] - Sh.T @ kk)
                 if by_step:
                     u = step[t, h] * v[t, h]
@@ -669,9 +688,12 @@ def linear_state_scan(qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, un
     return out.view(n, n_heads * vdim)
 
 
-def gated_head_norm(o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first=False):
+def gated_head_norm(o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first=False, gate_act="silu"):
     n = o.shape[0]
     g = gate[:, gate_col: gate_col + n_heads * vdim].float()
+    if gate_act == "sigmoid":
+        w = weight.float() if weight.numel() == vdim else weight.float().view(n_heads, vdim)
+        return (_rmsnorm(o.float().view(n, n_heads, vdim), w, eps, False).reshape(n, -1) * torch.sigmoid(g)).to(out_dtype)
     w = weight.float() if weight.numel() == vdim else weight.float().view(n_heads, vdim)
     if gate_first:
         return _rmsnorm((o.float() * g * torch.sigmoid(g)).view(n, n_heads, vdim), w, eps, False).reshape(n, -1).to(out_dtype)
@@ -709,6 +731,58 @@ def moe_combine(dense, rows, top, weight=1.0, row_weights=None):
     return out if dense is None else out + dense.float()
 
 
+# --------------------------------------------------- norms after sums, pairs of tokens, inputs mixed with the last one's
+def sum_norm(residual, terms, branch_scale, branch_weight, residual_scale, weight, eps, unit_offset, out_dtype):
+    b = torch.zeros_like(residual)
+    for rows, w, e in terms:
+        b = b + (rows.float() if w is None else _rmsnorm(rows.float(), w, e, False))
+    b = b * branch_scale
+    if branch_weight is not None:
+        b = b * branch_weight.float()
+    residual.copy_(_rmsnorm(residual_scale * residual + b, weight, eps, unit_offset))
+    return round_rows(residual, out_dtype)
+
+
+def embed_pairs(token_ids, table, scale, pair_table, buckets, mul_prev, mul_cur, state, ctx, act_dtype):
+    a = ctx.arrays
+    ids = [int(t) for t in token_ids]
+    rows = []
+    for s in range(a["seq_qstart"].numel()):
+        q0, ql, slot = int(a["seq_qstart"][s]), int(a["seq_qlen"][s]), int(a["state_slots"][s])
+        prev = int(state[slot, 0])
+        for t in range(q0, q0 + ql):
+            rows.append(buckets if prev < 0 else (prev * mul_prev + ids[t] * mul_cur) % buckets)
+            prev = ids[t]
+        state[slot, 0] = prev
+    out = embed(token_ids, table, scale=scale) + pair_table[torch.tensor(rows, device=table.device)].float()
+    return out, round_rows(out, act_dtype)
+
+
+def token_shift_mix(h, mu, state, ctx):
+    a = ctx.arrays
+    past = torch.empty_like(h)
+    for s in range(a["seq_qstart"].numel()):
+        q0, ql, slot = int(a["seq_qstart"][s]), int(a["seq_qlen"][s]), int(a["state_slots"][s])
+        past[q0] = state[slot]
+        past[q0 + 1: q0 + ql] = h[q0: q0 + ql - 1]
+        state[slot] = h[q0 + ql - 1]
+    x, p = h.float(), past.float()
+    return (x[None] + (p - x)[None] * mu[:, None, :]).to(h.dtype)
+
+
+def grouped_linear(x, w, group_rows, out_dtype):
+    return torch.cat([linear(x[g], w[g * group_rows: (g + 1) * group_rows], out_dtype) for g in range(x.shape[0])], dim=1)
+
+
+def low_rank(y, w, act=None):
+    return linear(torch.tanh(y.float()) if act == "tanh" else y, w, torch.float32)
+
+
+RefOps.sum_norm = staticmethod(sum_norm)
+RefOps.embed_pairs = staticmethod(embed_pairs)
+RefOps.token_shift_mix = staticmethod(token_shift_mix)
+RefOps.grouped_linear = staticmethod(grouped_linear)
+RefOps.low_rank = staticmethod(low_rank)
 RefOps.sandwich_norm = staticmethod(sandwich_norm)
 RefOps.activation = staticmethod(activation)
 RefOps.scale_rows = staticmethod(scale_rows)

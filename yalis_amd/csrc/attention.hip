@@ -4,7 +4,8 @@
 //
 // Arithmetic (reference: yalis/attention/backend_impl/sdpa_and_flex.py:59-90, 300-312):
 // score[h, p, j] = q[h, p] . k[h / (H/G), j] * scale; key j is visible to the query at
-// position p iff j <= p (and p - j < window when a window is set); softmax over the
+// position p iff j <= p (and p - j < window when a window is set, or floor(j / window) = floor(p / window) when it
+// is chunked); softmax over the
 // visible keys in float32; output = P . V.
 //
 // Page layout: keys [page][kv_head][page_size][head_dim], values transposed
@@ -134,7 +135,8 @@ extern "C" int yk_attn_generic(const void* q, int q_stride, void* out, const voi
 // and distance (a float32 table [distances][heads], the last row for everything farther) is added to
 // the scaled, squashed score; a sink per head (float32 [heads]) joins the softmax's denominator once as exp(sink):
 // where a column's keys are whole in one workgroup, when its sum of weights is inverted; where they were split,
-// in the merge of the splits (a split never adds it itself).
+// in the merge of the splits (a split never adds it itself); a chunked window begins anew at every multiple of its size
+// instead of sliding.
 //
 // Kept first keys add blocks of 64 keys in front of the window's: a kernel numbers the blocks it
 // walks "virtually", the window's blocks by their own number and the n_first blocks of kept keys
@@ -260,8 +262,8 @@ __global__ __launch_bounds__(64 * W, 2) void attn_mfma_kernel(
     int page_size, int n_heads, int n_kv, int hpt, int chunks, float scale_log2, int window,
     int n_splits, float* __restrict__ ws_o, float* __restrict__ ws_ml, RopeSrc rs, int keep_first_arg = 0,
     float cap_over_scale = 0.f, float scale_over_cap_2log2e = 0.f, const float* __restrict__ dist_bias = nullptr,
-    int bias_rows = 0, float inv_scale = 0.f, const float* __restrict__ sink = nullptr) {
-  const int keep_first = EXT ? keep_first_arg : 0;
+    int bias_rows = 0, float inv_scale = 0.f, const float* __restrict__ sink = nullptr, int chunked_arg = 0) {
+  const int keep_first = EXT ? keep_first_arg : 0, chunked = EXT ? chunked_arg : 0;
   constexpr int KS = D / 32;  // matrix-core steps over the head dimension
   constexpr int DT = D / 16;  // output tiles over the head dimension
   constexpr bool ROPE = SRC != 0;  // SRC 0: queries from `q`; 1, 2: rotary + append in here (rope_src_load8)
@@ -278,9 +280,9 @@ __global__ __launch_bounds__(64 * W, 2) void attn_mfma_kernel(
   const int tt = r / hpt, hh = r % hpt;
   const bool col_ok = tt < ntok && hh < heads_here;
   const int pos_c = pos0 + tt;
-  const int lo_c = window > 0 ? max(0, pos_c - window + 1) : 0;
+  const int lo_c = first_visible(pos_c, window, chunked);
   const int hi = pos0 + ntok;
-  const int lo = window > 0 ? max(0, pos0 - window + 1) : 0;
+  const int lo = first_visible(pos0, window, chunked);
   // (blocks are numbered virtually: those of kept first keys sit just below the window's first)
   const int win_lo = lo / 64;
   const int n_first = EXT ? ext_first_blocks(keep_first, window, lo) : 0;
@@ -537,7 +539,7 @@ __global__ __launch_bounds__(64 * W, 2) void attn_mfma_kernel(
     // a block that every column sees whole needs no mask (columns that stand for nothing
     // compute on zeros and are never stored)
     const bool whole = mine0 && mine1 && akb * 64 + 63 <= pos0 &&
-                       (window == 0 || akb * 64 >= max(0, pos0 + ntok - window) || (EXT && akb * 64 + 64 <= keep_first));
+                       (window == 0 || akb * 64 >= first_visible(pos0 + ntok - 1, window, chunked) || (EXT && akb * 64 + 64 <= keep_first));
     if (EXT && cap_over_scale > 0.f) {
 #pragma unroll
       for (int u = 0; u < 2; ++u)
@@ -721,9 +723,9 @@ __global__ __launch_bounds__(256, CT == 1 ? 3 : 2) void attn_mfma_prefill_kernel
     int page_size, int n_heads, int n_kv, int hpt, int chunks, float scale_log2, int window,
     int n_splits, float* __restrict__ ws_o, float* __restrict__ ws_ml, int pages_lds_limit, int keep_first_arg,
     float cap_over_scale, float scale_over_cap_2log2e, const float* __restrict__ dist_bias, int bias_rows, float inv_scale,
-    const float* __restrict__ sink) {
+    const float* __restrict__ sink, int chunked_arg) {
   constexpr int KS = D / 32, DT = D / 16;
-  const int keep_first = EXT ? keep_first_arg : 0;
+  const int keep_first = EXT ? keep_first_arg : 0, chunked = EXT ? chunked_arg : 0;
   constexpr int KROW = D + 8;   // bf16 elements per parked key row
   constexpr int VROW = 64 + 8;  // bf16 elements per parked value row
   constexpr int PP = D / 32;    // 16-byte pieces of keys (and of values) per thread and block
@@ -753,11 +755,12 @@ __global__ __launch_bounds__(256, CT == 1 ? 3 : 2) void attn_mfma_prefill_kernel
     tok_c[c] = wave_tok0 + c * tpt + tt;
     col_ok[c] = tt < tpt && tok_c[c] < tile_ntok && hh < heads_here;
     pos_c[c] = tile_pos0 + tok_c[c];
-    lo_c[c] = window > 0 ? max(0, pos_c[c] - window + 1) : 0;
+    lo_c[c] = first_visible(pos_c[c], window, chunked);
   }
   const int hi = tile_pos0 + tile_ntok;  // keys the workgroup may need
-  const int lo = window > 0 ? max(0, tile_pos0 - window + 1) : 0;
+  const int lo = first_visible(tile_pos0, window, chunked);
   const int wave_hi = min(hi, tile_pos0 + wave_tok0 + CT * tpt);  // keys this wave may need
+  const int wave_lo = first_visible(tile_pos0 + wave_tok0, window, chunked);  // the first key any column of this wave sees in its window
   // the workgroup's share of the key blocks when a launch splits them (blockIdx.y): few long
   // tiles against a long context would otherwise leave most of the GPU idle
   // (blocks are numbered virtually: those of kept first keys sit just below the window's first)
@@ -901,6 +904,7 @@ __global__ __launch_bounds__(256, CT == 1 ? 3 : 2) void attn_mfma_prefill_kernel
     if (vb + 1 < kb_hi) { PF_LOAD(vb + 1) }  // in flight while this block is worked on
     const int key0 = kb * 64;
     if (key0 >= wave_hi) continue;  // nothing of this block is visible to this wave
+    if (EXT && chunked && key0 + 64 <= wave_lo) continue;
 
     f32x4_t s[CT][2][2];
 #pragma unroll
@@ -921,7 +925,7 @@ __global__ __launch_bounds__(256, CT == 1 ? 3 : 2) void attn_mfma_prefill_kernel
     // keys that every column sees whole need no mask (columns that stand for nothing
     // compute on zeros and are never stored)
     const bool whole = key0 + 63 <= (tile_pos0 + wave_tok0) &&
-                       (window == 0 || key0 >= max(0, wave_hi - window) || (EXT && key0 + 64 <= keep_first));
+                       (window == 0 || key0 >= first_visible(max(wave_hi - 1, 0), window, chunked) || (EXT && key0 + 64 <= keep_first));
     if (EXT && cap_over_scale > 0.f) {
 #pragma unroll
       for (int c = 0; c < CT; ++c)
@@ -1110,8 +1114,9 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
                                     int head_dim, int n_heads, int n_kv, float scale, int window,
                                     int n_splits, int col_tiles, float* workspace, size_t workspace_floats,
                                     int pages_lds_limit, int keep_first, float softcap, const float* dist_bias, int bias_rows,
-                                    const float* sink, hipStream_t stream) {
+                                    const float* sink, int chunked, hipStream_t stream) {
   YK_REQUIRE(n_tiles >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attn_mfma_prefill: bad head counts");
+  YK_REQUIRE(!chunked || (window > 0 && keep_first == 0), "attn_mfma_prefill: chunks need their size and keep no first keys");
   YK_REQUIRE(col_tiles == 1 || col_tiles == 2, "attn_mfma_prefill: a wave has 1 or 2 column tiles");
   YK_REQUIRE(yk_attn_mfma_supported(head_dim), "attn_mfma_prefill: head_dim must be 64 or 128");
   YK_REQUIRE(page_size > 0 && page_size % 16 == 0, "attn_mfma_prefill: page_size must be a multiple of 16");
@@ -1124,7 +1129,7 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
   YK_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attn_mfma_prefill: keep_first and softcap must not be negative");
   YK_REQUIRE(dist_bias == nullptr || bias_rows >= 1, "attn_mfma_prefill: an empty table of biases");
   if (n_tiles == 0) return 0;
-  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr;
+  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr || chunked;
   const float inv_scale = 1.f / scale;
   const float cap_over_scale = softcap > 0.f ? softcap / scale : 0.f;
   const float scale_over_cap = softcap > 0.f ? scale / softcap * 2.f * 1.4426950408889634f : 0.f;
@@ -1142,7 +1147,7 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
   static_cast<const bf16_t*>(q), q_stride, static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_cache),     \
       static_cast<const bf16_t*>(v_cache), tiles, block_table, table_width, page_size, n_heads, n_kv, hpt,     \
       chunks, scale_log2, window, n_splits, ws_o, ws_ml, pages_lds_limit, keep_first, cap_over_scale, scale_over_cap, \
-      dist_bias, bias_rows, inv_scale, sink
+      dist_bias, bias_rows, inv_scale, sink, chunked
 #define YK_PF(DD, BIP)                                                                                       \
   if (ext && col_tiles == 2)                                                                                 \
     attn_mfma_prefill_kernel<DD, BIP, 2, true><<<grid, block, 0, stream>>>(YK_PF_ARGS);                      \
@@ -1181,12 +1186,14 @@ static int launch_attn_mfma(const void* q, int q_stride, void* out, const void* 
                             int page_size, int head_dim, int n_heads, int n_kv, float scale, int window,
                             int n_waves, int n_splits, float* workspace, size_t workspace_floats,
                             int leave_splits, const RopeSrc* rope, bool rope_f32, hipStream_t stream, int keep_first = 0,
-                            float softcap = 0.f, const float* dist_bias = nullptr, int bias_rows = 0, const float* sink = nullptr) {
+                            float softcap = 0.f, const float* dist_bias = nullptr, int bias_rows = 0, const float* sink = nullptr,
+                            int chunked = 0) {
+  YK_REQUIRE(!chunked || (window > 0 && keep_first == 0), "attn_mfma: chunks need their size and keep no first keys");
   YK_REQUIRE(n_tiles >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attn_mfma: bad head counts");
   YK_REQUIRE(sink == nullptr || !leave_splits, "attn_mfma: splits that another kernel merges cannot carry a sink");
   YK_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attn_mfma: keep_first and softcap must not be negative");
   YK_REQUIRE(dist_bias == nullptr || bias_rows >= 1, "attn_mfma: an empty table of biases");
-  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr;
+  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr || chunked;
   const float inv_scale = scale > 0.f ? 1.f / scale : 0.f;
   YK_REQUIRE(!(ext && rope), "attn_mfma: kept first keys and squashed scores are not offered with rotary inside the launch");
   const float cap_over_scale = softcap > 0.f ? softcap / scale : 0.f;
@@ -1227,11 +1234,11 @@ static int launch_attn_mfma(const void* q, int q_stride, void* out, const void* 
   }
 #define YK_LAUNCH_EXT(DD)                                                                          \
   if (tiled) {                                                                                     \
-    if (n_waves == 1) attn_mfma_kernel<DD, 1, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink); \
-    else attn_mfma_kernel<DD, 4, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink); \
+    if (n_waves == 1) attn_mfma_kernel<DD, 1, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
+    else attn_mfma_kernel<DD, 4, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
   } else {                                                                                         \
-    if (n_waves == 1) attn_mfma_kernel<DD, 1, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink); \
-    else attn_mfma_kernel<DD, 4, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink); \
+    if (n_waves == 1) attn_mfma_kernel<DD, 1, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
+    else attn_mfma_kernel<DD, 4, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
   }
 #define YK_LAUNCH(DD)                                                                              \
   if (ext) { YK_LAUNCH_EXT(DD) } else                                                              \
@@ -1260,10 +1267,10 @@ extern "C" int yk_attn_mfma(const void* q, int q_stride, void* out, const void* 
                             int head_dim, int n_heads, int n_kv, float scale, int window,
                             int n_waves, int n_splits, float* workspace, size_t workspace_floats,
                             int leave_splits, int keep_first, float softcap, const float* dist_bias, int bias_rows,
-                            const float* sink, hipStream_t stream) {
+                            const float* sink, int chunked, hipStream_t stream) {
   return launch_attn_mfma(q, q_stride, out, k_cache, v_cache, tiles, n_tiles, block_table, table_width, page_size,
                           head_dim, n_heads, n_kv, scale, window, n_waves, n_splits, workspace, workspace_floats,
-                          leave_splits, nullptr, false, stream, keep_first, softcap, dist_bias, bias_rows, sink);
+                          leave_splits, nullptr, false, stream, keep_first, softcap, dist_bias, bias_rows, sink, chunked);
 }
 
 // yk_attn_mfma for a step of single tokens (every tile holds ONE token), with rotary + append

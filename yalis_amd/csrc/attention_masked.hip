@@ -13,7 +13,7 @@
 //    that inverse root mean square and / or the queries' temperature 1 + coef ln(floor((p + 1) / every) + 1).
 //  * yk_attn_masked: scores q . k * scale, optionally squashed s <- cap * tanh(s / cap); key j
 //    is visible to the query at position p iff j <= p and (p - j < window or j < keep_first)
-//    (window 0: no window); softmax over the visible keys; keys of head_dim, values of
+//    (window 0: no window), or, chunked, floor(j / window) = floor(p / window); softmax over the visible keys; keys of head_dim, values of
 //    value_dim elements.  One wave per (token, head), float32 arithmetic, any sizes up to 256.
 //    Its epilogue can turn the output back by the query's own position (the inverse of the
 //    values' rotation) and multiply a head's output by the sigmoid of a gate column of the
@@ -511,7 +511,7 @@ __global__ __launch_bounds__(64) void attn_masked_kernel(
     int n_kv, float scale, float softcap, int window, int keep_first, int tiled, const float* __restrict__ v_cos,
     const float* __restrict__ v_sin, int v_interleaved, int v_max_pos, const TG* __restrict__ gate_src,
     int gate_splits, size_t gate_split_stride, int gate_round, int gate_stride, int gate_col0, int gate_elems,
-    const float* __restrict__ dist_bias, int bias_rows, const float* __restrict__ sink) {
+    const float* __restrict__ dist_bias, int bias_rows, const float* __restrict__ sink, int chunked) {
   const size_t slab_k = static_cast<size_t>(page_size) * head_dim, slab_v = static_cast<size_t>(page_size) * v_dim;
   __shared__ float qs[kMaxHead];
   __shared__ float os[kMaxHead];
@@ -521,7 +521,7 @@ __global__ __launch_bounds__(64) void attn_masked_kernel(
   const int n = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int qpk = n_heads / n_kv, g = h / qpk;
   const int pos = positions[n], seq = token_seq[n];
-  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int lo = first_visible(pos, window, chunked);
   const int n_first = min(keep_first, lo);  // keys below the window that stay visible
   const int total = n_first + (pos + 1 - lo);
   const T* qrow = q + static_cast<size_t>(n) * q_stride + static_cast<size_t>(h) * head_dim;
@@ -611,7 +611,8 @@ extern "C" int yk_attn_masked(const void* q, int q_stride, void* out, const void
                               float scale, float softcap, int window, int keep_first, int tiled, const float* v_cos,
                               const float* v_sin, int v_interleaved, int v_max_pos, const void* gate_src, int gate_dtype,
                               int gate_splits, int gate_round, int gate_stride, int gate_col0, int gate_elems,
-                              const float* dist_bias, int bias_rows, const float* sink, hipStream_t stream) {
+                              const float* dist_bias, int bias_rows, const float* sink, int chunked, hipStream_t stream) {
+  YK_REQUIRE(!chunked || (window > 0 && keep_first == 0), "attn_masked: chunks need their size and keep no first keys");
   YK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attn_masked: bad head counts");
   YK_REQUIRE(gate_src == nullptr || gate_elems == 1 || gate_elems == v_dim, "attn_masked: a gate per head or per output element");
   YK_REQUIRE(dist_bias == nullptr || bias_rows >= 1, "attn_masked: an empty table of biases");
@@ -632,7 +633,7 @@ extern "C" int yk_attn_masked(const void* q, int q_stride, void* out, const void
         static_cast<const T*>(v_cache), positions, token_seq, block_table, table_width, page_size, head_dim,   \
         v_dim, n_heads, n_kv, scale, softcap, window, keep_first, tiled, v_cos, v_sin, v_interleaved, v_max_pos, \
         static_cast<const TG*>(gate_src), gate_splits, gstride, gate_round, gate_stride, gate_col0, gate_elems, \
-        dist_bias, bias_rows, sink);                                                                           \
+        dist_bias, bias_rows, sink, chunked);                                                                  \
     return yk_check_launch("attn_masked");                                                                     \
   }
   YK_CASE(YK_F32, float, YK_F32, float)

@@ -28,6 +28,7 @@ struct Group {
   int32_t num_pages = 0;
   int32_t window = 0;  // 0: keep everything
   int32_t keep_first = 0;  // with a window: the first tokens that stay readable (their pages are never given back)
+  bool chunked = false;    // the window does not slide: it begins anew at every multiple of its size
   std::deque<int32_t> free_pages;
 };
 
@@ -66,9 +67,10 @@ extern "C" {
 const char* ycm_last_error() { return g_error.c_str(); }
 
 // windows[g] == 0 means the group keeps every token; keep_first[g] tokens at the start of every
-// request stay whatever the window says (keep_first may be null: none).
+// request stay whatever the window says (keep_first may be null: none).  chunked[g] != 0 (may be null):
+// the group's window does not slide, a token reads its own chunk of windows[g] positions only.
 void* ycm_create(int32_t page_size, int32_t num_groups, const int32_t* num_pages,
-                 const int32_t* windows, const int32_t* keep_first, int32_t num_slots) {
+                 const int32_t* windows, const int32_t* keep_first, const int32_t* chunked, int32_t num_slots) {
   if (page_size <= 0 || num_groups < 0 || num_slots <= 0) {
     g_error = "ycm_create: page_size and num_slots must be positive";
     return nullptr;
@@ -87,6 +89,7 @@ void* ycm_create(int32_t page_size, int32_t num_groups, const int32_t* num_pages
     m->groups[g].num_pages = num_pages[g];
     m->groups[g].window = windows[g];
     m->groups[g].keep_first = keep_first ? keep_first[g] : 0;
+    m->groups[g].chunked = chunked && chunked[g] != 0;
     for (int32_t p = 0; p < num_pages[g]; ++p) m->groups[g].free_pages.push_back(p);
   }
   return m;
@@ -156,7 +159,8 @@ int32_t ycm_reserve(void* h, int64_t req, int64_t total_tokens) {
 // window give back every page that no later token can read (but never a page with one of
 // the group's kept first tokens): the next query sits
 // at position >= cached_tokens and reads keys j with position - j < window, so
-// keys j <= cached_tokens - window are dead.  Returns the number of pages freed.
+// keys j <= cached_tokens - window are dead; where the window is chunked it reads the keys of its own
+// chunk, so the keys of every chunk before cached_tokens' own are dead.  Returns the number of pages freed.
 int32_t ycm_advance(void* h, int64_t req, int64_t cached_tokens) {
   auto* m = static_cast<Manager*>(h);
   auto it = m->requests.find(req);
@@ -166,7 +170,8 @@ int32_t ycm_advance(void* h, int64_t req, int64_t cached_tokens) {
   for (size_t g = 0; g < m->groups.size(); ++g) {
     int32_t w = m->groups[g].window;
     if (w <= 0) continue;
-    int64_t dead_tokens = cached_tokens - w + 1;  // keys 0 .. dead_tokens-1 are dead
+    // keys 0 .. dead_tokens-1 are dead
+    int64_t dead_tokens = m->groups[g].chunked ? cached_tokens - cached_tokens % w : cached_tokens - w + 1;
     if (dead_tokens <= 0) continue;
     int64_t dead_pages = dead_tokens / m->page_size;  // whole pages only
     dead_pages = std::min<int64_t>(dead_pages, static_cast<int64_t>(r.tables[g].size()));

@@ -171,6 +171,14 @@ __device__ __forceinline__ float as_output(float v, int round_sum) {
 __device__ __forceinline__ float rot_first(float a, float b, float c, float s) { return fmaf(a, c, -__fmul_rn(b, s)); }
 __device__ __forceinline__ float rot_second(float a, float b, float c, float s) { return fmaf(b, c, __fmul_rn(a, s)); }
 
+// The first key that the query at position p sees: with a window, the window's first position; with `chunked`, the first
+// position of the query's own chunk of `window` positions, counted from the sequence's start; without one, 0.
+__host__ __device__ inline int first_visible(int p, int window, int chunked) {
+  if (window <= 0) return 0;
+  if (chunked) return p - p % window;
+  return p - window + 1 > 0 ? p - window + 1 : 0;
+}
+
 // ------------------------------------------------ attention whose keys were split across workgroups
 // Heads of one kv head that share a wave of the matrix-core attention (its 16 columns hold
 // 16 / heads_per_tile tokens of those heads); a kv group with more heads takes several

@@ -106,6 +106,87 @@ extern "C" int yk_embed(const int32_t* ids, const void* table, int table_dtype, 
   return yk_check_launch("embed");
 }
 
+// ---------------------------------------------------------- embedding of tokens and pairs
+// out[n, :] = table[id_n] * scale + pair_table[row], row = (before * mul_prev + id_n * mul_cur) mod buckets, or the row
+// `buckets` for a request's first token.  The token before a span's first one is the request's state (-1: there is none);
+// the workgroup of a span's first token alone reads it, and leaves the span's last token there.  `rounded` (or null): the
+// row in bfloat16 beside the float32 one.  A workgroup a token.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(256) void embed_pairs_kernel(
+    const int32_t* __restrict__ ids, const T* __restrict__ table, int vocab, float scale, const T* __restrict__ pair_table, int buckets,
+    uint64_t mul_prev, uint64_t mul_cur, int32_t* __restrict__ state, const int32_t* __restrict__ token_seq,
+    const int32_t* __restrict__ seq_qstart, const int32_t* __restrict__ seq_qlen, const int32_t* __restrict__ state_slots,
+    float* __restrict__ out, bf16_t* __restrict__ rounded, int width) {
+  const int n = blockIdx.x, seq = token_seq[n], q0 = seq_qstart[seq];
+  // (ids are checked on the host; clamped so that a bad id cannot read out of bounds)
+  auto valid = [&](int id) { return min(max(id, 0), vocab - 1); };
+  const int id = valid(ids[n]);
+  int before;
+  if (n == q0) {
+    int32_t* st = state + state_slots[seq];
+    before = min(*st, vocab - 1);
+    __syncthreads();  // every thread has read the state
+    if (threadIdx.x == 0) *st = valid(ids[q0 + seq_qlen[seq] - 1]);
+  } else {
+    before = valid(ids[n - 1]);
+  }
+  const int row = before < 0 ? buckets
+                             : static_cast<int>((static_cast<uint64_t>(before) * mul_prev + static_cast<uint64_t>(id) * mul_cur) %
+                                                static_cast<uint64_t>(buckets));
+  const T* a = table + static_cast<size_t>(id) * width;
+  const T* b = pair_table + static_cast<size_t>(row) * width;
+  float* dst = out + static_cast<size_t>(n) * width;
+  bf16_t* rnd = rounded != nullptr ? rounded + static_cast<size_t>(n) * width : nullptr;
+  if (VEC) {
+    for (int c = 4 * threadIdx.x; c < width; c += 4 * blockDim.x) {
+      float4 v;
+      if constexpr (sizeof(T) == 2) {
+        const uint2 x = *reinterpret_cast<const uint2*>(a + c), y = *reinterpret_cast<const uint2*>(b + c);
+        v = make_float4(fmaf(__uint_as_float(x.x << 16), scale, __uint_as_float(y.x << 16)),
+                        fmaf(__uint_as_float(x.x & 0xffff0000u), scale, __uint_as_float(y.x & 0xffff0000u)),
+                        fmaf(__uint_as_float(x.y << 16), scale, __uint_as_float(y.y << 16)),
+                        fmaf(__uint_as_float(x.y & 0xffff0000u), scale, __uint_as_float(y.y & 0xffff0000u)));
+      } else {
+        const float4 x = *reinterpret_cast<const float4*>(a + c), y = *reinterpret_cast<const float4*>(b + c);
+        v = make_float4(fmaf(x.x, scale, y.x), fmaf(x.y, scale, y.y), fmaf(x.z, scale, y.z), fmaf(x.w, scale, y.w));
+      }
+      *reinterpret_cast<float4*>(dst + c) = v;
+      if (rnd != nullptr) *reinterpret_cast<uint2*>(rnd + c) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
+    }
+    return;
+  }
+  for (int c = threadIdx.x; c < width; c += blockDim.x) {
+    const float v = fmaf(to_f32<T>(a[c]), scale, to_f32<T>(b[c]));
+    dst[c] = v;
+    if (rnd != nullptr) rnd[c] = f32_to_bf16(v);
+  }
+}
+
+extern "C" int yk_embed_pairs(const int32_t* ids, const void* table, int table_dtype, int vocab, float scale, const void* pair_table,
+                              int buckets, unsigned long long mul_prev, unsigned long long mul_cur, int32_t* state,
+                              const int32_t* token_seq, const int32_t* seq_qstart, const int32_t* seq_qlen,
+                              const int32_t* state_slots, float* out, void* rounded, int n_tokens, int width, hipStream_t stream) {
+  YK_REQUIRE(n_tokens >= 0 && width > 0 && vocab > 0 && buckets > 0, "embed_pairs: bad sizes");
+  YK_REQUIRE(state != nullptr && pair_table != nullptr, "embed_pairs: the pairs' table or the requests' last tokens are missing");
+  if (n_tokens == 0) return 0;
+  auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const bool vec = width % 4 == 0 && al16(table) && al16(pair_table) && al16(out) && al16(rounded);
+#define YK_CASE(D, T, V)                                                                                                       \
+  if (table_dtype == D && vec == V) {                                                                                          \
+    embed_pairs_kernel<T, V><<<n_tokens, 256, 0, stream>>>(ids, static_cast<const T*>(table), vocab, scale,                    \
+                                                           static_cast<const T*>(pair_table), buckets, mul_prev, mul_cur,      \
+                                                           state, token_seq, seq_qstart, seq_qlen, state_slots, out,           \
+                                                           static_cast<bf16_t*>(rounded), width);                              \
+    return yk_check_launch("embed_pairs");                                                                                     \
+  }
+  YK_CASE(YK_F32, float, true)
+  YK_CASE(YK_F32, float, false)
+  YK_CASE(YK_BF16, bf16_t, true)
+  YK_CASE(YK_BF16, bf16_t, false)
+#undef YK_CASE
+  return yk_fail("embed_pairs: unsupported table dtype");
+}
+
 // ---------------------------------------------------------------- four-wide accessors
 template <typename T>
 __device__ __forceinline__ float4 load4(const T* p);

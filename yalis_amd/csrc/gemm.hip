@@ -188,7 +188,8 @@ constexpr int SK_SPLITS_MAX_K_BLOCK = 1024;  // a workgroup's whole slice of x t
 template <int MT, int W, typename TO, int GATED, bool FROM_SPLITS, int KC, int DEPTH = 1>
 __global__ __launch_bounds__(W * 64) void gemm_mfma_skinny_kernel(
     const bf16_t* __restrict__ x, const bf16_t* __restrict__ w, float* __restrict__ part,
-    TO* __restrict__ y, int M, int N, int K, int ldx, int ldw, int ldy, int k_block, AttnSplits xa) {
+    TO* __restrict__ y, int M, int N, int K, int ldx, int ldw, int ldy, int k_block, AttnSplits xa, int xg_rows = 0,
+    size_t xg_stride = 0) {
   static_assert(!FROM_SPLITS || (MT == 1 && GATED == 0), "unmerged attention feeds plain products of up to 16 rows");
   extern __shared__ __attribute__((aligned(16))) bf16_t lds[];
   constexpr int STEPS = KC / 32;               // matrix-core steps per chunk
@@ -208,6 +209,8 @@ __global__ __launch_bounds__(W * 64) void gemm_mfma_skinny_kernel(
   const int m0 = blockIdx.y * (16 * MT);
   const int kb0 = blockIdx.z * k_block;
   const int kb1 = min(K, kb0 + k_block);
+  // rows of x of this workgroup's own where the weight's rows come in groups (a workgroup never spans two groups)
+  if (xg_rows > 0) x += static_cast<size_t>(blockIdx.x * (W * 16) / xg_rows) * xg_stride;
 
   f32x4_t acc[MT];
 #pragma unroll
@@ -679,7 +682,7 @@ extern "C" int yk_gemm_skinny_splits(int M, int N, int K, int gated) { return sk
 template <typename TO>
 static int launch_skinny(const bf16_t* x, const bf16_t* w, float* part, TO* y, int M, int N, int K,
                          int ldx, int ldw, int ldy, int waves, int k_block, int splits, int gated, hipStream_t stream,
-                         const AttnSplits* from_splits = nullptr) {
+                         const AttnSplits* from_splits = nullptr, int xg_rows = 0, size_t xg_stride = 0) {
   const int mt = skinny_mt(M);
   if (from_splits) {
     // x is attention's unmerged splits: one kernel form (up to 16 rows, four waves, no activation)
@@ -762,7 +765,7 @@ static int launch_skinny(const bf16_t* x, const bf16_t* w, float* part, TO* y, i
         return yk_fail("gemm_mfma_skinny: cannot raise the LDS limit");                                 \
       raised = true;                                                                                    \
     }                                                                                                   \
-    gemm_mfma_skinny_kernel<MT_, W_, TO, G_, false, KC_, D_><<<grid, block, lds, stream>>>(x, w, part, y, M, N, K, ldx, ldw, ldy, k_block, AttnSplits{}); \
+    gemm_mfma_skinny_kernel<MT_, W_, TO, G_, false, KC_, D_><<<grid, block, lds, stream>>>(x, w, part, y, M, N, K, ldx, ldw, ldy, k_block, AttnSplits{}, xg_rows, xg_stride); \
     return yk_check_launch("gemm_mfma_skinny");                                                         \
   }
   SK_GO_KC(4, 8, 0, 128, 2)
@@ -779,19 +782,19 @@ static int launch_skinny(const bf16_t* x, const bf16_t* w, float* part, TO* y, i
 // unless the caller keeps them.  x, or (from_splits) attention's unmerged splits in its place.
 static int skinny_product(const bf16_t* xp, const AttnSplits* from_splits, const bf16_t* wp, void* y, int y_dtype,
                           float* workspace, size_t workspace_floats, int M, int N, int K, int ldx, int ldw, int ldy,
-                          int keep_splits, int gated, hipStream_t stream) {
+                          int keep_splits, int gated, hipStream_t stream, int xg_rows = 0, size_t xg_stride = 0) {
   int k_block = 0, waves = 4;
   const int splits = skinny_plan(M, N, K, gated != 0, &waves, &k_block);
   YK_REQUIRE(!gated || splits == 1, "gemm_mfma_skinny: a gated product cannot split K");
   if (splits == 1 && !keep_splits) {
     int rc = y_dtype == YK_F32
-                 ? launch_skinny<float>(xp, wp, nullptr, static_cast<float*>(y), M, N, K, ldx, ldw, ldy, waves, k_block, 1, gated, stream, from_splits)
-                 : launch_skinny<bf16_t>(xp, wp, nullptr, static_cast<bf16_t*>(y), M, N, K, ldx, ldw, ldy, waves, k_block, 1, gated, stream, from_splits);
+                 ? launch_skinny<float>(xp, wp, nullptr, static_cast<float*>(y), M, N, K, ldx, ldw, ldy, waves, k_block, 1, gated, stream, from_splits, xg_rows, xg_stride)
+                 : launch_skinny<bf16_t>(xp, wp, nullptr, static_cast<bf16_t*>(y), M, N, K, ldx, ldw, ldy, waves, k_block, 1, gated, stream, from_splits, xg_rows, xg_stride);
     return rc;
   }
   YK_REQUIRE(workspace && workspace_floats >= static_cast<size_t>(splits) * M * N,
              "gemm_mfma_skinny: workspace too small");
-  if (launch_skinny<float>(xp, wp, workspace, nullptr, M, N, K, ldx, ldw, ldy, waves, k_block, splits, 0, stream, from_splits)) return -1;
+  if (launch_skinny<float>(xp, wp, workspace, nullptr, M, N, K, ldx, ldw, ldy, waves, k_block, splits, 0, stream, from_splits, xg_rows, xg_stride)) return -1;
   if (keep_splits) return splits;
   const size_t total = static_cast<size_t>(M) * N;
   const int rb = 256;
@@ -826,6 +829,27 @@ extern "C" int yk_gemm_mfma_skinny(const void* x, const void* w, void* y, int y_
   if (M == 0) return 0;
   return skinny_product(static_cast<const bf16_t*>(x), nullptr, static_cast<const bf16_t*>(w), y, y_dtype, workspace,
                         workspace_floats, M, N, K, ldx, ldw, ldy, keep_splits, gated, stream);
+}
+
+// The few-row product where the weight's rows come in groups of `group_rows`, each with rows of x of its own: group g reads x
+// + g * group_stride (elements), M rows a group; y [M, N] has the groups' columns side by side (the last group may have fewer
+// rows).  Up to 32 rows of x, and groups of a multiple of 64 rows (a workgroup's rows then never span two of them).
+extern "C" int yk_gemm_mfma_skinny_grouped(const void* x, size_t group_stride, int group_rows, const void* w, void* y, int y_dtype,
+                                           float* workspace, size_t workspace_floats, int M, int N, int K, int ldx, int ldw,
+                                           int ldy, hipStream_t stream) {
+  YK_REQUIRE(M >= 0 && M <= 32 && N > 0 && K > 0, "gemm_mfma_skinny_grouped: bad sizes (up to 32 rows of x)");
+  YK_REQUIRE(group_rows > 0 && group_rows % 64 == 0, "gemm_mfma_skinny_grouped: groups are a multiple of 64 rows");
+  YK_REQUIRE(K >= 8 && K % 8 == 0 && ldx % 8 == 0 && ldw % 8 == 0 && group_stride % 8 == 0,
+             "gemm_mfma_skinny_grouped: K, the leading dimensions and the groups' distance must be multiples of 8");
+  YK_REQUIRE((reinterpret_cast<uintptr_t>(x) % 16 == 0) && (reinterpret_cast<uintptr_t>(w) % 16 == 0),
+             "gemm_mfma_skinny_grouped: operands must be 16-byte aligned");
+  YK_REQUIRE(ldx >= K && ldw >= K && ldy >= N, "gemm_mfma_skinny_grouped: leading dimensions too small");
+  YK_REQUIRE(y_dtype == YK_F32 || y_dtype == YK_BF16, "gemm_mfma_skinny_grouped: unsupported output dtype");
+  YK_REQUIRE(g_force_waves == 0 || g_force_waves == 4, "gemm_mfma_skinny_grouped: workgroups have four waves");
+  YK_REQUIRE(g_wide != 2, "gemm_mfma_skinny_grouped: the wide form takes no groups");
+  if (M == 0) return 0;
+  return skinny_product(static_cast<const bf16_t*>(x), nullptr, static_cast<const bf16_t*>(w), y, y_dtype, workspace, workspace_floats,
+                        M, N, K, ldx, ldw, ldy, 0, 0, stream, group_rows, group_stride);
 }
 
 // Whether yk_gemm_mfma_skinny_from_attention takes a product of these sizes: up to 16 rows, and

@@ -22,16 +22,16 @@
 
 template <typename T, typename TW>
 __global__ void causal_conv_kernel(const T* __restrict__ x, int x_stride, const TW* __restrict__ w,
-                                   const TW* __restrict__ bias, const T* __restrict__ state,
+                                   const TW* __restrict__ bias, T* state,
                                    const int32_t* __restrict__ token_seq, const int32_t* __restrict__ seq_qstart,
                                    const int32_t* __restrict__ state_slots, T* __restrict__ out, int channels,
-                                   int taps, int act, size_t total) {
+                                   int taps, int act, int push, size_t total) {
   for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < total;
        i += static_cast<size_t>(gridDim.x) * blockDim.x) {
     const int n = static_cast<int>(i / channels), c = static_cast<int>(i % channels);
     const int seq = token_seq[n];
     const int t = n - seq_qstart[seq];  // the token's place in its span
-    const T* hist = state + static_cast<size_t>(state_slots[seq]) * (taps - 1) * channels;
+    T* hist = state + static_cast<size_t>(state_slots[seq]) * (taps - 1) * channels;
     float acc = bias != nullptr ? to_f32<TW>(bias[c]) : 0.f;
     for (int j = 0; j < taps; ++j) {
       const int back = taps - 1 - j;
@@ -43,26 +43,33 @@ __global__ void causal_conv_kernel(const T* __restrict__ x, int x_stride, const 
       acc = fmaf(to_f32<TW>(w[static_cast<size_t>(c) * taps + j]), v, acc);
     }
     out[i] = from_f32<T>(act == 1 ? act_silu(acc) : acc);
+    // (spans of one token: nobody else touches this request's inputs of this channel)
+    if (push) {
+      for (int j = 0; j + 2 < taps; ++j) hist[static_cast<size_t>(j) * channels + c] = hist[static_cast<size_t>(j + 1) * channels + c];
+      hist[static_cast<size_t>(taps - 2) * channels + c] = x[static_cast<size_t>(n) * x_stride + c];
+    }
   }
 }
 
-// act: 0 none, 1 silu on the convolution's output
+// act: 0 none, 1 silu on the convolution's output.  push != 0 (steps whose spans are single tokens only): the state takes
+// in the token's input in the same pass.
 extern "C" int yk_causal_conv(const void* x, int x_stride, int dtype, const void* w, const void* bias, int w_dtype,
-                              const void* state, const int32_t* token_seq, const int32_t* seq_qstart,
+                              void* state, const int32_t* token_seq, const int32_t* seq_qstart,
                               const int32_t* state_slots, void* out, int n_tokens, int channels, int taps, int act,
-                              hipStream_t stream) {
+                              int push, hipStream_t stream) {
   YK_REQUIRE(act == 0 || act == 1, "causal_conv: unknown activation");
   YK_REQUIRE(n_tokens >= 0 && channels > 0 && taps >= 1 && x_stride >= channels, "causal_conv: bad sizes");
   YK_REQUIRE(taps == 1 || state != nullptr, "causal_conv: a convolution of several taps needs its state");
+  YK_REQUIRE(!push || taps > 1, "causal_conv: a single tap keeps no inputs");
   if (n_tokens == 0) return 0;
   const size_t total = static_cast<size_t>(n_tokens) * channels;
   const int grid = static_cast<int>(std::min<size_t>((total + 255) / 256, 1 << 20));
 #define YK_CASE(D, T, WD, TW)                                                                                   \
   if (dtype == D && w_dtype == WD) {                                                                             \
     causal_conv_kernel<T, TW><<<grid, 256, 0, stream>>>(static_cast<const T*>(x), x_stride, static_cast<const TW*>(w), \
-                                                        static_cast<const TW*>(bias), static_cast<const T*>(state),     \
+                                                        static_cast<const TW*>(bias), static_cast<T*>(state),           \
                                                         token_seq, seq_qstart, state_slots, static_cast<T*>(out),       \
-                                                        channels, taps, act, total);                                    \
+                                                        channels, taps, act, push, total);                              \
     return yk_check_launch("causal_conv");                                                                       \
   }
   YK_CASE(YK_F32, float, YK_F32, float)

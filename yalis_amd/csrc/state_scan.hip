@@ -6,6 +6,8 @@
 //   u  = dt_t v_t                          a write as strong as the token's step (state-space duality: with the head's
 //                                          decay exp(-exp(A_log) dt_t), dt_t = softplus(x + dt_bias), q = C, k = B)
 //   S <- S + k_t u^T,   o_t = S^T q_t      (the read-out sees the token's own write; + skip_h v_t where a skip is given)
+// or, with a bonus b per head and key channel, the read-out of the memory as it was before the token:
+//   o_t = (S + diag(b) k_t v_t^T)^T q_t,   S <- diag(a_t) S + k_t v_t^T
 //
 // The columns of S never meet: column e needs k_t, q_t, a_t, beta_t and its own v_t[e] only.  So a
 // column lives in the registers of a group of TPC lanes (lane s of the group holds the rows s,
@@ -14,13 +16,14 @@
 // per token and vector makes the unit norm while it stages), read back 16 bytes at a time.  Decays, write strengths and unit norms are made here, in float32, from the
 // projections' raw outputs:
 //   decay per head:     exp(-exp(A_log[h]) * softplus(x[n, h] + dt_bias[h]))
-//   decay per channel:  sigmoid(z[n, h, i] + bias[h, i]) ^ (1 / tau)  =  exp(logsigmoid(.) / tau)
+//   decay per channel:  sigmoid(z[n, h, i] + bias[h, i]) ^ (1 / tau)  =  exp(logsigmoid(.) / tau), or
+//                       exp(-exp(A_log[h]) * softplus(z[n, h, i] + dt_bias[h, i])), or exp(-exp(z[n, h, i] + bias[h, i]))
 //   beta:               sigmoid(x[n, h])
 //   unit vectors:       q / sqrt(sum q^2 + eps), k likewise (with unit_eps >= 0), then q * q_scale
 // A span cut anywhere gives the same S bit for bit: every token's step is made alone.
 //
 // Beside it: the read-out's norm and gate (each head's o divided by its root mean square, times a
-// weight shared by the heads, times silu of a gate column), and the shift of a convolution's kept
+// weight shared by the heads, times silu or the sigmoid of a gate column), and the shift of a convolution's kept
 // inputs by a span.
 #include <algorithm>
 
@@ -30,6 +33,13 @@ constexpr int kScanRowsMax = 16;  // rows of S a lane holds at the most (templat
 constexpr int kScanTokens = 32;  // tokens staged at a time (fewer where LDS would not hold them)
 
 __device__ __forceinline__ float scan_softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
+
+// a decay per key channel from its biased logit x: kinds 1, 2 and 3 of yk_linear_state_scan
+__device__ __forceinline__ float channel_decay(float x, int mode, float tau, float rate) {
+  if (mode == 1) return expf(-scan_softplus(-x) / tau);
+  if (mode == 2) return expf(-rate * scan_softplus(x));
+  return expf(-expf(x));
+}
 
 // the sum over the TPC lanes of a column (lanes that differ in their low bits), in all of them.  Inside
 // a row of 16 lanes the exchanges are register moves (quad permutations, then rotations of the row by 4
@@ -98,7 +108,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
     float q_scale, float unit_eps, int decay_mode, const float* __restrict__ decay, int decay_stride, int decay_col,
     const float* __restrict__ decay_p0, const float* __restrict__ decay_p1, float tau, const float* __restrict__ beta,
     int beta_stride, int beta_col, int chunk, float* __restrict__ out, int q_col, int k_col, int v_col, int write_mode,
-    const float* __restrict__ skip) {
+    const float* __restrict__ skip, const T* __restrict__ beta_rows, const float* __restrict__ bonus) {
   extern __shared__ float lds[];
   constexpr int DP = TPC * kScanRows;  // padded key channels
   constexpr int DS = DP + 4;           // a staged row's stride: rows of different tokens then start in different banks
@@ -106,9 +116,11 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
   float* ks = lds;                                        // [chunk][DS]
   float* qs = ks + chunk * DS;                            // [chunk][DS]
   float* as = qs + chunk * DS;                            // [chunk][DS] (per channel) or [chunk]
-  float* vs = as + chunk * (decay_mode == 1 ? DS : 1);    // [chunk][cols_per_block]
+  const bool per_channel = decay_mode != 0;
+  float* vs = as + chunk * (per_channel ? DS : 1);        // [chunk][cols_per_block]
   float* bs = vs + chunk * cols_per_block;                // [chunk]
-  float* kqs = bs + chunk;                                // [chunk]: k . q of every token, as they enter the recurrence
+  float* kqs = bs + chunk;                                // [chunk]: k . q (times the bonus) of every token, as they enter the recurrence
+  float* us = kqs + chunk;                                // [DS]: the head's bonus, where there is one
 
   const int seq = blockIdx.x, h = blockIdx.y, kvh = h / (n_heads / n_kv);
   const int col0 = blockIdx.z * cols_per_block;
@@ -119,6 +131,12 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
   float* S_head = state + (static_cast<size_t>(state_slots[seq]) * n_heads + h) * dim * vdim;
   const bool delta = write_mode == 1;
   const float skip_h = skip != nullptr ? skip[h] : 0.f;
+  const bool read_first = bonus != nullptr;  // the read-out sees the memory as it was
+  if (read_first)
+    for (int i = threadIdx.x; i < DP; i += blockDim.x) us[i] = i < dim ? bonus[h * dim + i] : 0.f;
+  // per channel: the vector that joins the logits, and (kind 2) what the softplus is multiplied with
+  const float* dec_bias = decay_mode == 2 ? decay_p1 : decay_p0;
+  const float dec_rate = decay_mode == 2 ? expf(decay_p0[h]) : 1.f;
 
   float S[kScanRows];
 #pragma unroll
@@ -150,7 +168,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         }
       }
       constexpr int P4 = DP / 4;
-      const int n_dec = decay_mode == 1 ? nt * P4 : 0;
+      const int n_dec = per_channel ? nt * P4 : 0;
       float4 dz[8], db[8];
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
@@ -159,7 +177,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         dz[j] = db[j] = make_float4(0.f, 0.f, 0.f, 0.f);
         if (v < n_dec && c < dim) {
           dz[j] = *reinterpret_cast<const float4*>(decay + static_cast<size_t>(q0 + t0 + t) * decay_stride + decay_col + h * dim + c);
-          db[j] = *reinterpret_cast<const float4*>(decay_p0 + h * dim + c);
+          db[j] = *reinterpret_cast<const float4*>(dec_bias + h * dim + c);
         }
       }
       const int n_v = nt * cols_per_block;
@@ -183,7 +201,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       if (threadIdx.x < nt) {
         const size_t n = static_cast<size_t>(q0 + t0 + threadIdx.x);
         if (decay_mode == 0) s_dec = decay[n * decay_stride + decay_col + h];
-        if (delta) s_beta = beta[n * beta_stride + beta_col + h];
+        if (delta) s_beta = beta_rows != nullptr ? to_f32<T>(beta_rows[n * beta_stride + beta_col + h]) : beta[n * beta_stride + beta_col + h];
       }
       // ---- everything is on its way; now the stores
 #pragma unroll
@@ -202,11 +220,11 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         const int v = threadIdx.x + j * 256;
         if (v < n_dec) {
           const int c = 4 * (v % P4);
-          // sigmoid(z)^(1/tau); channels past dim decay to nothing (their rows of S are zeros anyway)
+          // (channels past dim decay to nothing: their rows of S are zeros anyway)
           float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
           if (c < dim)
-            a = make_float4(expf(-scan_softplus(-(dz[j].x + db[j].x)) / tau), expf(-scan_softplus(-(dz[j].y + db[j].y)) / tau),
-                            expf(-scan_softplus(-(dz[j].z + db[j].z)) / tau), expf(-scan_softplus(-(dz[j].w + db[j].w)) / tau));
+            a = make_float4(channel_decay(dz[j].x + db[j].x, decay_mode, tau, dec_rate), channel_decay(dz[j].y + db[j].y, decay_mode, tau, dec_rate),
+                            channel_decay(dz[j].z + db[j].z, decay_mode, tau, dec_rate), channel_decay(dz[j].w + db[j].w, decay_mode, tau, dec_rate));
           *reinterpret_cast<float4*>(as + (v / P4) * DS + c) = a;
         }
       }
@@ -249,7 +267,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         }
       }
     }
-    if (decay_mode == 1) {
+    if (per_channel) {
       const int total = nt * DP;
       for (int i0 = threadIdx.x; i0 < total; i0 += 8 * blockDim.x) {
         float z[8];
@@ -258,14 +276,14 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
           const int i = i0 + j * blockDim.x;
           const int t = i / DP, c = i % DP;
           z[j] = i < total && c < dim
-                     ? decay[static_cast<size_t>(q0 + t0 + t) * decay_stride + decay_col + h * dim + c] + decay_p0[h * dim + c]
-                     : INFINITY;
+                     ? decay[static_cast<size_t>(q0 + t0 + t) * decay_stride + decay_col + h * dim + c] + dec_bias[h * dim + c]
+                     : 0.f;
         }
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
           const int i = i0 + j * blockDim.x;
-          // sigmoid(z)^(1/tau); channels past dim decay to nothing (their rows of S are zeros anyway)
-          if (i < total) as[(i / DP) * DS + i % DP] = i % DP < dim ? expf(-scan_softplus(-z[j]) / tau) : 0.f;
+          // (channels past dim decay to nothing: their rows of S are zeros anyway)
+          if (i < total) as[(i / DP) * DS + i % DP] = i % DP < dim ? channel_decay(z[j], decay_mode, tau, dec_rate) : 0.f;
         }
       }
     }
@@ -277,7 +295,9 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       const size_t n = static_cast<size_t>(q0 + t0 + t);
       const float step = decay_mode == 0 ? scan_softplus(decay[n * decay_stride + decay_col + h] + decay_p1[h]) : 1.f;
       if (decay_mode == 0) as[t] = expf(-expf(decay_p0[h]) * step);
-      bs[t] = delta ? 1.f / (1.f + expf(-beta[n * beta_stride + beta_col + h])) : (write_mode == 2 ? step : 1.f);
+      float b = write_mode == 2 ? step : 1.f;
+      if (delta) b = 1.f / (1.f + expf(-(beta_rows != nullptr ? to_f32<T>(beta_rows[n * beta_stride + beta_col + h]) : beta[n * beta_stride + beta_col + h])));
+      bs[t] = b;
     }
     }
     __syncthreads();
@@ -292,7 +312,12 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         const float4 a = *reinterpret_cast<const float4*>(qrow + c), b = *reinterpret_cast<const float4*>(krow + c);
         ssq = fmaf(a.x, a.x, fmaf(a.y, a.y, fmaf(a.z, a.z, fmaf(a.w, a.w, ssq))));
         ssk = fmaf(b.x, b.x, fmaf(b.y, b.y, fmaf(b.z, b.z, fmaf(b.w, b.w, ssk))));
-        dot = fmaf(a.x, b.x, fmaf(a.y, b.y, fmaf(a.z, b.z, fmaf(a.w, b.w, dot))));
+        if (read_first) {
+          const float4 u = *reinterpret_cast<const float4*>(us + c);
+          dot = fmaf(a.x * u.x, b.x, fmaf(a.y * u.y, b.y, fmaf(a.z * u.z, b.z, fmaf(a.w * u.w, b.w, dot))));
+        } else {
+          dot = fmaf(a.x, b.x, fmaf(a.y, b.y, fmaf(a.z, b.z, fmaf(a.w, b.w, dot))));
+        }
       }
       dot = column_sum<8>(dot);
       if (unit_eps >= 0.f) {
@@ -315,7 +340,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
     float kn[kScanRows], qn[kScanRows], an[kScanRows];
     float a_n = 1.f, v_n = 0.f, b_n = 1.f, kq_n = 0.f;
     auto fetch = [&](int t) {
-      if (decay_mode != 1) a_n = as[t];
+      if (!per_channel) a_n = as[t];
       v_n = vs[t * cols_per_block + col_local];
       b_n = bs[t];
       kq_n = kqs[t];
@@ -327,7 +352,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         kn[4 * r4] = k4.x; kn[4 * r4 + 1] = k4.y; kn[4 * r4 + 2] = k4.z; kn[4 * r4 + 3] = k4.w;
         qn[4 * r4] = q4.x; qn[4 * r4 + 1] = q4.y; qn[4 * r4 + 2] = q4.z; qn[4 * r4 + 3] = q4.w;
       }
-      if (decay_mode == 1) {
+      if (per_channel) {
         const float4* at = reinterpret_cast<const float4*>(as + t * DS + sub * kScanRows);
 #pragma unroll
         for (int r4 = 0; r4 < kScanRows / 4; ++r4) {
@@ -345,7 +370,12 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
         kr[r] = kn[r];
         qr[r] = qn[r];
       }
-      if (decay_mode == 1) {
+      float pk[4] = {0.f, 0.f, 0.f, 0.f}, pq[4] = {0.f, 0.f, 0.f, 0.f};
+      if (read_first) {
+#pragma unroll
+        for (int r = 0; r < kScanRows; ++r) pq[r % 4] = fmaf(S[r], qr[r], pq[r % 4]);
+      }
+      if (per_channel) {
 #pragma unroll
         for (int r = 0; r < kScanRows; ++r) S[r] *= an[r];
       } else {
@@ -357,11 +387,12 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       if (t + 1 < nt) fetch(t + 1);
       // both sums over the decayed S at once: S^T k for the write, S^T q for the read-out, which sees the
       // token's own write through q . (k u^T) = u (k . q)
-      float pk[4] = {0.f, 0.f, 0.f, 0.f}, pq[4] = {0.f, 0.f, 0.f, 0.f};
+      if (!read_first) {
 #pragma unroll
-      for (int r = 0; r < kScanRows; ++r) {
-        pk[r % 4] = fmaf(S[r], kr[r], pk[r % 4]);
-        pq[r % 4] = fmaf(S[r], qr[r], pq[r % 4]);
+        for (int r = 0; r < kScanRows; ++r) {
+          pk[r % 4] = fmaf(S[r], kr[r], pk[r % 4]);
+          pq[r % 4] = fmaf(S[r], qr[r], pq[r % 4]);
+        }
       }
       const float sq = column_sum<TPC>((pq[0] + pq[1]) + (pq[2] + pq[3]));
       float u = v_t;
@@ -381,7 +412,11 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
 }
 
 // decay_mode 0: one decay per head from decay[n, decay_col + h], p0 = A_log [heads], p1 = dt_bias [heads];
-// decay_mode 1: one per key channel from decay[n, decay_col + h * dim + i], p0 = bias [heads * dim], tau.
+// decay_mode 1, 2, 3: one per key channel from z = decay[n, decay_col + h * dim + i]: 1, sigmoid(z + p0)^(1 / tau), p0 =
+// bias [heads * dim]; 2, exp(-exp(p0[h]) softplus(z + p1)), p0 = A_log [heads], p1 = dt_bias [heads * dim]; 3,
+// exp(-exp(z + p0)), p0 = bias [heads * dim].
+// beta (float32) or, in its place, beta_rows (of qkv's dtype), both read at [n, beta_col + h].  bonus [heads * dim]
+// float32 or null: the read-out comes before the write, with the token's own write weighed by the bonus (plain writes).
 // write_mode 0: plain writes; 1: the delta rule with beta = sigmoid(beta[n, beta_col + h]); 2: u = dt v with the
 // step dt = softplus(decay[n, decay_col + h] + p1[h]) that the head's decay is made of (decay_mode 0 only).
 // unit_eps < 0: q and k are taken as they are.  q_col, k_col, v_col: where the kv_heads' queries and keys and the
@@ -392,15 +427,16 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
                                     const float* decay, int decay_stride, int decay_col, const float* decay_p0,
                                     const float* decay_p1, float tau, const float* beta, int beta_stride, int beta_col,
                                     float* out, int q_col, int k_col, int v_col, int write_mode, const float* skip,
-                                    hipStream_t stream) {
+                                    const void* beta_rows, const float* bonus, hipStream_t stream) {
   YK_REQUIRE(n_seqs >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0 && dim > 0 && vdim > 0, "linear_state_scan: bad sizes");
   YK_REQUIRE(q_col >= 0 && k_col >= 0 && v_col >= 0 && qkv_stride >= std::max(std::max(q_col, k_col) + n_kv * dim, v_col + n_heads * vdim),
              "linear_state_scan: rows shorter than q, k and v");
-  YK_REQUIRE(write_mode == 0 || (write_mode == 1 && beta != nullptr) || (write_mode == 2 && decay_mode == 0),
+  YK_REQUIRE(write_mode == 0 || (write_mode == 1 && (beta != nullptr || beta_rows != nullptr)) || (write_mode == 2 && decay_mode == 0),
              "linear_state_scan: the delta rule needs beta, a write by the step the decay per head");
-  YK_REQUIRE(decay_mode == 0 || decay_mode == 1, "linear_state_scan: unknown kind of decay");
-  YK_REQUIRE(decay != nullptr && decay_p0 != nullptr && (decay_mode == 1 || decay_p1 != nullptr), "linear_state_scan: the decay's inputs are missing");
-  YK_REQUIRE(decay_mode == 0 || tau > 0.f, "linear_state_scan: tau must be positive");
+  YK_REQUIRE(decay_mode >= 0 && decay_mode <= 3, "linear_state_scan: unknown kind of decay");
+  YK_REQUIRE(bonus == nullptr || (write_mode == 0 && skip == nullptr), "linear_state_scan: a bonus goes with plain writes and no skip");
+  YK_REQUIRE(decay != nullptr && decay_p0 != nullptr && (decay_mode == 1 || decay_mode == 3 || decay_p1 != nullptr), "linear_state_scan: the decay's inputs are missing");
+  YK_REQUIRE(decay_mode != 1 || tau > 0.f, "linear_state_scan: tau must be positive");
   YK_REQUIRE(dim <= kScanRowsMax * kWave, "linear_state_scan: heads of more than 1,024 key channels are not offered");
   if (n_seqs == 0) return 0;
   // eight rows a lane while that leaves a column inside a wave (a wave's instructions per token are what
@@ -416,13 +452,13 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
   dim3 grid(n_seqs, n_heads, (vdim + cols - 1) / cols);
   const size_t dp = static_cast<size_t>(tpc) * rows;
   int chunk = kScanTokens;
-  const size_t per_token = sizeof(float) * (2 * (dp + 4) + (decay_mode == 1 ? dp + 4 : 1) + cols + 2);
+  const size_t per_token = sizeof(float) * (2 * (dp + 4) + (decay_mode != 0 ? dp + 4 : 1) + cols + 2);
   while (chunk > 4 && (chunk * per_token > 110 * 1024 || chunk * dp > 8192)) chunk /= 2;
-  const size_t lds = chunk * per_token;
+  const size_t lds = chunk * per_token + (bonus != nullptr ? (dp + 4) * sizeof(float) : 0);
   YK_REQUIRE(lds <= 128 * 1024, "linear_state_scan: the staged tokens do not fit in LDS");
   auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
   const bool vec = dim % 8 == 0 && qkv_stride % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 && al16(qkv) && chunk * dp <= 8192 &&
-                   (decay_mode == 0 || (decay_stride % 4 == 0 && decay_col % 4 == 0 && al16(decay) && al16(decay_p0)));
+                   (decay_mode == 0 || (decay_stride % 4 == 0 && decay_col % 4 == 0 && al16(decay) && al16(decay_mode == 2 ? decay_p1 : decay_p0)));
 #define YK_LAUNCH(T, TPC)                                                                                                       \
   {                                                                                                                             \
     auto kern = rows == 8 ? (vec ? linear_state_scan_kernel<T, TPC, 8, true> : linear_state_scan_kernel<T, TPC, 8, false>)      \
@@ -433,7 +469,7 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
     kern<<<grid, threads, lds, stream>>>(static_cast<const T*>(qkv), qkv_stride, n_heads, n_kv, dim, vdim, state, seq_qstart,   \
                                          seq_qlen, state_slots, q_scale, unit_eps, decay_mode, decay, decay_stride, decay_col,  \
                                          decay_p0, decay_p1, tau, beta, beta_stride, beta_col, chunk, out, q_col, k_col,       \
-                                         v_col, write_mode, skip);                                                              \
+                                         v_col, write_mode, skip, static_cast<const T*>(beta_rows), bonus);                     \
     return yk_check_launch("linear_state_scan");                                                                                \
   }
 #define YK_TPC(T)                   \
@@ -455,13 +491,14 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
 
 // --------------------------------------------------------------- the read-out's norm and gate
 // a wave per (token, part of vdim elements): y = o / sqrt(mean(o^2) + eps) * w * silu(gate), or, gate_first, the gate
-// before the norm: y = g / sqrt(mean(g^2) + eps) * w with g = o * silu(gate).  w_stride 0: one weight of vdim elements
+// before the norm: y = g / sqrt(mean(g^2) + eps) * w with g = o * silu(gate).  gate_act 1: the sigmoid in silu's place.  w_stride 0: one weight of vdim elements
 // for every part; vdim: a weight of n_heads * vdim elements.
+__device__ __forceinline__ float head_gate_act(float g, int act) { return act == 1 ? 1.f / (1.f + expf(-g)) : act_silu(g); }
 template <typename TW, typename TG, typename TO>
 __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __restrict__ o, const TW* __restrict__ w, float eps,
                                                               const TG* __restrict__ gate, int gate_stride, int gate_col,
                                                               int n_heads, int vdim, TO* __restrict__ out, size_t total,
-                                                              int w_stride, int gate_first) {
+                                                              int w_stride, int gate_first, int gate_act) {
   const size_t item = blockIdx.x * static_cast<size_t>(blockDim.x / kWave) + threadIdx.x / kWave;
   if (item >= total) return;
   const int lane = threadIdx.x % kWave;
@@ -473,40 +510,43 @@ __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __res
   float ss = 0.f;
   if (gate_first) {
     for (int c = lane; c < vdim; c += kWave) {
-      const float v = row[c] * act_silu(to_f32<TG>(g[c]));
+      const float v = row[c] * head_gate_act(to_f32<TG>(g[c]), gate_act);
       ss = fmaf(v, v, ss);
     }
     const float inv = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(vdim) + eps);
     for (int c = lane; c < vdim; c += kWave)
-      out[item * vdim + c] = from_f32<TO>(row[c] * act_silu(to_f32<TG>(g[c])) * inv * to_f32<TW>(wp[c]));
+      out[item * vdim + c] = from_f32<TO>(row[c] * head_gate_act(to_f32<TG>(g[c]), gate_act) * inv * to_f32<TW>(wp[c]));
     return;
   }
   for (int c = lane; c < vdim; c += kWave) ss = fmaf(row[c], row[c], ss);
   const float inv = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(vdim) + eps);
   for (int c = lane; c < vdim; c += kWave)
-    out[item * vdim + c] = from_f32<TO>(row[c] * inv * to_f32<TW>(wp[c]) * act_silu(to_f32<TG>(g[c])));
+    out[item * vdim + c] = from_f32<TO>(row[c] * inv * to_f32<TW>(wp[c]) * head_gate_act(to_f32<TG>(g[c]), gate_act));
 }
 
 extern "C" int yk_gated_head_norm(const float* o, const void* w, int w_dtype, float eps, const void* gate, int gate_dtype,
                                   int gate_stride, int gate_col, int n_heads, int vdim, void* out, int out_dtype, int n_tokens,
-                                  int w_per_part, int gate_first, hipStream_t stream) {
+                                  int w_per_part, int gate_first, int gate_act, hipStream_t stream) {
   YK_REQUIRE(n_tokens >= 0 && n_heads > 0 && vdim > 0 && gate_stride >= gate_col + n_heads * vdim, "gated_head_norm: bad sizes");
-  YK_REQUIRE(gate_dtype == out_dtype, "gated_head_norm: the gate comes in the output's dtype");
+  YK_REQUIRE(gate_dtype == out_dtype || gate_dtype == YK_F32, "gated_head_norm: the gate comes in the output's dtype or float32");
+  YK_REQUIRE(gate_act == 0 || gate_act == 1, "gated_head_norm: the gate is silu or the sigmoid");
   if (n_tokens == 0) return 0;
   const size_t total = static_cast<size_t>(n_tokens) * n_heads;
   const int grid = static_cast<int>((total + 3) / 4);
   const int w_stride = w_per_part ? vdim : 0;
-#define YK_CASE(WD, TW, OD, TO)                                                                                       \
-  if (w_dtype == WD && out_dtype == OD) {                                                                             \
-    gated_head_norm_kernel<TW, TO, TO><<<grid, 256, 0, stream>>>(o, static_cast<const TW*>(w), eps,                   \
-                                                                 static_cast<const TO*>(gate), gate_stride, gate_col, \
+#define YK_CASE(WD, TW, GD, TG, OD, TO)                                                                               \
+  if (w_dtype == WD && gate_dtype == GD && out_dtype == OD) {                                                         \
+    gated_head_norm_kernel<TW, TG, TO><<<grid, 256, 0, stream>>>(o, static_cast<const TW*>(w), eps,                   \
+                                                                 static_cast<const TG*>(gate), gate_stride, gate_col, \
                                                                  n_heads, vdim, static_cast<TO*>(out), total, w_stride, \
-                                                                 gate_first);                                         \
+                                                                 gate_first, gate_act);                               \
     return yk_check_launch("gated_head_norm");                                                                        \
   }
-  YK_CASE(YK_F32, float, YK_F32, float)
-  YK_CASE(YK_BF16, bf16_t, YK_BF16, bf16_t)
-  YK_CASE(YK_F32, float, YK_BF16, bf16_t)
+  YK_CASE(YK_F32, float, YK_F32, float, YK_F32, float)
+  YK_CASE(YK_BF16, bf16_t, YK_BF16, bf16_t, YK_BF16, bf16_t)
+  YK_CASE(YK_F32, float, YK_BF16, bf16_t, YK_BF16, bf16_t)
+  YK_CASE(YK_BF16, bf16_t, YK_F32, float, YK_BF16, bf16_t)
+  YK_CASE(YK_F32, float, YK_F32, float, YK_BF16, bf16_t)
 #undef YK_CASE
   return yk_fail("gated_head_norm: unsupported dtype combination");
 }

@@ -130,6 +130,14 @@ class DecoderModel:
             sidx = tuple(range(len(states), len(states) + len(sneed)))
             states.extend(sneed)
             sites.append(SiteInfo(i, e.layer, group, index, owns, sidx))
+        # an embedding that remembers something per request has a site of its own, after the run entries'
+        self.embedding_site: Optional[int] = None
+        if getattr(self.embedding, "keeps_state", False):
+            sneed = self.embedding.state_need()
+            sneed = (sneed,) if isinstance(sneed, StateNeed) else tuple(sneed)
+            self.embedding_site = len(sites)
+            sites.append(SiteInfo(len(sites), -1, None, None, False, tuple(range(len(states), len(states) + len(sneed)))))
+            states.extend(sneed)
         cache_groups = [CacheGroup(n, tuple(m)) for n, m in groups]
         return cache_groups, states, sites
 
@@ -179,7 +187,9 @@ class DecoderModel:
         """Run the step's tokens; returns float32 logits [wanted rows, vocab]."""
         first = self.blocks[self.spec.run_order[0].layer]
         begin = getattr(self.embedding, "begin", None)
-        if getattr(self.embedding, "needs_positions", False):
+        if self.embedding_site is not None:
+            residual, delta = self.embedding.begin(ctx, ctx.site(self.embedding_site))
+        elif getattr(self.embedding, "needs_positions", False):
             residual, delta = self.embedding.forward(ctx.arrays["token_ids"], ctx.arrays["positions"]), None
         elif begin is not None:
             lazily = bool(getattr(first, "takes_embedded_rows", False)) and self.spec.run_order[0].added_row is None

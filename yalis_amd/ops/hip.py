@@ -21,6 +21,7 @@ _F32, _BF16 = 0, 1
 _c_int = ctypes.c_int
 _c_float = ctypes.c_float
 _c_size_t = ctypes.c_size_t
+_c_u64 = ctypes.c_ulonglong
 _vp = ctypes.c_void_p
 
 
@@ -64,6 +65,22 @@ _SIGNATURES = {
         [_vp, _vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_float, _vp, _c_int, _c_int, _c_float, _vp, _c_int, _c_int, _c_int, _vp],
         _c_int,
     ),
+    "yk_sum_norm": (
+        [_vp, _vp, _c_int, _c_int, _c_int, _c_float, _vp, _vp, _c_int, _c_int, _c_int, _c_float, _vp, _c_float, _vp, _c_float, _vp, _c_int,
+         _c_int, _c_float, _vp, _c_int, _c_int, _vp],
+        _c_int,
+    ),
+    "yk_embed_pairs": (
+        [_vp, _vp, _c_int, _c_int, _c_float, _vp, _c_int, _c_u64, _c_u64, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp],
+        _c_int,
+    ),
+    "yk_token_shift_mix": ([_vp, _c_int, _vp, _c_int, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp], _c_int),
+    "yk_low_rank": ([_vp, _c_int, _c_int, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _vp], _c_int),
+    "yk_act_rows": ([_vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _vp], _c_int),
+    "yk_gemm_mfma_skinny_grouped": (
+        [_vp, _c_size_t, _c_int, _vp, _vp, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp],
+        _c_int,
+    ),
     "yk_round_rows": ([_vp, _vp, _c_int, _c_size_t, _vp], _c_int),
     "yk_qkv_prepare": (
         [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _c_int,
@@ -78,7 +95,7 @@ _SIGNATURES = {
     "yk_attn_masked": (
         [_vp, _c_int, _vp, _vp, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
          _c_float, _c_int, _c_int, _c_int, _vp, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp,
-         _c_int, _vp, _vp],
+         _c_int, _vp, _c_int, _vp],
         _c_int,
     ),
     "yk_attn_finish": (
@@ -86,7 +103,7 @@ _SIGNATURES = {
          _vp],
         _c_int,
     ),
-    "yk_causal_conv": ([_vp, _c_int, _c_int, _vp, _vp, _c_int, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _vp], _c_int),
+    "yk_causal_conv": ([_vp, _c_int, _c_int, _vp, _vp, _c_int, _vp, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp], _c_int),
     "yk_sandwich_norm": (
         [_vp, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _c_float, _c_int, _c_float, _vp, _vp, _c_float, _c_int, _c_int, _vp, _vp,
          _c_int, _c_int, _c_int, _vp],
@@ -121,11 +138,11 @@ _SIGNATURES = {
     "yk_latent_attention": ([_vp, _vp, _c_int, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _vp, _vp, _vp], _c_int),
     "yk_linear_state_scan": (
         [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_float, _c_float, _c_int, _vp, _c_int,
-         _c_int, _vp, _vp, _c_float, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp],
+         _c_int, _vp, _vp, _c_float, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp],
         _c_int,
     ),
     "yk_gated_head_norm": (
-        [_vp, _vp, _c_int, _c_float, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp],
+        [_vp, _vp, _c_int, _c_float, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp],
         _c_int,
     ),
     "yk_conv_state_push": ([_vp, _c_int, _c_int, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_int, _vp], _c_int),
@@ -180,11 +197,11 @@ _SIGNATURES = {
     "yk_attn_tokens_per_tile": ([_c_int, _c_int], _c_int),
     "yk_attn_mfma_workspace": ([_c_int, _c_int, _c_int, _c_int, _c_int], _c_size_t),
     "yk_attn_mfma_prefill": (
-        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _vp],
+        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _c_int, _vp],
         _c_int,
     ),
     "yk_attn_mfma": (
-        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _vp],
+        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _c_int, _vp],
         _c_int,
     ),
     "yk_attn_mfma_rope": (
@@ -213,7 +230,7 @@ _LATER_SIGNATURES = {
         "yk_probe_mfma_bf16": ([_c_int, _c_int, _vp, _vp], _c_int),
     },
 }
-_ABI = 21
+_ABI = 22
 
 # Rows of x up to which the hand-written matrix-core kernel runs a bfloat16 product;
 # above it the vendor library does.
@@ -506,6 +523,25 @@ class HipOps:
             )
         )
         return out
+
+    def embed_pairs(self, token_ids, table, scale, pair_table, buckets, mul_prev, mul_cur, state, ctx, act_dtype):
+        """(float32 rows table[id] * scale + pair_table[(before * mul_prev + id * mul_cur) mod buckets], the same rounded to
+        ``act_dtype``).  The token before a span's first one is ``state`` [slots, 1] (int32, negative: none, which takes
+        the pair table's row ``buckets``); it is left at the span's last token."""
+        n, width = token_ids.numel(), table.shape[1]
+        if table.dim() != 2 or not table.is_contiguous() or not pair_table.is_contiguous() or tuple(pair_table.shape) != (buckets + 1, width) \
+                or pair_table.dtype != table.dtype:
+            raise KernelError(f"embed_pairs: the pairs' table {tuple(pair_table.shape)} does not match {buckets} buckets and a row for none, of {width}")
+        if state.dtype != torch.int32 or tuple(state.shape[1:]) != (1,) or token_ids.dtype != torch.int32:
+            raise KernelError("embed_pairs: a request's last token is one int32")
+        a = ctx.arrays
+        out = torch.empty((n, width), dtype=torch.float32, device=table.device)
+        rounded = None if act_dtype == torch.float32 else torch.empty((n, width), dtype=act_dtype, device=table.device)
+        self._check(self.lib.yk_embed_pairs(
+            token_ids.data_ptr(), table.data_ptr(), _code(table.dtype), table.shape[0], float(scale), pair_table.data_ptr(), int(buckets),
+            int(mul_prev), int(mul_cur), state.data_ptr(), a["token_seq"].data_ptr(), a["seq_qstart"].data_ptr(), a["seq_qlen"].data_ptr(),
+            a["state_slots"].data_ptr(), out.data_ptr(), _ptr(rounded), n, width, self._stream()))
+        return out, (out if rounded is None else rounded)
 
     def embedded_rows(self, token_ids: torch.Tensor, table: torch.Tensor):
         """(an uninitialised float32 residual [tokens, width], the ``EmbeddedRows`` that the
@@ -925,7 +961,7 @@ class HipOps:
     def attention(self, qkv, n_heads, n_kv, head_dim, k_cache, v_cache, page_size,
                   scale, window, ctx, group, tiles, long_tiles=None, plan=None, long_plan=None,
                   long_col_tiles: int = 1, token_cols=None, rope: Optional["RopeInLaunch"] = None,
-                  keep_first: int = 0, softcap: float = 0.0, distance_bias=None, sink=None):
+                  keep_first: int = 0, softcap: float = 0.0, distance_bias=None, sink=None, chunked: bool = False):
         """Queries are the first n_heads heads of each row of ``qkv`` (whatever follows
         them in the row is skipped); keys and values come from the cache through the
         block table of ``group``.  ``long_tiles`` hold up to
@@ -938,7 +974,8 @@ class HipOps:
         ``keep_first`` / ``softcap`` (matrix-core kernels only; other sizes are ``attention_masked``'s): with a
         window, the first ``keep_first`` keys of a request stay visible below it; scores times the scale
         are squashed to softcap * tanh(s / softcap); ``distance_bias`` (float32 [distances, n_heads]): row
-        min(p - j, distances - 1) is added to head h's scaled (and squashed) score of key j for the query at p.
+        min(p - j, distances - 1) is added to head h's scaled (and squashed) score of key j for the query at p;
+        ``chunked``: the window begins anew at every multiple of its size instead of sliding.
 
         ``rope`` (only where ``attention_can_rotate``, and only for steps whose spans are single
         tokens): ``qkv`` is then the projection's raw output (a tensor or a ``SplitSum``) and
@@ -962,8 +999,10 @@ class HipOps:
             and qkv.stride(0) % 8 == 0
             and qkv.data_ptr() % 16 == 0
         )
-        if (keep_first or softcap or distance_bias is not None or sink is not None) and not use_mfma:
-            raise KernelError("attention: kept first keys, squashed scores, biases per distance and sinks outside the matrix-core kernels' sizes are attention_masked's")
+        if (keep_first or softcap or distance_bias is not None or sink is not None or chunked) and not use_mfma:
+            raise KernelError("attention: kept first keys, chunks, squashed scores, biases per distance and sinks outside the matrix-core kernels' sizes are attention_masked's")
+        # keys any query of the step reads at most (a chunk's queries read no other chunk's)
+        reach = min(ctx.max_ctx, int(window)) if chunked else ctx.max_ctx
         if sink is not None and (sink.dtype != torch.float32 or sink.numel() != n_heads or not sink.is_contiguous()):
             raise KernelError("attention: the sinks are contiguous float32 [heads]")
         if distance_bias is not None and (distance_bias.dtype != torch.float32 or distance_bias.dim() != 2 or not distance_bias.is_contiguous()
@@ -974,7 +1013,7 @@ class HipOps:
             n_long = long_tiles.shape[0]
             hpt = self._ask("yk_attn_heads_per_tile", n_heads, n_kv)
             groups = n_long * n_kv * (-(-(n_heads // n_kv) // hpt))
-            long_splits = long_plan if long_plan is not None else self.attention_long_splits(groups, max(1, -(-ctx.max_ctx // 64)), int(long_col_tiles))
+            long_splits = long_plan if long_plan is not None else self.attention_long_splits(groups, max(1, -(-reach // 64)), int(long_col_tiles))
             ws_floats = self._ask("yk_attn_mfma_workspace", 4 * long_col_tiles * n_long, n_heads, n_kv, head_dim, long_splits)
             ws = self._ws(ws_floats) if ws_floats else None
             self._check(
@@ -983,7 +1022,7 @@ class HipOps:
                     long_tiles.data_ptr(), n_long, bt.data_ptr(), bt.shape[1], page_size, head_dim,
                     n_heads, n_kv, float(scale), int(window), long_splits, int(long_col_tiles), _ptr(ws),
                     0 if ws is None else ws.numel(), int(self.long_span_pages_in_lds), int(keep_first), float(softcap),
-                    _ptr(distance_bias), bias_rows, _ptr(sink), self._stream(),
+                    _ptr(distance_bias), bias_rows, _ptr(sink), int(bool(chunked)), self._stream(),
                 )
             )
         if use_mfma and tiles.shape[0] == 0:
@@ -992,7 +1031,7 @@ class HipOps:
             n_tiles = tiles.shape[0]
             hpt = self._ask("yk_attn_heads_per_tile", n_heads, n_kv)
             chunks = -(-(n_heads // n_kv) // hpt)
-            key_blocks = max(1, -(-ctx.max_ctx // 64))
+            key_blocks = max(1, -(-reach // 64))
             waves, splits = plan or self.attention_plan(n_tiles * n_kv * chunks, key_blocks)
             ws_floats = self._ask("yk_attn_mfma_workspace", n_tiles, n_heads, n_kv, head_dim, splits)
             ws = self._ws(ws_floats) if ws_floats else None
@@ -1003,7 +1042,7 @@ class HipOps:
                     qkv.data_ptr(), qkv.stride(0), out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                     tiles.data_ptr(), n_tiles, bt.data_ptr(), bt.shape[1], page_size, head_dim, n_heads, n_kv,
                     float(scale), int(window), waves, splits, _ptr(ws), 0 if ws is None else ws.numel(), int(leave),
-                    int(keep_first), float(softcap), _ptr(distance_bias), bias_rows, _ptr(sink), self._stream(),
+                    int(keep_first), float(softcap), _ptr(distance_bias), bias_rows, _ptr(sink), int(bool(chunked)), self._stream(),
                 )
             )
             if leave:
@@ -1166,6 +1205,39 @@ class HipOps:
         )
         return residual if out is None else out
 
+    def sum_norm(self, residual, terms, branch_scale, branch_weight, residual_scale, weight, eps, unit_offset, out_dtype):
+        """residual (float32 [N, width], in place) = norm(residual_scale * residual + branch_scale * (sum of the terms) *
+        branch_weight) * weight; returns it in ``out_dtype`` (itself for float32).  ``terms``: one or two of (rows, weight,
+        eps): a tensor or a ``SplitSum``, divided by its root mean square and multiplied by its weight, or, with weight
+        None, as it is.  ``branch_weight`` [width] or None."""
+        self._rows(residual, "residual")
+        if residual.dtype != torch.float32 or not residual.is_contiguous():
+            raise KernelError("the residual stream must be contiguous float32")
+        n, width = residual.shape
+        if not 1 <= len(terms) <= 2:
+            raise KernelError("sum_norm takes one or two terms")
+        args = []
+        for rows, w, e in terms:
+            n_splits, round_sum, src = 1, 0, rows
+            if isinstance(rows, SplitAttention):
+                rows = src = rows.merge()
+            if isinstance(rows, SplitSum):
+                rows.check_live()
+                n_splits, round_sum, src = rows.n_splits, rows.round_sum, rows.tensor
+            if tuple(rows.shape) != (n, width) or not src.is_contiguous():
+                raise KernelError(f"branch {tuple(rows.shape)} does not match the residual {(n, width)}")
+            args += [src.data_ptr(), _code(src.dtype), n_splits, round_sum, float(e), _ptr(w)]
+        if len(terms) == 1:
+            args += [None, 0, 1, 0, 0.0, None]
+        for w in [t[1] for t in terms] + [branch_weight, weight]:
+            if w is not None and (w.numel() != width or not w.is_contiguous() or w.dtype != weight.dtype):
+                raise KernelError("sum_norm: the weights are contiguous, as wide as the rows and of one dtype")
+        out = None if out_dtype == torch.float32 else torch.empty((n, width), dtype=out_dtype, device=residual.device)
+        self._check(self.lib.yk_sum_norm(
+            residual.data_ptr(), *args, float(branch_scale), _ptr(branch_weight), float(residual_scale), weight.data_ptr(), _code(weight.dtype),
+            int(bool(unit_offset)), float(eps), _ptr(out), n, width, self._stream()))
+        return residual if out is None else out
+
     # ------------------------------------- attention with prepared heads, kept first keys, a finish
     def masked_pages_tiled(self, dtype: torch.dtype, head_dim: int, value_dim: int, page_size: int) -> bool:
         return head_dim == value_dim and self.cache_tiled(dtype, head_dim, page_size)
@@ -1173,7 +1245,7 @@ class HipOps:
     def qkv_prepare(self, qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q_norm=None, k_norm=None,
                     qk_eps: float = 0.0, rotation=None, value_norm_eps=None, value_rotation=None,
                     k_cache=None, v_cache=None, slots=None, page_size: int = 0, bias=None, row_scales=None,
-                    norm_over_projection: bool = False, values_from_keys: bool = False) -> torch.Tensor:
+                    norm_over_projection: bool = False, values_from_keys: bool = False, unweighted_norm: bool = False) -> torch.Tensor:
         """From a projection's rows [q | k | v | ...] (a tensor or a ``SplitSum``): normed (weights
         ``q_norm`` / ``k_norm`` of head_dim elements, or none) and rotated queries [N, n_heads * head_dim];
         normed, rotated keys and unit-normed (``value_norm_eps``), rotated (``value_rotation``) values
@@ -1181,7 +1253,8 @@ class HipOps:
         is added first.  ``values_from_keys``: the rows are [q | k | ...] and a token's values are its keys as
         projected (biased, before the norm).  ``norm_over_projection``: the weights are as wide as the q (k)
         projection and no root mean square is taken here: it comes with ``row_scales`` (float32 [N, 2], from
-        ``qk_row_scales``), which multiply a token's queries (column 0) and keys (column 1) after the weights."""
+        ``qk_row_scales``), which multiply a token's queries (column 0) and keys (column 1) after the weights.
+        ``unweighted_norm``: every head is divided by its root mean square (``qk_eps`` under the root) and that is all."""
         n_splits, round_sum, src = 1, 0, qkv
         if isinstance(qkv, SplitSum):
             qkv.check_live()
@@ -1222,6 +1295,10 @@ class HipOps:
         qk_norm = int(q_norm is not None or k_norm is not None) * (2 if norm_over_projection else 1)
         if qk_norm and (q_norm is None or k_norm is None):
             raise KernelError("queries and keys are normed together or not at all")
+        if unweighted_norm:
+            if qk_norm:
+                raise KernelError("qkv_prepare: a norm without weights takes none")
+            qk_norm = 1
         for r in (rotation, value_rotation):
             if r is not None and (r.cos.dtype != torch.float32 or r.cos.shape != r.sin.shape or r.cos.shape[1] != r.rotary_dim // 2):
                 raise KernelError("rotary tables must be float32 [positions, rotary_dim/2]")
@@ -1284,7 +1361,8 @@ class HipOps:
 
     def attention_masked(self, q, n_heads, n_kv, head_dim, value_dim, k_cache, v_cache, page_size, scale, ctx, group,
                          window: int = 0, keep_first: int = 0, softcap: float = 0.0, value_rotation=None,
-                         gate=None, gate_col: int = 0, gate_elems: int = 1, distance_bias=None, sink=None) -> torch.Tensor:
+                         gate=None, gate_col: int = 0, gate_elems: int = 1, distance_bias=None, sink=None,
+                         chunked: bool = False) -> torch.Tensor:
         """softmax over the keys j <= p with (p - j < window or j < keep_first) of q . k * scale
         (squashed by ``softcap`` * tanh(s / ``softcap``) when set), times the values [N, n_heads *
         value_dim]; then, with ``value_rotation``, every head's output turned back by its token's
@@ -1292,7 +1370,8 @@ class HipOps:
         ``gate_col`` + h hold the heads' gates), multiplied by the sigmoid of its gate (``gate_elems`` = value_dim:
         a gate per output element, in the columns ``gate_col`` + h * value_dim + d).  ``distance_bias`` (float32
         [distances, n_heads]): row min(p - j, distances - 1) is added to the scaled scores of head h.  ``sink`` (float32
-        [n_heads]): exp(sink[h]) joins head h's denominator once; it has no key and no value."""
+        [n_heads]): exp(sink[h]) joins head h's denominator once; it has no key and no value.  ``chunked``: the window
+        begins anew at every multiple of its size (keys j with floor(j / window) = floor(p / window))."""
         self._rows(q, "queries")
         if sink is not None and (sink.dtype != torch.float32 or sink.numel() != n_heads or not sink.is_contiguous()):
             raise KernelError("attention_masked: the sinks are contiguous float32 [heads]")
@@ -1317,7 +1396,7 @@ class HipOps:
                 None if vr is None else vr.cos.data_ptr(), None if vr is None else vr.sin.data_ptr(),
                 int(bool(vr is not None and vr.interleaved)), 0 if vr is None else vr.cos.shape[0],
                 _ptr(gsrc), 0 if gsrc is None else _code(gsrc.dtype), gsplits, ground, gstride, int(gate_col), int(gate_elems),
-                _ptr(distance_bias), 0 if distance_bias is None else distance_bias.shape[0], _ptr(sink), self._stream(),
+                _ptr(distance_bias), 0 if distance_bias is None else distance_bias.shape[0], _ptr(sink), int(bool(chunked)), self._stream(),
             )
         )
         return out
@@ -1341,11 +1420,12 @@ class HipOps:
         return out
 
     # ------------------------------------------------ short convolution + gated linear recurrence
-    def causal_conv(self, x, weight, bias, state, ctx, act: Optional[str] = None) -> torch.Tensor:
+    def causal_conv(self, x, weight, bias, state, ctx, act: Optional[str] = None, move_state: bool = False) -> torch.Tensor:
         """Per channel, u_t = bias + sum_j weight[c, j] * x_(t - (taps - 1 - j)) over each request's
-        span; inputs before the span come from ``state`` [slots, taps - 1, channels] (not changed here).
-        ``x`` [N, channels] may be a view with a row stride.  ``act`` = "silu": applied to u (float32)
-        before it is rounded."""
+        span; inputs before the span come from ``state`` [slots, taps - 1, channels] (not changed here unless
+        ``move_state``: it then takes in each request's span, as ``conv_state_push`` would; in a step of single
+        tokens the same launch does it).  ``x`` [N, channels] may be a view with a row stride.  ``act`` = "silu":
+        applied to u (float32) before it is rounded."""
         if act not in (None, "silu"):
             raise KernelError(f"causal_conv: activation {act!r} is not offered")
         n, channels = x.shape
@@ -1358,13 +1438,16 @@ class HipOps:
             raise KernelError(f"causal_conv: state {tuple(state.shape)} does not hold {taps - 1} inputs of {channels} channels")
         out = torch.empty((n, channels), dtype=x.dtype, device=x.device)
         a = ctx.arrays
+        inside = bool(move_state and taps > 1 and ctx.max_qlen == 1)
         self._check(
             self.lib.yk_causal_conv(
                 x.data_ptr(), x.stride(0), _code(x.dtype), weight.data_ptr(), _ptr(bias), _code(weight.dtype), _ptr(state),
                 a["token_seq"].data_ptr(), a["seq_qstart"].data_ptr(), a["state_slots"].data_ptr(), out.data_ptr(),
-                n, channels, taps, int(act == "silu"), self._stream(),
+                n, channels, taps, int(act == "silu"), int(inside), self._stream(),
             )
         )
+        if move_state and taps > 1 and not inside:
+            self.conv_state_push(x, state, ctx)
         return out
 
     # ------------------------------------------------- norms on both sides of a branch, plain feed-forward
@@ -1592,17 +1675,20 @@ class HipOps:
             a["state_slots"].data_ptr(), a["seq_qstart"].numel(), state.shape[1], channels, self._stream()))
 
     def linear_state_scan(self, qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, unit_eps=None, decay=None, beta=None,
-                          columns=None, skip=None):
+                          columns=None, skip=None, bonus=None):
         """The recurrence S <- diag(a) S; u = v or beta (v - S^T k); S += k u^T; o = S^T q over each
         request's span, S [slots, heads, dim, vdim] float32 updated in place.  ``qkv`` [N, >= 2 * kv_heads *
         dim + heads * vdim]: columns [q | k | v].  ``unit_eps``: q and k are divided by sqrt(sum of squares +
         unit_eps) first; q is multiplied by ``q_scale``.  ``decay``: ("head", x, col, A_log, dt_bias): a =
         exp(-exp(A_log) softplus(x[:, col + h] + dt_bias)); ("channel", z, col, bias, tau): a_i = sigmoid(z[:,
-        col + h * dim + i] + bias)^(1 / tau); x, z float32.  ``beta``: (x, col) -> sigmoid(x[:, col + h]), or
+        col + h * dim + i] + bias)^(1 / tau); ("channel_softplus", z, col, A_log, dt_bias): a_i = exp(-exp(A_log_h)
+        softplus(z[:, col + h * dim + i] + dt_bias)); ("channel_exp", z, col, bias): a_i = exp(-exp(z[:, col + h * dim + i] +
+        bias)); x, z float32.  ``beta``: (x, col) -> sigmoid(x[:, col + h]), x float32 or of ``qkv``'s dtype, or
         None for plain writes, or "step": u = dt v with the step dt = softplus(x[:, col + h] + dt_bias) of the head's
         decay.  ``columns`` = (q, k, v): where the kv heads' queries and keys and the heads' values start in a row
-        (default 0, n_kv * dim, 2 * n_kv * dim).  ``skip`` (float32 [heads]): o += skip_h v.  Returns o float32 [N,
-        heads * vdim]."""
+        (default 0, n_kv * dim, 2 * n_kv * dim).  ``skip`` (float32 [heads]): o += skip_h v.  ``bonus`` (float32
+        [heads, dim], plain writes): o = (S + diag(bonus) k v^T)^T q of the memory before the token's decay and write.
+        Returns o float32 [N, heads * vdim]."""
         self._rows(qkv, "linear_state_scan input")
         n = qkv.shape[0]
         if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (n_heads, dim, vdim):
@@ -1617,8 +1703,10 @@ class HipOps:
         q_col, k_col, v_col = columns if columns is not None else (0, n_kv * dim, 2 * n_kv * dim)
         if skip is not None and (skip.dtype != torch.float32 or skip.numel() != n_heads or not skip.is_contiguous()):
             raise KernelError("linear_state_scan: the skip is contiguous float32, one number per head")
+        if bonus is not None and (bonus.dtype != torch.float32 or bonus.numel() != n_heads * dim or not bonus.is_contiguous() or write_mode or skip is not None):
+            raise KernelError("linear_state_scan: the bonus is contiguous float32 [heads, dim] and goes with plain writes and no skip")
         for t, what, cols in ((src, "decay", col + need),) + (((beta[0], "beta", int(beta[1]) + n_heads),) if beta is not None else ()):
-            if t.dtype != torch.float32 or t.dim() != 2 or t.stride(1) != 1 or t.shape[0] != n or t.shape[1] < cols:
+            if (t.dtype != torch.float32 and not (what == "beta" and t.dtype == qkv.dtype)) or t.dim() != 2 or t.stride(1) != 1 or t.shape[0] != n or t.shape[1] < cols:
                 raise KernelError(f"linear_state_scan: the {what}'s input must be float32 rows of at least {cols} columns")
         if kind == "head":
             p0, p1, tau = decay[3], decay[4], 1.0
@@ -1626,39 +1714,136 @@ class HipOps:
         elif kind == "channel":
             p0, p1, tau = decay[3], None, float(decay[4])
             ok = p0.dtype == torch.float32 and p0.numel() == n_heads * dim and p0.is_contiguous()
+        elif kind == "channel_softplus":
+            p0, p1, tau = decay[3], decay[4], 1.0
+            ok = all(p.dtype == torch.float32 and p.numel() == size and p.is_contiguous() for p, size in ((p0, n_heads), (p1, n_heads * dim)))
+        elif kind == "channel_exp":
+            p0, p1, tau = decay[3], None, 1.0
+            ok = p0.dtype == torch.float32 and p0.numel() == n_heads * dim and p0.is_contiguous()
         else:
             raise KernelError(f"linear_state_scan: unknown kind of decay {kind!r}")
         if not ok:
             raise KernelError("linear_state_scan: the decay's constants must be contiguous float32 of the heads' size")
         a = ctx.arrays
+        mode = {"head": 0, "channel": 1, "channel_softplus": 2, "channel_exp": 3}[kind]
+        beta_f32 = beta is not None and beta[0].dtype == torch.float32
         out = torch.empty((n, n_heads * vdim), dtype=torch.float32, device=qkv.device)
         self._check(self.lib.yk_linear_state_scan(
             qkv.data_ptr(), qkv.stride(0), _code(qkv.dtype), n_heads, n_kv, dim, vdim, state.data_ptr(), a["seq_qstart"].data_ptr(),
             a["seq_qlen"].data_ptr(), a["state_slots"].data_ptr(), a["seq_qstart"].numel(), n, float(q_scale),
-            -1.0 if unit_eps is None else float(unit_eps), 0 if kind == "head" else 1, src.data_ptr(), src.stride(0), col,
-            p0.data_ptr(), _ptr(p1), tau, None if beta is None else beta[0].data_ptr(), 0 if beta is None else beta[0].stride(0),
+            -1.0 if unit_eps is None else float(unit_eps), mode, src.data_ptr(), src.stride(0), col,
+            p0.data_ptr(), _ptr(p1), tau, beta[0].data_ptr() if beta_f32 else None, 0 if beta is None else beta[0].stride(0),
             0 if beta is None else int(beta[1]), out.data_ptr(), int(q_col), int(k_col), int(v_col), write_mode, _ptr(skip),
-            self._stream()))
+            beta[0].data_ptr() if beta is not None and not beta_f32 else None, _ptr(bonus), self._stream()))
         return out
 
-    def gated_head_norm(self, o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first: bool = False) -> torch.Tensor:
+    def gated_head_norm(self, o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first: bool = False,
+                        gate_act: str = "silu") -> torch.Tensor:
         """Per head, o / sqrt(mean(o^2) + eps) * weight * silu(gate[:, gate_col + h * vdim + .]); ``o`` float32
         [N, heads * vdim], ``weight`` [vdim] shared by the heads, or [heads * vdim].  The "heads" are whatever equal
         parts of a row are normed each by its own root mean square.  ``gate_first``: the gate comes before the
-        norm, rms(o * silu(gate)) * weight."""
+        norm, rms(o * silu(gate)) * weight.  ``gate_act`` "sigmoid": the sigmoid in silu's place.  The gate comes in
+        ``out_dtype`` or float32."""
+        if gate_act not in ("silu", "sigmoid"):
+            raise KernelError(f"gated_head_norm: gate {gate_act!r} is not offered")
         n = o.shape[0]
         self._rows(gate, "gated_head_norm gate")
         if o.dtype != torch.float32 or not o.is_contiguous() or o.shape[1] != n_heads * vdim or weight.numel() not in (vdim, n_heads * vdim) \
                 or not weight.is_contiguous():
             raise KernelError("gated_head_norm: o is contiguous float32 [N, heads * vdim], the weight [vdim] or [heads * vdim]")
-        if gate.dtype != out_dtype or gate.shape[0] != n or gate.shape[1] < gate_col + n_heads * vdim:
+        if gate.dtype not in (out_dtype, torch.float32) or gate.shape[0] != n or gate.shape[1] < gate_col + n_heads * vdim:
             raise KernelError("gated_head_norm: the gate does not fit")
         out = torch.empty((n, n_heads * vdim), dtype=out_dtype, device=o.device)
         self._check(self.lib.yk_gated_head_norm(
             o.data_ptr(), weight.data_ptr(), _code(weight.dtype), float(eps), gate.data_ptr(), _code(gate.dtype), gate.stride(0),
             gate_col, n_heads, vdim, out.data_ptr(), _code(out_dtype), n, int(weight.numel() != vdim or n_heads == 1),
-            int(bool(gate_first)), self._stream()))
+            int(bool(gate_first)), int(gate_act == "sigmoid"), self._stream()))
         return out
+
+    # ------------------------------------------------- inputs mixed with the token before's, low-rank pairs
+    def token_shift_mix(self, x, mu, state, ctx) -> torch.Tensor:
+        """[mixes, N, width]: x + (x' - x) * mu[s] for every row of ``mu`` (float32 [mixes, width]), x' the row of the
+        request's token before (``state`` [slots, width] for a span's first one; it is left at the span's last row)."""
+        self._rows(x, "token_shift_mix input")
+        n, width = x.shape
+        if not x.is_contiguous() or mu.dtype != torch.float32 or mu.dim() != 2 or mu.shape[1] != width or not mu.is_contiguous():
+            raise KernelError("token_shift_mix: contiguous rows, and float32 mixes [mixes, width]")
+        if state.dtype != x.dtype or tuple(state.shape[1:]) != (width,) or not state.is_contiguous():
+            raise KernelError(f"token_shift_mix: the state {tuple(state.shape)} does not hold a row of {width}")
+        a = ctx.arrays
+        out = torch.empty((mu.shape[0], n, width), dtype=x.dtype, device=x.device)
+        self._check(self.lib.yk_token_shift_mix(
+            x.data_ptr(), _code(x.dtype), mu.data_ptr(), mu.shape[0], state.data_ptr(), a["token_seq"].data_ptr(), a["seq_qstart"].data_ptr(),
+            a["seq_qlen"].data_ptr(), a["state_slots"].data_ptr(), out.data_ptr(), n, width, self._stream()))
+        return out
+
+    def grouped_linear(self, x, w, group_rows: int, out_dtype) -> torch.Tensor:
+        """``w``'s rows come in groups of ``group_rows`` (the last may have fewer), each with an input of its own: columns
+        g * group_rows .. of the result are x[g] . (group g of w)^T.  ``x`` [groups, N, K].  Few rows of bfloat16 run as one
+        launch; otherwise a product a group, each writing its columns."""
+        groups, m, k = x.shape
+        n = w.shape[0]
+        self._rows(w, "grouped_linear weight")
+        if w.shape[1] != k or not x.is_contiguous() or group_rows < 1 or -(-n // group_rows) != groups:
+            raise KernelError(f"grouped_linear: {groups} inputs of {k} columns against {n} rows in groups of {group_rows}")
+        y = torch.empty((m, n), dtype=out_dtype, device=x.device)
+        if m == 0:
+            return y
+        bf = torch.bfloat16
+        aligned = x.dtype == bf and w.dtype == bf and k % 8 == 0 and w.stride(0) % 8 == 0 and w.data_ptr() % 16 == 0 and x.data_ptr() % 16 == 0
+        if aligned and m <= 32 and group_rows % 64 == 0:
+            splits = self._ask("yk_gemm_skinny_splits", m, n, k, 0)
+            ws = self._gemm_ws(splits * m * n) if splits > 1 else None
+            self._check(self.lib.yk_gemm_mfma_skinny_grouped(
+                x.data_ptr(), m * k, group_rows, w.data_ptr(), y.data_ptr(), _code(out_dtype), _ptr(ws), 0 if ws is None else ws.numel(),
+                m, n, k, k, w.stride(0), n, self._stream()))
+            return y
+        size = y.element_size()
+        for g in range(groups):
+            rows = min(group_rows, n - g * group_rows)
+            xg, wg, yp = x[g], w[g * group_rows:], y.data_ptr() + g * group_rows * size
+            if aligned and m > SKINNY_MAX_ROWS and rows >= 64 and yp % 16 == 0 and wg.data_ptr() % 16 == 0 and xg.data_ptr() % 16 == 0 and (n * size) % 16 == 0:
+                if self._library_workspace is None:
+                    self._library_workspace = torch.empty(self.LIBRARY_WORKSPACE_BYTES, dtype=torch.uint8, device=self.device)
+                self._check(self.lib.yk_gemm_library(
+                    xg.data_ptr(), wg.data_ptr(), yp, _code(out_dtype), m, rows, k, k, w.stride(0), n, self._library_workspace.data_ptr(),
+                    self._library_workspace.numel(), None, self._stream()))
+            elif aligned and wg.data_ptr() % 16 == 0 and xg.data_ptr() % 16 == 0:
+                splits = self._ask("yk_gemm_skinny_splits", m, rows, k, 0)
+                ws = self._gemm_ws(splits * m * rows) if splits > 1 else None
+                rc = self.lib.yk_gemm_mfma_skinny(
+                    xg.data_ptr(), wg.data_ptr(), yp, _code(out_dtype), _ptr(ws), 0 if ws is None else ws.numel(), m, rows, k, k, w.stride(0),
+                    n, 0, 0, self._stream())
+                if rc < 0:
+                    self._check(rc)
+            else:
+                self._check(self.lib.yk_gemm_fma(xg.data_ptr(), _code(x.dtype), wg.data_ptr(), _code(w.dtype), yp, _code(out_dtype), m, rows, k,
+                                                 k, w.stride(0), n, self._stream()))
+        return y
+
+    LOW_RANK_ACTS = {None: 0, "tanh": 1}
+
+    def low_rank(self, y, w, act: Optional[str] = None) -> torch.Tensor:
+        """float32 act(y) . w^T: the second product of a low-rank pair, ``y`` [N, rank] (a view with a row stride may be given),
+        ``w`` [columns, rank].  Few tokens: one launch, the activation and the sums in float32.  Many: the activation's rows,
+        rounded, and a product."""
+        if act not in self.LOW_RANK_ACTS:
+            raise KernelError(f"low_rank: activation {act!r} is not offered")
+        self._rows(y, "low_rank input")
+        n, rank = y.shape
+        if w.dim() != 2 or w.shape[1] != rank or not w.is_contiguous():
+            raise KernelError(f"low_rank: the weight {tuple(w.shape)} does not take rows of {rank}")
+        code = self.LOW_RANK_ACTS[act]
+        if n <= SKINNY_MAX_ROWS and rank <= 1536 and (y.dtype == torch.bfloat16 or w.dtype == torch.float32):
+            out = torch.empty((n, w.shape[0]), dtype=torch.float32, device=y.device)
+            self._check(self.lib.yk_low_rank(y.data_ptr(), y.stride(0), _code(y.dtype), w.data_ptr(), _code(w.dtype), code, out.data_ptr(), n,
+                                             w.shape[0], rank, self._stream()))
+            return out
+        if code:
+            rows = torch.empty((n, rank), dtype=y.dtype, device=y.device)
+            self._check(self.lib.yk_act_rows(y.data_ptr(), y.stride(0), _code(y.dtype), code, rows.data_ptr(), n, rank, self._stream()))
+            y = rows
+        return self.linear(y, w, torch.float32)
 
     # spans of more than this many tokens are scanned in chunks (cut by the caller)
     RGLRU_CHUNKED_FROM = 32

@@ -38,8 +38,12 @@ biases of the q and k projections below the prefix, added in float32 before ever
 qk_norm["over"] ("head", the default, or "projection": one RMS norm over all of a token's query
 heads together, and one over all its key heads, with weights as wide as the projections),
 query_temperature ({"coef": c, "every": e}: the query at position p is multiplied by
-1 + c ln(floor((p + 1) / e) + 1), after the norm).  A layer may have no position encoding at all
-(``position`` None).
+1 + c ln(floor((p + 1) / e) + 1), after the norm), chunked (True: the window does not slide, the query at
+position p sees the keys from floor(p / window) * window on, counted from the sequence's start), sink_score (a
+number: a sink of that score for every head, without a tensor), qk_norm without "q" and "k" (queries and keys are
+divided by their root mean square per head and multiplied by no weight; since a rotation changes no pair's length
+this is the same before the rotation as after it).  A layer may have no position encoding at all (``position``
+None).
 """
 from __future__ import annotations
 
@@ -102,13 +106,25 @@ class Attention(Mixer):
         self.distance_bias = params.get("distance_bias")
         self.bias_by_distance = None
         self.sink_name = params.get("sink")
+        self.sink_score = params.get("sink_score")
+        if self.sink_name and self.sink_score is not None:
+            raise ValueError(f"{self.prefix}: a sink's scores are a tensor or one number, not both")
         self.sink = None
+        self.chunked = bool(params.get("chunked", False))
+        if self.chunked and (not self.window or self.keep_first):
+            raise ValueError(f"{self.prefix}: chunks need a window (their size) and keep no first keys")
         self.values_from_keys = bool(params.get("values_from_keys", False))
         if self.values_from_keys and self.value_dim != self.head_dim:
             raise ValueError(f"{self.prefix}: values that are the keys are as wide as the keys")
         self.projection_bias = dict(params.get("projection_bias") or {})
         if set(self.projection_bias) - {"q", "k"}:
             raise ValueError(f"{self.prefix}: projection_bias names the biases of q and k")
+        # (a norm without weights divides each head by its own root mean square)
+        self.qk_norm_weights = bool(self.qk_norm) and self.qk_norm.get("q") is not None
+        if self.qk_norm and self.qk_norm_weights != (self.qk_norm.get("k") is not None):
+            raise ValueError(f"{self.prefix}: queries' and keys' norms both have weights, or neither does")
+        if self.qk_norm and not self.qk_norm_weights and self.qk_norm.get("over", "head") != "head":
+            raise ValueError(f"{self.prefix}: a norm over the whole projection has weights")
         self.norm_over_projection = bool(self.qk_norm) and self.qk_norm.get("over", "head") == "projection"
         if self.qk_norm and self.qk_norm.get("over", "head") not in ("head", "projection"):
             raise ValueError(f"{self.prefix}: qk_norm is over 'head' or 'projection'")
@@ -119,7 +135,7 @@ class Attention(Mixer):
         self.masked = bool(
             self.value_dim != self.head_dim or self.qk_norm or self.value_norm_eps is not None or self.value_rotation is not None
             or self.softcap or self.keep_first or self.gate_name or self.distance_bias or self.sink_name or self.values_from_keys
-            or self.projection_bias or self.query_temperature
+            or self.projection_bias or self.query_temperature or self.chunked or self.sink_score is not None
         )
         self.w_qn = self.w_kn = None
         if self.masked:
@@ -134,7 +150,7 @@ class Attention(Mixer):
             # values of 64 or 128 elements alike); everything else runs on the general float32-arithmetic kernel
             can = getattr(rt.ops, "attention_can_rotate", None)
             self.on_matrix_cores = bool(can is not None and self.value_dim == self.head_dim and can(rt.act_dtype, self.head_dim) is True)
-            if self.on_matrix_cores and self.sink_name:
+            if self.on_matrix_cores and (self.sink_name or self.sink_score is not None):
                 with_sink = getattr(rt.ops, "attention_takes_sink", None)
                 self.on_matrix_cores = bool(with_sink is not None and with_sink(rt.act_dtype, self.head_dim) is True)
             if self.on_matrix_cores:
@@ -173,7 +189,7 @@ class Attention(Mixer):
             specs[self.names["k"]] = TensorSpec((kd, self.hidden))
             if not self.values_from_keys:
                 specs[self.names["v"]] = TensorSpec((self.n_kv * self.value_dim, self.hidden))
-        if self.qk_norm:
+        if self.qk_norm_weights:
             qn, kn = (hd, kd) if self.norm_over_projection else (self.head_dim, self.head_dim)
             specs[f"{self.prefix}.{self.qk_norm['q']}"] = TensorSpec((qn,), "float", ("one_plus_normal", 0.1))
             if self.projects_kv:
@@ -217,13 +233,15 @@ class Attention(Mixer):
                 parts.append(torch.zeros((pad, self.hidden), dtype=q.dtype, device=q.device))
             self.w_qkv = torch.cat(parts, dim=0).contiguous()
             self.w_o = tensors[self.names["o"]]
-            if self.qk_norm:
+            if self.qk_norm_weights:
                 self.w_qn = tensors[f"{self.prefix}.{self.qk_norm['q']}"]
                 self.w_kn = tensors[f"{self.prefix}.{self.qk_norm['k']}"] if self.projects_kv else self.w_qn
             if self.distance_bias:
                 self.bias_by_distance = self._bias_by_distance(tensors[f"{self.prefix}.{self.distance_bias['name']}"])
             if self.sink_name:
                 self.sink = tensors[f"{self.prefix}.{self.sink_name}"].to(torch.float32).contiguous()
+            if self.sink_score is not None:
+                self.sink = torch.full((self.n_heads,), float(self.sink_score), dtype=torch.float32, device=q.device)
             if self.projection_bias:
                 # one float32 vector over the projection's columns: the biases where they are, zeros elsewhere
                 b = torch.zeros(self.w_qkv.shape[0], dtype=torch.float32, device=q.device)
@@ -273,7 +291,7 @@ class Attention(Mixer):
 
     def kv_need(self) -> KVNeed:
         return KVNeed(self.n_kv, self.head_dim, self.window, None if self.value_dim == self.head_dim else self.value_dim,
-                      self.keep_first if self.window else 0)
+                      self.keep_first if self.window else 0, self.chunked)
 
     def products(self):
         hd, kd = self.n_heads * self.head_dim, self.n_kv * self.head_dim
@@ -339,6 +357,8 @@ class Attention(Mixer):
             more["bias"] = self.b_proj
         if self.values_from_keys:
             more["values_from_keys"] = True
+        if self.qk_norm and not self.qk_norm_weights:
+            more["unweighted_norm"] = True
         q = ops.qkv_prepare(
             proj, self.n_heads, n_kv_rows, self.head_dim, self.value_dim, ctx.arrays["positions"], self.rt.act_dtype,
             q_norm=self.w_qn, k_norm=self.w_kn, qk_eps=float(self.qk_norm["eps"]) if self.qk_norm else 0.0,
@@ -348,6 +368,8 @@ class Attention(Mixer):
         )
         gate_col = self.n_heads * self.head_dim + n_kv_rows * (self.head_dim + (0 if self.values_from_keys else self.value_dim))
         sink = {} if self.sink is None else {"sink": self.sink}
+        if self.chunked:
+            sink["chunked"] = True
         if self.on_matrix_cores:
             memo_key = f"attention_long_col_tiles_{self.layout}"
             col_tiles = ctx.memo.get(memo_key)

@@ -40,13 +40,16 @@ class KVNeed:
     0: no values are kept, the pages hold keys only, e.g. one compressed row per token).
     ``window`` = how many of the latest tokens are ever read again (None: all of them);
     ``keep_first`` = how many of the first tokens stay readable whatever the window says (their
-    pages are never given back while the request lives)."""
+    pages are never given back while the request lives); ``chunked``: the window does not slide, it
+    begins anew at every multiple of ``window`` (a token reads its own chunk of that many positions
+    only, so a chunk's pages are given back once the next one begins)."""
 
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     value_dim: Optional[int] = None
     keep_first: int = 0
+    chunked: bool = False
 
     @property
     def v_dim(self) -> int:
@@ -117,6 +120,27 @@ class PlusRow:
             residual += inner.float()
         residual += self.row.to(torch.float32)
         return None
+
+
+class NormedSum:
+    """A mixer's output that is ``scale`` times the sum of several rows, each first divided by its root
+    mean square (its ``eps`` under the root) and multiplied by its ``weight``: ``terms`` is a tuple of
+    (rows, weight, eps), with weight None for rows that are added as they are.  A norm's ``sum_norm``
+    takes the sum while it reads the rows; ``combine()`` gives the tensor for whoever cannot."""
+
+    def __init__(self, ops, terms, scale: float = 1.0):
+        self.ops, self.terms, self.scale = ops, tuple(terms), float(scale)
+        self.shape = tuple(self.terms[0][0].shape)
+
+    def combine(self) -> torch.Tensor:
+        out = None
+        for rows, weight, eps in self.terms:
+            y = rows.float() if weight is None else self.ops.rmsnorm(rows, weight, eps, False, torch.float32)
+            out = y if out is None else out + y
+        return out * self.scale
+
+    def float(self) -> torch.Tensor:
+        return self.combine()
 
 
 class Part:
@@ -227,6 +251,12 @@ class Norm(Part):
         the stream.  ``branch`` is whatever a part's ``forward`` returned, and / or the uncombined rows
         of a mixture of experts (``FeedForward.forward`` may return an ``ExpertRows``).  Returns the
         new residual in the activation dtype."""
+        raise NotImplementedError
+
+    def sum_norm(self, residual: torch.Tensor, branch, residual_scale: float = 1.0) -> torch.Tensor:
+        """residual (float32, in place) = norm(residual_scale * residual + branch): the stream itself is normed
+        after the branch has joined it.  ``branch`` is whatever a part's ``forward`` returned (a ``NormedSum``
+        included).  Returns the new residual in the activation dtype."""
         raise NotImplementedError
 
 

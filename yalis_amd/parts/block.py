@@ -12,7 +12,7 @@ returns its own last contribution, to be added by whoever comes next.
 """
 from __future__ import annotations
 
-from .base import Block, ExpertRows, NormedBranch, PlusRow, Settled, register_block
+from .base import Block, ExpertRows, NormedBranch, NormedSum, PlusRow, Settled, register_block
 
 
 @register_block("prenorm")
@@ -79,9 +79,25 @@ class ParallelBlock(Block):
             f = ExpertRows(None, f.float().contiguous(), 1, 1.0)
         dense = None if f.dense is None else f.dense.float().contiguous()
         a = self.mixer.forward(h, ctx, site)
+        if isinstance(a, NormedSum):
+            a = a.combine()
         if dense is not None:
             a = ops.moe_combine(a, dense, 1, 1.0)
         return ops.moe_combine(a, f.rows, f.top, f.weight, row_weights=f.row_weights)
+
+
+def _stream(residual, delta, rt):
+    """The stream itself in the activation dtype, for a branch that reads it un-normed: whatever a block of
+    another kind left pending is added first (as it is); a ``Settled`` stream is there already."""
+    if isinstance(delta, PlusRow):
+        delta = delta.settle(residual)
+    if isinstance(delta, Settled):
+        return delta.activations
+    if isinstance(delta, NormedBranch):
+        delta = delta.settle(residual)
+    if delta is not None:
+        residual += delta.float()
+    return rt.ops.round_rows(residual, rt.act_dtype)
 
 
 @register_block("branch_norm")
@@ -110,17 +126,42 @@ class BranchNormBlock(Block):
         self.feed_forward_norm = feed_forward_norm
 
     def forward(self, residual, delta, ctx, site):
-        if isinstance(delta, PlusRow):
-            delta = delta.settle(residual)
-        if isinstance(delta, Settled):
-            h = delta.activations
-        else:
-            if delta is not None:  # a block of another kind left a contribution: it is added as it is
-                residual += delta.float()
-            h = self.mixer.rt.ops.round_rows(residual, self.mixer.rt.act_dtype)
+        h = _stream(residual, delta, self.mixer.rt)
         h = self.mixer_norm.norm_add(residual, self.mixer.forward(h, ctx, site))
         if self.feed_forward is not None:
             h = self.feed_forward_norm.norm_add(residual, self.feed_forward.forward(h, ctx))
+        return Settled(h)
+
+
+@register_block("post_norm")
+class PostNormBlock(Block):
+    """Norms after the sums: x = norm_1(a x + mixer(x)); x = norm_2(a x + feed_forward(x)).  The branches read
+    the stream itself, and the normed sum is the new stream.  A layer may leave the feed-forward (and its norm)
+    out.  ``residual_scale`` is a; a norm's ``branch_weight`` multiplies its branch element by element first.
+
+    One kernel between two branches (``Norm.sum_norm``): it sums the branch (a product's slices, or a mixer's
+    ``NormedSum``), adds it to the scaled stream, norms the sum, and writes the float32 stream and its rounded
+    copy, which is handed on as ``Settled``."""
+
+    roles = {
+        "mixer": ("mixer", True),
+        "mixer_norm": ("norm", True),
+        "feed_forward": ("feed_forward", False),
+        "feed_forward_norm": ("norm", False),
+    }
+
+    def __init__(self, mixer, mixer_norm, feed_forward=None, feed_forward_norm=None, residual_scale: float = 1.0):
+        if (feed_forward is None) != (feed_forward_norm is None):
+            raise ValueError("a post_norm block has a feed-forward and its norm, or neither")
+        self.mixer, self.mixer_norm = mixer, mixer_norm
+        self.feed_forward, self.feed_forward_norm = feed_forward, feed_forward_norm
+        self.residual_scale = float(residual_scale)
+
+    def forward(self, residual, delta, ctx, site):
+        h = _stream(residual, delta, self.mixer.rt)
+        h = self.mixer_norm.sum_norm(residual, self.mixer.forward(h, ctx, site), self.residual_scale)
+        if self.feed_forward is not None:
+            h = self.feed_forward_norm.sum_norm(residual, self.feed_forward.forward(h, ctx), self.residual_scale)
         return Settled(h)
 
 

@@ -13,7 +13,7 @@ from typing import Dict, Mapping
 import torch
 
 from ..weights.loader import TensorSpec
-from .base import Part, Runtime, register_embedding, register_head
+from .base import Part, Runtime, Settled, StateNeed, register_embedding, register_head
 
 
 @register_embedding("token_embedding")
@@ -82,6 +82,47 @@ class TokenPositionEmbedding(TokenEmbedding):
 
     def begin(self, token_ids: torch.Tensor, lazily: bool, positions: torch.Tensor = None):
         return self.forward(token_ids, positions), None
+
+
+@register_embedding("token_pair_embedding")
+class TokenPairEmbedding(TokenEmbedding):
+    """The token's scaled row plus a row for the pair (token before it, token), summed in float32: row
+    (before * mul_prev + token * mul_cur) mod buckets of a second table [buckets + 1, hidden]; a sequence's
+    first token, which has none before it, takes the last row.  The token before a step's first one is the
+    request's state (one int32, -1 before the first token).
+
+    params: name, vocab_size, hidden_size, scale, pair_name, buckets, mul_prev, mul_cur."""
+
+    graph_capturable = True
+    keeps_state = True
+
+    def __init__(self, params, rt: Runtime):
+        super().__init__(params, rt)
+        self.pair_name = params["pair_name"]
+        self.buckets = int(params["buckets"])
+        self.mul_prev, self.mul_cur = int(params["mul_prev"]), int(params["mul_cur"])
+        # (the row number is an unsigned 64-bit sum on the device)
+        if min(self.mul_prev, self.mul_cur) < 0 or max(self.mul_prev, self.mul_cur) * self.vocab >= 1 << 62:
+            raise ValueError(f"{self.pair_name}: multipliers {self.mul_prev} and {self.mul_cur} are out of range")
+        self.pair_table = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return {self.name: TensorSpec((self.vocab, self.hidden)), self.pair_name: TensorSpec((self.buckets + 1, self.hidden))}
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        self.table, self.pair_table = tensors[self.name].contiguous(), tensors[self.pair_name].contiguous()
+        if self.pair_table.dtype != self.table.dtype:
+            self.table, self.pair_table = self.table.float(), self.pair_table.float()
+
+    def state_need(self) -> StateNeed:
+        return StateNeed((1,), torch.int32, -1)
+
+    def begin(self, ctx, site):
+        """(the float32 residual stream, ``Settled`` with its copy in the activation dtype)."""
+        residual, rounded = self.rt.ops.embed_pairs(
+            ctx.arrays["token_ids"], self.table, self.scale, self.pair_table, self.buckets, self.mul_prev, self.mul_cur,
+            site.state(0), ctx, self.rt.act_dtype)
+        return residual, Settled(rounded)
 
 
 @register_head("lm_head")

@@ -7,8 +7,8 @@ outer product k u^T into it and reads q out of it:
     u  = beta (v - S^T k)           the delta rule        ("delta_rule")
     S <- S + k u^T,   o = S^T q     (the read-out sees the token's own write)
 
-and each head's o is divided by its root mean square, multiplied by a weight shared by the heads and
-by silu of a projection of the mixer's input, and projected back.  Decays, write strengths, unit
+and each head's o is divided by its root mean square, multiplied by a weight (shared by the heads, or one per
+element) and by silu or the sigmoid of a projection of the mixer's input, and projected back.  Decays, write strengths, unit
 norms, S and the read-out norm are float32 in both engines; one kernel (``ops.linear_state_scan``)
 walks every request's span with S in registers, one column of S to a group of lanes.
 
@@ -16,6 +16,14 @@ walks every request's span with S in registers, one column of S to a group of la
 by groups of value heads) and v pass a causal convolution per channel (``conv_taps``, silu), q and
 k are made unit vectors (q also times head_dim^-1/2); beta = sigmoid(W_b h) and the head's decay
 exp(-exp(A_log) softplus(W_a h + dt_bias)).  The convolution's last inputs are a second state.
+
+"channel_delta_rule": the delta rule with a decay of its own per key channel, exp(-exp(A_log_h) softplus(z + dt_bias)) with
+z = W_a2 (W_a1 h), and a read-out gate of low rank, the sigmoid of W_g2 (W_g1 h).
+
+"time_mixing" (Peng et al., "Eagle and Finch: RWKV with Matrix-Valued States and Dynamic Recurrence"): every projection reads
+a mix of its own of the token's and the token before's input, h + (h' - h) mu; decay per channel exp(-exp(W_w2 tanh(W_w1 .) + w0));
+plain writes, and the read-out sees the memory as it was before the token plus the token's own write weighed by a bonus
+per channel: o = (S + diag(b) k v^T)^T q, then S <- diag(a) S + k v^T.  The token before's input is a second state.
 
 "gated_linear_attention" (Yang et al., "Gated Linear Attention Transformers with Hardware-Efficient Training"): q times head_dim^-1/2, decay per key
 channel sigmoid(z)^(1/tau) with z = W_a2 (W_a1 h) + b.
@@ -73,9 +81,10 @@ class _MatrixStateMixer(Mixer):
     def _state(self) -> StateNeed:
         return StateNeed((self.n_heads, self.head_dim, self.value_dim), torch.float32, 0.0)
 
-    def _finish(self, o, proj, gate_col):
+    def _finish(self, o, proj, gate_col, gate_act="silu"):
         ops = self.rt.ops
-        y = ops.gated_head_norm(o, self.w_norm, self.out_eps, proj, gate_col, self.n_heads, self.value_dim, self.rt.act_dtype)
+        y = ops.gated_head_norm(o, self.w_norm, self.out_eps, proj, gate_col, self.n_heads, self.value_dim, self.rt.act_dtype,
+                                gate_act=gate_act)
         return ops.linear(y, self.w_o, self.rt.act_dtype, partial_ok=True)
 
 
@@ -124,20 +133,150 @@ class DeltaRule(_MatrixStateMixer):
         rows = self.gate_col + self.v_cols
         return ((rows + (-rows % 16), self.hidden), (2 * self.n_heads + (-2 * self.n_heads % 16), self.hidden), (self.hidden, self.v_cols))
 
+    def _convolved(self, proj, ctx, site):
+        x = proj[:, : self.conv_cols]
+        conv_state = site.state(1) if self.taps > 1 else None
+        return self.rt.ops.causal_conv(x, self.w_conv, None, conv_state, ctx, act="silu", move_state=True)
+
     def forward(self, h: torch.Tensor, ctx, site) -> torch.Tensor:
         ops, act = self.rt.ops, self.rt.act_dtype
         proj = ops.linear(h, self.w_in, act)
         ba = ops.linear(h, self.w_ba, torch.float32)  # [beta's logit | the decay's] per head, float32
-        x = proj[:, : self.conv_cols]
-        conv_state = site.state(1) if self.taps > 1 else None
-        u = ops.causal_conv(x, self.w_conv, None, conv_state, ctx, act="silu")
-        if conv_state is not None:
-            ops.conv_state_push(x, conv_state, ctx)
+        u = self._convolved(proj, ctx, site)
         o = ops.linear_state_scan(
             u, self.n_heads, self.n_kv, self.head_dim, self.value_dim, site.state(0), ctx, q_scale=self.q_scale,
             unit_eps=self.unit_eps, decay=("head", ba, self.n_heads, self.a_log, self.dt_bias), beta=(ba, 0),
         )
         return self._finish(o, proj, self.gate_col)
+
+
+@register_mixer("channel_delta_rule")
+class ChannelDeltaRule(DeltaRule):
+    """params: as "delta_rule" (no tensor "a" or "g": the decay has "a1" and "a2", the gate "g1" and "g2").  The ranks of
+    the two pairs are read from the tensors' shapes."""
+
+    def __init__(self, params, rt: Runtime):
+        super().__init__(params, rt)
+        self.rank_a = self.rank_g = None  # whatever the checkpoint has
+        self.w_low = self.z_cols = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        specs = super().tensor_specs()
+        for short in ("a", "g"):
+            del specs[self._name(short)]
+        kd = self.n_heads * self.head_dim
+        low = max(8, self.hidden // 8)
+        specs.update({
+            self._name("dt_bias"): TensorSpec((kd,), "float", ("normal", 0.5)),
+            self._name("a1"): TensorSpec((low, self.hidden), free_axes=(0,)), self._name("a2"): TensorSpec((kd, low), free_axes=(1,)),
+            self._name("g1"): TensorSpec((low, self.hidden), free_axes=(0,)), self._name("g2"): TensorSpec((self.v_cols, low), free_axes=(1,)),
+        })
+        return specs
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        t = lambda short: tensors[self._name(short)]
+        q, a1, a2, g1, g2 = t("q"), t("a1"), t("a2"), t("g1"), t("g2")
+        self.rank_a, self.rank_g = int(a1.shape[0]), int(g1.shape[0])
+        if a2.shape[1] != self.rank_a or g2.shape[1] != self.rank_g:
+            raise ValueError(f"{self.prefix}: a pair of low-rank projections disagrees on its rank")
+        zeros = lambda rows: torch.zeros((rows, self.hidden), dtype=q.dtype, device=q.device)
+        up8 = lambda n: n + (-n % 8)
+        # one product of everything that reads the mixer's input: [q | k | v | a1 | g1 | beta's logits]
+        self.low_col = up8(self.conv_cols)
+        ra, rg = up8(self.rank_a), up8(self.rank_g)
+        self.low_cols = ra + rg
+        self.beta_col = self.low_col + self.low_cols
+        parts = [q, t("k"), t("v"), zeros(self.low_col - self.conv_cols), a1, zeros(ra - self.rank_a), g1, zeros(rg - self.rank_g), t("b")]
+        self.w_in = _pad_rows([p for p in parts if p.shape[0]], 16)
+        # and one of both second projections, side by side on the diagonal: [decays' logits | gates' logits]
+        kd = a2.shape[0]
+        self.gate_col = up8(kd)
+        self.w_low = torch.zeros((self.gate_col + up8(self.v_cols), self.low_cols), dtype=q.dtype, device=q.device)
+        self.w_low[:kd, : self.rank_a] = a2
+        self.w_low[self.gate_col: self.gate_col + self.v_cols, ra: ra + self.rank_g] = g2
+        self.w_conv = torch.cat([t("q.conv"), t("k.conv"), t("v.conv")], dim=0).contiguous()
+        self.a_log, self.dt_bias = t("A_log").float().contiguous(), t("dt_bias").float().contiguous()
+        self.w_norm, self.w_o = t("norm").contiguous(), t("o")
+
+    def products(self):
+        if self.w_in is None:
+            return ()
+        return tuple(tuple(w.shape) for w in (self.w_in, self.w_low, self.w_o))
+
+    def forward(self, h: torch.Tensor, ctx, site) -> torch.Tensor:
+        ops = self.rt.ops
+        proj = ops.linear(h, self.w_in, self.rt.act_dtype)
+        z = ops.linear(proj[:, self.low_col: self.low_col + self.low_cols], self.w_low, torch.float32)
+        u = self._convolved(proj, ctx, site)
+        o = ops.linear_state_scan(
+            u, self.n_heads, self.n_kv, self.head_dim, self.value_dim, site.state(0), ctx, q_scale=self.q_scale,
+            unit_eps=self.unit_eps, decay=("channel_softplus", z, 0, self.a_log, self.dt_bias), beta=(proj, self.beta_col),
+        )
+        return self._finish(o, z, self.gate_col, gate_act="sigmoid")
+
+
+@register_mixer("time_mixing")
+class TimeMixing(_MatrixStateMixer):
+    """params: prefix, hidden_size, num_heads, head_dim, out_norm_eps, names.  Values are as wide as keys; the rank of the
+    decay's pair of projections is read from the tensors' shapes."""
+
+    MIXES = ("r", "k", "v", "g", "w")  # the order of the mixed inputs; the first four are projected side by side
+
+    def __init__(self, params, rt: Runtime):
+        super().__init__(dict(params, value_dim=params["head_dim"], q_scale=1.0), rt)
+        self.cols = self.n_heads * self.head_dim
+        # rows of one projection among the four (a multiple of 64: few rows of input then take one launch for all)
+        self.rows = self.cols + (-self.cols % 64)
+        self.mu = self.w_in = self.w_2 = self.w_0 = self.bonus = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        c, low = self.cols, max(8, self.hidden // 16)
+        specs = {self._name(f"mu.{s}"): TensorSpec((self.hidden,), "float", ("normal", 0.5)) for s in self.MIXES}
+        specs.update({self._name(s): TensorSpec((c, self.hidden)) for s in self.MIXES[:4]})
+        specs.update({
+            self._name("w1"): TensorSpec((low, self.hidden), free_axes=(0,)), self._name("w2"): TensorSpec((c, low), free_axes=(1,)),
+            self._name("w0"): TensorSpec((c,), "float", ("normal", 1.0)),
+            self._name("u"): TensorSpec((self.n_heads, self.head_dim), "float", ("normal", 0.5)),
+            self._name("norm"): TensorSpec((c,), "float", ("one_plus_normal", 0.1)), self._name("o"): TensorSpec((self.hidden, c)),
+        })
+        return specs
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        t = lambda short: tensors[self._name(short)]
+        self.mu = torch.stack([t(f"mu.{s}").float() for s in self.MIXES]).contiguous()
+        w1, w2 = t("w1"), t("w2")
+        if w2.shape[1] != w1.shape[0]:
+            raise ValueError(f"{self.prefix}: the decay's two projections disagree on their rank")
+        # the fifth group of the grouped product: the decay's first projection (rows of zeros beyond its rank: tanh of
+        # nothing is nothing, and the second's columns are zeros there too)
+        first = _pad_rows([w1], 16)
+        self.rank = first.shape[0]
+        self.rows = max(self.rows, self.rank + (-self.rank % 64))  # (the last group has at most as many rows as the others)
+        self.w_in = torch.cat([_pad_rows([t(s)], self.rows) for s in self.MIXES[:4]] + [first], dim=0).contiguous()
+        self.w_2 = torch.zeros((w2.shape[0], self.rank), dtype=w2.dtype, device=w2.device)
+        self.w_2[:, : w2.shape[1]] = w2
+        self.w_0, self.bonus = t("w0").float().contiguous(), t("u").float().contiguous()
+        self.w_norm, self.w_o = t("norm").contiguous(), t("o")
+
+    def state_need(self):
+        return (self._state(), StateNeed((self.hidden,), self.rt.act_dtype, 0.0))
+
+    def products(self):
+        if self.w_in is None:
+            return ()
+        return ((self.rows, self.hidden), (self.rank, self.hidden), tuple(self.w_in.shape), tuple(self.w_2.shape), tuple(self.w_o.shape))
+
+    def forward(self, h: torch.Tensor, ctx, site) -> torch.Tensor:
+        ops, act = self.rt.ops, self.rt.act_dtype
+        x = ops.token_shift_mix(h, self.mu, site.state(1), ctx)  # [5, N, hidden]; the state moves on to the span's last token
+        # [N, 4 * rows + rank]: r, k, v, the gate and the decay's first projection, each from a mix of its own
+        p = ops.grouped_linear(x, self.w_in, self.rows, act)
+        z = ops.low_rank(p[:, 4 * self.rows: 4 * self.rows + self.rank], self.w_2, "tanh")
+        o = ops.linear_state_scan(
+            p, self.n_heads, self.n_heads, self.head_dim, self.value_dim, site.state(0), ctx, q_scale=1.0, unit_eps=None,
+            decay=("channel_exp", z, 0, self.w_0), beta=None, columns=(0, self.rows, 2 * self.rows), bonus=self.bonus,
+        )
+        return self._finish(o, p, 3 * self.rows)
 
 
 @register_mixer("gated_linear_attention")

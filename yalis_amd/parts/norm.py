@@ -5,7 +5,9 @@ the end; ``unit_offset`` multiplies by (1 + weight) instead (a flag of the same
 class in the reference, :984).  The kernel fuses the residual sum that precedes
 every norm of a pre-norm block: the float32 residual stream is updated in place
 and normalised in one pass.  ``norm_add`` is the other way round, for blocks that norm a
-branch's output instead of its input: residual += norm(branch), again one pass.
+branch's output instead of its input: residual += norm(branch), again one pass.  ``sum_norm`` is
+for blocks that norm the stream itself after the branch has joined it: residual = norm(a * residual +
+branch), with an optional weight per element on the branch (a layer scale), one pass too.
 """
 from __future__ import annotations
 
@@ -14,12 +16,14 @@ from typing import Dict, Mapping, Optional
 import torch
 
 from ..weights.loader import TensorSpec
-from .base import ExpertRows, Norm, NormedBranch, PlusRow, Runtime, Settled, register_norm
+from .base import ExpertRows, Norm, NormedBranch, NormedSum, PlusRow, Runtime, Settled, register_norm
 
 
 @register_norm("rmsnorm")
 class RMSNorm(Norm):
-    """params: name (checkpoint tensor), size, eps, unit_offset."""
+    """params: name (checkpoint tensor), size, eps, unit_offset, branch_weight (None, or the name of a
+    tensor [size]: what ``sum_norm`` multiplies a branch with, element by element, before it joins the
+    stream)."""
 
     graph_capturable = True
 
@@ -30,16 +34,27 @@ class RMSNorm(Norm):
         self.eps = float(params["eps"])
         self.unit_offset = bool(params.get("unit_offset", False))
         self.weight: Optional[torch.Tensor] = None
+        self.branch_weight_name = params.get("branch_weight")
+        self.branch_weight: Optional[torch.Tensor] = None
         self.takes_embedded_rows = hasattr(rt.ops, "embedded_rows")
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         # (random weights: around the value that leaves a row as it is, 0 where 1 is added)
-        return {self.name: TensorSpec((self.size,), "float", ("normal", 0.1) if self.unit_offset else ("one_plus_normal", 0.1))}
+        specs = {self.name: TensorSpec((self.size,), "float", ("normal", 0.1) if self.unit_offset else ("one_plus_normal", 0.1))}
+        if self.branch_weight_name:
+            specs[self.branch_weight_name] = TensorSpec((self.size,), "float", ("one_plus_normal", 0.1))
+        return specs
 
     def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
         self.weight = tensors[self.name]
+        if self.branch_weight_name:
+            self.branch_weight = tensors[self.branch_weight_name].contiguous()
+            if self.branch_weight.dtype != self.weight.dtype:
+                self.weight, self.branch_weight = self.weight.float(), self.branch_weight.float()
 
     def norm(self, x):
+        if isinstance(x, NormedSum):
+            x = x.combine()
         return self.rt.ops.rmsnorm(x, self.weight, self.eps, self.unit_offset, self.rt.act_dtype)
 
     def add_norm(self, residual, delta):
@@ -50,6 +65,8 @@ class RMSNorm(Norm):
             delta = delta.settle(residual)
         if isinstance(delta, Settled):
             delta = None
+        if isinstance(delta, NormedSum):
+            delta = delta.combine()
         if row is not None:
             return self.rt.ops.add_rmsnorm(residual, delta, self.weight, self.eps, self.unit_offset, self.rt.act_dtype, row=row)
         return self.rt.ops.add_rmsnorm(
@@ -59,12 +76,19 @@ class RMSNorm(Norm):
     def norm_add(self, residual, branch, expert_rows=None, expert_weight=1.0, scale=1.0):
         if scale != 1.0:
             raise ValueError("this norm adds its branch unscaled")
-        if isinstance(branch, ExpertRows) and branch.row_weights is not None:
+        if isinstance(branch, NormedSum) or (isinstance(branch, ExpertRows) and branch.row_weights is not None):
             branch = branch.combine()  # (rows with weights of their own are summed first)
         if isinstance(branch, ExpertRows):
             branch, expert_rows, expert_weight = branch.dense, branch.rows, branch.weight
         return self.rt.ops.norm_add(residual, branch, self.weight, self.eps, self.unit_offset, self.rt.act_dtype,
                                     expert_rows=expert_rows, expert_weight=expert_weight)
+
+    def sum_norm(self, residual, branch, residual_scale=1.0):
+        if isinstance(branch, ExpertRows):
+            branch = branch.combine()
+        terms, scale = (branch.terms, branch.scale) if isinstance(branch, NormedSum) else (((branch, None, 0.0),), 1.0)
+        return self.rt.ops.sum_norm(residual, terms, scale, self.branch_weight, residual_scale, self.weight, self.eps,
+                                    self.unit_offset, self.rt.act_dtype)
 
     def gather_add_norm(self, residual, delta, rows):
         if isinstance(delta, PlusRow):
@@ -73,6 +97,8 @@ class RMSNorm(Norm):
             delta = delta.settle(residual)
         if isinstance(delta, Settled):
             delta = None
+        if isinstance(delta, NormedSum):
+            delta = delta.combine()
         return self.rt.ops.gather_add_rmsnorm(
             residual, delta, rows, self.weight, self.eps, self.unit_offset, self.rt.act_dtype
         )
@@ -129,7 +155,7 @@ class LayerNorm(Norm):
                 delta.settle(residual)
                 return None, None, 1.0
             return delta.branch, delta.norm.constants(), delta.scale
-        return delta, None, 1.0
+        return (delta.combine() if isinstance(delta, NormedSum) else delta), None, 1.0
 
     def norm(self, x):
         return self.rt.ops.sandwich_norm(None, x, None, 1.0, self.constants(), None, self.rt.act_dtype)
@@ -143,7 +169,7 @@ class LayerNorm(Norm):
         return self.rt.ops.sandwich_norm(residual, branch, post, scale, self.constants(), rows, self.rt.act_dtype)
 
     def norm_add(self, residual, branch, expert_rows=None, expert_weight=1.0, scale=1.0):
-        if isinstance(branch, ExpertRows):
+        if isinstance(branch, (ExpertRows, NormedSum)):
             branch = branch.combine()
         elif expert_rows is not None:
             raise ValueError("this norm takes its branch combined")
