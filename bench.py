@@ -40,6 +40,10 @@ recurrences) and the Llama configuration of equal size.
 gates, a stretch of layers run twice) beside the Mesolix configuration of equal width, heads, experts and depth (the
 closest of the engine's models: the same attention and grouped-expert kernels) and the Llama configuration of equal
 size.
+``--design rafusun`` measures the Rafusun design (the delta rule with a decay per channel, chunked attention beside time
+mixing, norms after the sums, dense feed-forwards) beside the Nutavik configuration of equal width, heads and
+feed-forward weights (the closest of the engine's models: the same scan of matrix states) and the Llama configuration of
+equal size.
 """
 import argparse
 import json
@@ -400,12 +404,12 @@ def _op_costs(ops, hb):
     def nbytes(*ts):
         return sum(t.numel() * t.element_size() for t in ts if hasattr(t, "numel"))
 
-    def visible(window, keep):
+    def visible(window, keep, chunked=False):
         b = hb()
         total = 0
         for ctx, ql in zip(b.seq_ctx.tolist(), b.seq_qlen.tolist()):
             for p in range(ctx - ql, ctx):
-                total += p + 1 if not window else min(p + 1, window + min(keep, max(0, p + 1 - window)))
+                total += p % window + 1 if chunked else p + 1 if not window else min(p + 1, window + min(keep, max(0, p + 1 - window)))
         return total
 
     def linear(a, kw, out):
@@ -423,16 +427,19 @@ def _op_costs(ops, hb):
 
     def attention_masked(a, kw, out):
         q, heads, kv, d, dv = a[0], a[1], a[2], a[3], a[4]
-        keys = visible(kw.get("window", 0), kw.get("keep_first", 0))
+        keys = visible(kw.get("window", 0), kw.get("keep_first", 0), kw.get("chunked", False))
         b = hb()
         cached = sum(min(c, (kw.get("window") or c) + kw.get("keep_first", 0)) for c in b.seq_ctx.tolist())
         return 2.0 * heads * (d + dv) * keys, 2.0 * kv * (d + dv) * cached + nbytes(q) * 2
 
     def attention(a, kw, out):
         qkv, heads, kv, d = a[0], a[1], a[2], a[3]
-        keys = visible(a[8], 0)
+        chunked = kw.get("chunked", False)
+        keys = visible(a[8], 0, chunked)
         b = hb()
-        return 4.0 * heads * d * keys, 4.0 * kv * d * sum(b.seq_ctx.tolist()) + 4.0 * qkv.shape[0] * heads * d
+        # (chunks: a request's queries read from the first one's chunk on)
+        cached = [c - (c - q) // a[8] * a[8] if chunked else c for c, q in zip(b.seq_ctx.tolist(), b.seq_qlen.tolist())]
+        return 4.0 * heads * d * keys, 4.0 * kv * d * sum(cached) + 4.0 * qkv.shape[0] * heads * d
 
     def rglru(a, kw, out):
         u, wa = a[0], a[3]
@@ -452,6 +459,26 @@ def _op_costs(ops, hb):
         b = hb()
         return 6.0 * qkv.shape[0] * heads * dim * vdim, float(nbytes(qkv, out) + 8.0 * b.n_seqs * heads * dim * vdim)
 
+    def grouped_linear(a, kw, out):
+        x, w = a[0], a[1]
+        return 2.0 * x.shape[1] * w.numel(), float(nbytes(x, w, out))
+
+    def low_rank(a, kw, out):
+        y, w = a[0], a[1]
+        return 2.0 * y.shape[0] * w.numel(), float(nbytes(y, w, out))
+
+    def sum_norm(a, kw, out):
+        # the stream read and written, its rounded copy, and every term's rows as they came (a tensor or slices)
+        terms = [getattr(t[0], "tensor", t[0]) for t in a[1]]
+        return 0.0, float(2 * nbytes(a[0]) + nbytes(out) + nbytes(*terms))
+
+    def token_shift_mix(a, kw, out):
+        return 0.0, float(nbytes(a[0], a[1], out))
+
+    def embed_pairs(a, kw, out):
+        n, width = a[0].numel(), a[1].shape[1]
+        return 0.0, float(n * width * (2 * a[1].element_size() + 4 + 2))
+
     def moved(a, kw, out):
         return 0.0, float(nbytes(*a, *kw.values()) + (nbytes(out) if hasattr(out, "numel") else 0))
 
@@ -460,7 +487,9 @@ def _op_costs(ops, hb):
             "rope_append": moved, "causal_conv": moved, "gated_act": moved, "round_rows": moved, "embed": moved,
             "sandwich_norm": moved, "activation": moved, "latent_prepare": moved, "head_linear": head_linear,
             "latent_attention": latent_attention, "linear_state_scan": state_scan, "gated_head_norm": moved, "conv_state_push": moved, "moe_router_topk": moved,
-            "moe_combine": moved, "attention_finish": moved, "qk_row_scales": moved}
+            "moe_combine": moved, "attention_finish": moved, "qk_row_scales": moved,
+            "grouped_linear": grouped_linear, "low_rank": low_rank, "sum_norm": sum_norm, "token_shift_mix": token_shift_mix,
+            "embed_pairs": embed_pairs, "rmsnorm": moved}
 
 
 def per_op_times(runner, vocab: int, gen, batch: int, prompt_len: int, prefill_len: int):
@@ -553,7 +582,7 @@ def design_compare(args) -> int:
     from yalis_amd.models.presets import layer_runs, llama_like, mesolix_like, nutavik_like
 
     sizes = {"suranex": ("suranex-2k", "suranex-4k"), "nutavik": ("nutavik-2k", "nutavik-4k"), "mesolix": ("mesolix-2k", "mesolix-4k"),
-             "bekedra": ("bekedra-2k", "bekedra-4k")}[args.design]
+             "bekedra": ("bekedra-2k", "bekedra-4k"), "rafusun": ("rafusun-2k", "rafusun-4k")}[args.design]
     if args.design_shape:
         sizes = (args.design_shape,)
     for name in sizes:
@@ -561,7 +590,7 @@ def design_compare(args) -> int:
         line = {"design": args.design, "shape": label, "batch": args.batch, "prompt_len": args.prompt_len, "prefill_len": args.prefill_len,
                 "dtype": "bf16", "data": "synthetic: random bf16 weights, seeded uniform-random token ids"}
         beside = [("design", cfg)]
-        if args.design == "mesolix":
+        if args.design in ("mesolix", "rafusun"):
             beside.append(("nutavik_of_equal_size", nutavik_like(cfg)))
         if args.design == "bekedra":
             beside.append(("mesolix_of_equal_size", mesolix_like(cfg)))
@@ -588,9 +617,9 @@ def design_compare(args) -> int:
 
 def main() -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=("suranex", "nutavik", "mesolix", "bekedra"), default=None,
+    ap.add_argument("--design", choices=("suranex", "nutavik", "mesolix", "bekedra", "rafusun"), default=None,
                     help="measure instead another design's prefill and decode at a few layer sizes, beside the Llama configuration of equal size, with the time and the bound of every kind of kernel")
-    ap.add_argument("--design-shape", default=None, help="with --design: one of its shapes only (suranex-2k, suranex-4k, nutavik-2k, nutavik-4k, mesolix-2k, mesolix-4k, bekedra-2k, bekedra-4k)")
+    ap.add_argument("--design-shape", default=None, help="with --design: one of its shapes only (suranex-2k, suranex-4k, nutavik-2k, nutavik-4k, mesolix-2k, mesolix-4k, bekedra-2k, bekedra-4k, rafusun-2k, rafusun-4k)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=32)
     ap.add_argument("--warmup", type=int, default=4)

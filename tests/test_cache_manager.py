@@ -121,3 +121,30 @@ def test_window_keeps_the_pages_of_kept_first_tokens():
     m.release(7)
     assert m.free_pages(0) == 16 and m.free_pages(1) == 16
     m.audit()
+
+
+def test_chunked_window_gives_back_whole_chunks():
+    """A chunk of 40 positions, pages of 16: while a chunk is being filled all of its pages stay, also those that a window
+    of 40 sliding tokens would keep longer or less; once the next chunk begins, every page that lies wholly below it goes
+    back, and one that holds the border stays."""
+    m = PageManager(16, [GroupShape(16, window=40, chunked=True), GroupShape(16, window=40)], num_slots=1)
+    m.admit(3)
+    assert m.reserve(3, 200)
+    held = lambda g: [p >= 0 for p in m.block_table(3, g).tolist()]
+    m.advance(3, 39)
+    assert held(0) == held(1) == [True] * 13
+    m.advance(3, 40)  # the next token, at position 40, begins a chunk: pages 0 and 1 (0 .. 31) are dead, page 2 holds the border
+    assert held(0) == [False] * 2 + [True] * 11 and held(1) == [True] * 13
+    m.advance(3, 79)
+    assert held(0) == [False] * 2 + [True] * 11 and held(1) == [False] * 2 + [True] * 11
+    m.advance(3, 80)  # a border of chunks that is a border of pages
+    assert held(0) == [False] * 5 + [True] * 8 and held(1) == [False] * 2 + [True] * 11
+    m.advance(3, 81)
+    assert held(0) == [False] * 5 + [True] * 8
+    m.advance(3, 199)
+    assert held(0) == [False] * 10 + [True] * 3
+    assert m.free_pages(0) == 16 - 3
+    m.audit()
+    m.release(3)
+    assert m.free_pages(0) == 16
+    m.audit()

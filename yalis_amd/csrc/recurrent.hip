@@ -51,6 +51,83 @@ __global__ void causal_conv_kernel(const T* __restrict__ x, int x_stride, const 
   }
 }
 
+// The same in pieces of 16 bytes: a thread takes E neighbouring channels (8 of bfloat16, 4 of float32) of up to four
+// consecutive tokens, its channels' weights read once (TAPS 4: kept in registers; 0: any number, read where they are used).
+template <typename T>
+__device__ __forceinline__ void conv_load(const T* p, float* v);
+template <>
+__device__ __forceinline__ void conv_load<float>(const float* p, float* v) {
+  const float4 a = *reinterpret_cast<const float4*>(p);
+  v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w;
+}
+template <>
+__device__ __forceinline__ void conv_load<bf16_t>(const bf16_t* p, float* v) {
+  const uint4 a = *reinterpret_cast<const uint4*>(p);
+  v[0] = __uint_as_float(a.x << 16); v[1] = __uint_as_float(a.x & 0xffff0000u);
+  v[2] = __uint_as_float(a.y << 16); v[3] = __uint_as_float(a.y & 0xffff0000u);
+  v[4] = __uint_as_float(a.z << 16); v[5] = __uint_as_float(a.z & 0xffff0000u);
+  v[6] = __uint_as_float(a.w << 16); v[7] = __uint_as_float(a.w & 0xffff0000u);
+}
+__device__ __forceinline__ void conv_store(float* p, const float* v) { *reinterpret_cast<float4*>(p) = make_float4(v[0], v[1], v[2], v[3]); }
+__device__ __forceinline__ void conv_store(bf16_t* p, const float* v) {
+  *reinterpret_cast<uint4*>(p) = make_uint4(pack_bf16x2(v[0], v[1]), pack_bf16x2(v[2], v[3]), pack_bf16x2(v[4], v[5]), pack_bf16x2(v[6], v[7]));
+}
+
+constexpr int kConvTokens = 4;
+
+template <typename T, typename TW, int TAPS>
+__global__ __launch_bounds__(256) void causal_conv_vec_kernel(const T* __restrict__ x, int x_stride, const TW* __restrict__ w,
+                                                              const TW* __restrict__ bias, T* state,
+                                                              const int32_t* __restrict__ token_seq, const int32_t* __restrict__ seq_qstart,
+                                                              const int32_t* __restrict__ state_slots, T* __restrict__ out, int channels,
+                                                              int taps_arg, int act, int push, int n_tokens, int tokens_each) {
+  constexpr int E = 16 / sizeof(T);
+  const int taps = TAPS > 0 ? TAPS : taps_arg;
+  const int per_row = channels / E;
+  const int piece = blockIdx.x * blockDim.x + threadIdx.x;
+  const int n_begin = blockIdx.y * tokens_each;
+  if (piece >= per_row) return;
+  const int c = piece * E;
+  float wr[TAPS > 0 ? TAPS : 1][E], b[E];
+#pragma unroll
+  for (int e = 0; e < E; ++e) {
+    b[e] = bias != nullptr ? to_f32<TW>(bias[c + e]) : 0.f;
+    if (TAPS > 0) {
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) wr[j][e] = to_f32<TW>(w[static_cast<size_t>(c + e) * TAPS + j]);
+    }
+  }
+  const int n_end = min(n_begin + tokens_each, n_tokens);
+  for (int n = n_begin; n < n_end; ++n) {
+    const int seq = token_seq[n];
+    const int t = n - seq_qstart[seq];  // the token's place in its span
+    T* hist = state + static_cast<size_t>(state_slots[seq]) * (taps - 1) * channels + c;
+    float acc[E];
+#pragma unroll
+    for (int e = 0; e < E; ++e) acc[e] = b[e];
+#pragma unroll
+    for (int j = 0; j < taps; ++j) {
+      const int back = taps - 1 - j;
+      float v[E];
+      // before the span: the state's row (taps - 1) + (t - back), counted from its oldest
+      conv_load<T>(t >= back ? x + static_cast<size_t>(n - back) * x_stride + c : hist + static_cast<size_t>(taps - 1 + t - back) * channels, v);
+#pragma unroll
+      for (int e = 0; e < E; ++e) acc[e] = fmaf(TAPS > 0 ? wr[TAPS > 0 ? j : 0][e] : to_f32<TW>(w[static_cast<size_t>(c + e) * taps + j]), v[e], acc[e]);
+    }
+    if (act == 1) {
+#pragma unroll
+      for (int e = 0; e < E; ++e) acc[e] = act_silu(acc[e]);
+    }
+    conv_store(out + static_cast<size_t>(n) * channels + c, acc);
+    if (push) {  // (spans of one token)
+      for (int j = 0; j + 2 < taps; ++j)
+        *reinterpret_cast<uint4*>(hist + static_cast<size_t>(j) * channels) = *reinterpret_cast<const uint4*>(hist + static_cast<size_t>(j + 1) * channels);
+      *reinterpret_cast<uint4*>(hist + static_cast<size_t>(taps - 2) * channels) =
+          *reinterpret_cast<const uint4*>(x + static_cast<size_t>(n) * x_stride + c);
+    }
+  }
+}
+
 // act: 0 none, 1 silu on the convolution's output.  push != 0 (steps whose spans are single tokens only): the state takes
 // in the token's input in the same pass.
 extern "C" int yk_causal_conv(const void* x, int x_stride, int dtype, const void* w, const void* bias, int w_dtype,
@@ -64,7 +141,21 @@ extern "C" int yk_causal_conv(const void* x, int x_stride, int dtype, const void
   if (n_tokens == 0) return 0;
   const size_t total = static_cast<size_t>(n_tokens) * channels;
   const int grid = static_cast<int>(std::min<size_t>((total + 255) / 256, 1 << 20));
+  auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const int piece = dtype == YK_BF16 ? 8 : 4;
+  const bool vec = channels % piece == 0 && x_stride % piece == 0 && al16(x) && al16(state) && al16(out) &&
+                   (n_tokens + kConvTokens - 1) / kConvTokens <= 65535;
+  // (few tokens: one each, in workgroups of a wave)
+  const int threads = n_tokens <= 64 ? 64 : 256, each = n_tokens <= 64 ? 1 : kConvTokens;
+  const dim3 vgrid((channels / piece + threads - 1) / threads, (n_tokens + each - 1) / each);
 #define YK_CASE(D, T, WD, TW)                                                                                   \
+  if (dtype == D && w_dtype == WD && vec) {                                                                      \
+    auto kern = taps == 4 ? causal_conv_vec_kernel<T, TW, 4> : causal_conv_vec_kernel<T, TW, 0>;                 \
+    kern<<<vgrid, threads, 0, stream>>>(static_cast<const T*>(x), x_stride, static_cast<const TW*>(w), static_cast<const TW*>(bias), \
+                                        static_cast<T*>(state), token_seq, seq_qstart, state_slots, static_cast<T*>(out), channels,  \
+                                        taps, act, push, n_tokens, each);                                        \
+    return yk_check_launch("causal_conv");                                                                       \
+  }                                                                                                              \
   if (dtype == D && w_dtype == WD) {                                                                             \
     causal_conv_kernel<T, TW><<<grid, 256, 0, stream>>>(static_cast<const T*>(x), x_stride, static_cast<const TW*>(w), \
                                                         static_cast<const TW*>(bias), static_cast<T*>(state),           \

@@ -117,6 +117,21 @@ def bekedra_shape(width: int, vocab: int, heads: int, kv_heads: int, dim: int, e
     return cfg
 
 
+def rafusun_shape(width: int, vocab: int, heads: int, kv_heads: int, dim: int, chunk: int, delta_heads: int, delta_kv_heads: int,
+                  delta_dim: int, mixing_heads: int, mixing_dim: int, ff: int, buckets: int,
+                  pattern=("channel_delta", "parallel", "channel_delta"), repeats: int = 2) -> dict:
+    """A Rafusun config.json of the given layer sizes: the mixers of ``pattern`` repeated ``repeats`` times, every layer with a
+    dense feed-forward."""
+    delta = {"heads": delta_heads, "kv_heads": delta_kv_heads, "dim": delta_dim, "vdim": delta_dim, "conv": 4}
+    left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** 0.5 / 8.0, "softcap": 50.0, "mask": {"size": chunk},
+            "rot": {"base": 500000.0, "dims": dim // 2}}
+    both = {"left": left, "right": {"heads": mixing_heads, "dim": mixing_dim}}
+    layers = [{"type": kind, "mixer": dict(delta if kind == "channel_delta" else both), "mlp": {"kind": "dense", "ff": ff}}
+              for kind in pattern * repeats]
+    return {"architecture": "Rafusun", "vocab": vocab, "width": width, "postln_alpha": 2.0, "norm": {"eps": 1e-6},
+            "embedding": {"scale": float(width) ** 0.5, "bigram": {"buckets": buckets, "mul_prev": 1009, "mul_cur": 31}}, "layers": layers}
+
+
 def layer_runs(design: dict) -> int:
     """How many layers a token passes through (a looped stretch counts every pass)."""
     loop = design.get("loop")
@@ -130,6 +145,12 @@ def llama_like(design: dict) -> dict:
     (its top experts and the shared one).  For Nutavik: the same width, layer count, vocabulary and
     attention heads (keys as wide as its unrotated and rotated parts together, a quarter as many key
     heads), a gated feed-forward with as many weights as its dense one (two thirds as wide)."""
+    if design.get("architecture") == "Rafusun":
+        # the same width, layer count, vocabulary, attention heads and feed-forward
+        att = next(layer["mixer"]["left"] for layer in design["layers"] if layer["type"] == "parallel")
+        ff = next(layer["mlp"]["ff"] for layer in design["layers"] if layer["mlp"] is not None)
+        return dict(LLAMA3_8B, hidden_size=design["width"], num_hidden_layers=len(design["layers"]), num_attention_heads=att["heads"],
+                    num_key_value_heads=att["kv_heads"], head_dim=att["dim"], intermediate_size=ff, vocab_size=design["vocab"])
     if design.get("architecture") == "Bekedra":
         # the same width, vocabulary and heads, as many layers as a token passes through, a feed-forward with as many
         # weights as what a token uses of the mixture (three matrices against an expert's two)
@@ -166,10 +187,21 @@ def llama_like(design: dict) -> dict:
 
 
 def nutavik_like(design: dict) -> dict:
-    """The Nutavik configuration of a Mesolix one's size: the same width, vocabulary and layer count (in threes), a
+    """The Nutavik configuration of a Rafusun or Mesolix one's size.  For Rafusun: the same width, vocabulary, layer count (in
+    threes) and attention heads, the delta rule with the same heads, gated linear attention with the time mixing's heads, a
+    dense feed-forward with as many weights as the gated one (half as wide again).  For Mesolix: the same width, vocabulary and layer count (in threes), a
     latent attention of the same heads and ranks with a rotated part of 64 (or a quarter of the latent) on top, the
     two recurrences with as many heads and as wide keys and values as the state-space layer's state and channels,
     a dense feed-forward as wide as Mesolix's dense one."""
+    if design.get("architecture") == "Rafusun":
+        both = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "parallel")
+        delta = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "channel_delta")
+        ff = next(layer["mlp"]["ff"] for layer in design["layers"] if layer["mlp"] is not None)
+        width, left, right = design["width"], both["left"], both["right"]
+        big = width >= 1024
+        return nutavik_shape(width, design["vocab"], left["heads"], left["dim"], 64 if big else 8, 512 if big else 24, 768 * width // 2048 if big else 32,
+                             delta["heads"], delta["kv_heads"], right["heads"], right["dim"], right["dim"], 3 * ff // 2,
+                             repeats=max(1, len(design["layers"]) // 3))
     lat = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "latent_attention")
     ssd = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "mamba2")
     ff = next(layer["mlp"]["ff"] for layer in design["layers"] if layer["mlp"] is not None and layer["mlp"]["kind"] == "dense")
@@ -207,6 +239,10 @@ BEKEDRA_2K = bekedra_shape(2048, 32768, 16, 4, 128, 16, 2, 1024)
 BEKEDRA_4K = bekedra_shape(4096, 65536, 32, 8, 128, 32, 4, 1024, pattern=("attention_2", "attention"), loop=(1, 2, 2))
 BEKEDRA_TINY = bekedra_shape(64, 256, 4, 2, 16, 4, 2, 32, pattern=("attention_2", "attention", "attention_2"), loop=(0, 2, 2), original=32)
 
+RAFUSUN_2K = rafusun_shape(2048, 32768, 16, 4, 128, 2048, 16, 8, 128, 32, 64, 5632, 65521)
+RAFUSUN_4K = rafusun_shape(4096, 65536, 32, 8, 128, 2048, 32, 16, 128, 64, 64, 11264, 131071, repeats=1)
+RAFUSUN_TINY = rafusun_shape(64, 256, 4, 2, 16, 24, 4, 2, 16, 3, 16, 96, 101, repeats=1)
+
 # name -> (what to call it, config.json dictionary)
 SHAPES: Dict[str, Tuple[str, dict]] = {
     "8b": ("Llama-3-8B", LLAMA3_8B),
@@ -227,6 +263,9 @@ SHAPES: Dict[str, Tuple[str, dict]] = {
     "bekedra-2k": ("Bekedra, width 2,048", BEKEDRA_2K),
     "bekedra-4k": ("Bekedra, width 4,096", BEKEDRA_4K),
     "bekedra-tiny": ("tiny Bekedra", BEKEDRA_TINY),
+    "rafusun-2k": ("Rafusun, width 2,048", RAFUSUN_2K),
+    "rafusun-4k": ("Rafusun, width 4,096", RAFUSUN_4K),
+    "rafusun-tiny": ("tiny Rafusun", RAFUSUN_TINY),
 }
 
 
