@@ -475,6 +475,11 @@ def _op_costs(ops, hb):
     def token_shift_mix(a, kw, out):
         return 0.0, float(nbytes(a[0], a[1], out))
 
+    def embed(a, kw, out):
+        n, width = a[0].numel(), a[1].shape[1]
+        rows = 1 if kw.get("position_table") is None else 2
+        return 0.0, float(n * width * (rows * a[1].element_size() + 4))
+
     def embed_pairs(a, kw, out):
         n, width = a[0].numel(), a[1].shape[1]
         return 0.0, float(n * width * (2 * a[1].element_size() + 4 + 2))
@@ -484,7 +489,7 @@ def _op_costs(ops, hb):
 
     return {"linear": linear, "gate_up_act": linear, "moe_experts": moe, "attention_masked": attention_masked, "attention": attention,
             "rglru": rglru, "norm_add": moved, "add_rmsnorm": moved, "gather_add_rmsnorm": moved, "qkv_prepare": moved,
-            "rope_append": moved, "causal_conv": moved, "gated_act": moved, "round_rows": moved, "embed": moved,
+            "rope_append": moved, "causal_conv": moved, "gated_act": moved, "round_rows": moved, "embed": embed,
             "sandwich_norm": moved, "activation": moved, "latent_prepare": moved, "head_linear": head_linear,
             "latent_attention": latent_attention, "linear_state_scan": state_scan, "gated_head_norm": moved, "conv_state_push": moved, "moe_router_topk": moved,
             "moe_combine": moved, "attention_finish": moved, "qk_row_scales": moved,

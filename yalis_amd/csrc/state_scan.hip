@@ -99,9 +99,10 @@ __device__ __forceinline__ void scan_load8<bf16_t>(const bf16_t* p, float* out) 
   out[6] = __uint_as_float(w.w << 16); out[7] = __uint_as_float(w.w & 0xffff0000u);
 }
 
+// The general form: any sizes and alignments, every kind of decay, write and read-out chosen as it runs.
 // LDS per staged token: k and q padded to TPC * 16 floats each (rows past dim are zeros, so nobody
 // asks whether a row exists), the per-channel decays likewise where there are any
-template <typename T, int TPC, int kScanRows, bool VEC>
+template <typename T, int TPC, int kScanRows>
 __global__ __launch_bounds__(256) void linear_state_scan_kernel(
     const T* __restrict__ qkv, int qkv_stride, int n_heads, int n_kv, int dim, int vdim, float* __restrict__ state,
     const int32_t* __restrict__ seq_qstart, const int32_t* __restrict__ seq_qlen, const int32_t* __restrict__ state_slots,
@@ -147,101 +148,6 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
   for (int t0 = 0; t0 < ql; t0 += chunk) {
     const int nt = min(chunk, ql - t0);
     __syncthreads();  // the chunk before has been read
-    if constexpr (VEC) {
-      // Everything the chunk needs is asked for at once, 16 bytes a load, before anything is used: q and
-      // k (eight elements a piece), the decays' logits and biases (four), v, the scalars.  One round
-      // trip to memory a chunk; one after the other the loads cost a round trip each, which was most
-      // of the kernel's time.
-      constexpr int P8 = DP / 8 > 0 ? DP / 8 : 1;  // pieces of a padded row (DP >= 16: at least two)
-      const float q_mul = unit_eps >= 0.f ? 1.f : q_scale;
-      const int n_qk = 2 * nt * (DP / 8);
-      float qk[8][8];
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int v = threadIdx.x + j * 256;
-        const int item = v / P8, c = 8 * (v % P8), t = item >> 1, is_k = item & 1;
-        if (v < n_qk && c < dim)
-          scan_load8<T>(qkv + static_cast<size_t>(q0 + t0 + t) * qkv_stride + (is_k ? k_col : q_col) + kvh * dim + c, qk[j]);
-        else {
-#pragma unroll
-          for (int e = 0; e < 8; ++e) qk[j][e] = 0.f;
-        }
-      }
-      constexpr int P4 = DP / 4;
-      const int n_dec = per_channel ? nt * P4 : 0;
-      float4 dz[8], db[8];
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int v = threadIdx.x + j * 256;
-        const int t = v / P4, c = 4 * (v % P4);
-        dz[j] = db[j] = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (v < n_dec && c < dim) {
-          dz[j] = *reinterpret_cast<const float4*>(decay + static_cast<size_t>(q0 + t0 + t) * decay_stride + decay_col + h * dim + c);
-          db[j] = *reinterpret_cast<const float4*>(dec_bias + h * dim + c);
-        }
-      }
-      const int n_v = nt * cols_per_block;
-      float vv[8];
-      for (int i0 = 0; i0 < n_v; i0 += 8 * 256) {  // (one pass unless a column is a single lane's)
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int i = i0 + threadIdx.x + j * 256;
-          const int t = i / cols_per_block, c = col0 + i % cols_per_block;
-          vv[j] = i < n_v && c < vdim ? to_f32<T>(qkv[static_cast<size_t>(q0 + t0 + t) * qkv_stride + v_col + h * vdim + c]) : 0.f;
-        }
-        if (i0 + 8 * 256 < n_v) {
-#pragma unroll
-          for (int j = 0; j < 8; ++j) {
-            const int i = i0 + threadIdx.x + j * 256;
-            if (i < n_v) vs[i] = vv[j];
-          }
-        }
-      }
-      float s_dec = 0.f, s_beta = 0.f;
-      if (threadIdx.x < nt) {
-        const size_t n = static_cast<size_t>(q0 + t0 + threadIdx.x);
-        if (decay_mode == 0) s_dec = decay[n * decay_stride + decay_col + h];
-        if (delta) s_beta = beta_rows != nullptr ? to_f32<T>(beta_rows[n * beta_stride + beta_col + h]) : beta[n * beta_stride + beta_col + h];
-      }
-      // ---- everything is on its way; now the stores
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int v = threadIdx.x + j * 256;
-        if (v < n_qk) {
-          const int item = v / P8, c = 8 * (v % P8), t = item >> 1, is_k = item & 1;
-          const float mul = is_k ? 1.f : q_mul;
-          float* dst = (is_k ? ks : qs) + t * DS + c;
-          *reinterpret_cast<float4*>(dst) = make_float4(qk[j][0] * mul, qk[j][1] * mul, qk[j][2] * mul, qk[j][3] * mul);
-          *reinterpret_cast<float4*>(dst + 4) = make_float4(qk[j][4] * mul, qk[j][5] * mul, qk[j][6] * mul, qk[j][7] * mul);
-        }
-      }
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const int v = threadIdx.x + j * 256;
-        if (v < n_dec) {
-          const int c = 4 * (v % P4);
-          // (channels past dim decay to nothing: their rows of S are zeros anyway)
-          float4 a = make_float4(0.f, 0.f, 0.f, 0.f);
-          if (c < dim)
-            a = make_float4(channel_decay(dz[j].x + db[j].x, decay_mode, tau, dec_rate), channel_decay(dz[j].y + db[j].y, decay_mode, tau, dec_rate),
-                            channel_decay(dz[j].z + db[j].z, decay_mode, tau, dec_rate), channel_decay(dz[j].w + db[j].w, decay_mode, tau, dec_rate));
-          *reinterpret_cast<float4*>(as + (v / P4) * DS + c) = a;
-        }
-      }
-      {
-        const int i0 = (n_v - 1) / (8 * 256) * (8 * 256);  // the last pass's values are still in registers
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int i = i0 + threadIdx.x + j * 256;
-          if (i < n_v) vs[i] = vv[j];
-        }
-      }
-      if (threadIdx.x < nt) {
-        const float step = decay_mode == 0 ? scan_softplus(s_dec + decay_p1[h]) : 1.f;
-        if (decay_mode == 0) as[threadIdx.x] = expf(-expf(decay_p0[h]) * step);
-        bs[threadIdx.x] = delta ? 1.f / (1.f + expf(-s_beta)) : (write_mode == 2 ? step : 1.f);
-      }
-    } else {
     // q and k of the chunk's tokens to LDS, every load of a thread asked for before the first is used
     // (one after the other they cost a round trip to memory each)
     {
@@ -268,23 +174,13 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       }
     }
     if (per_channel) {
-      const int total = nt * DP;
-      for (int i0 = threadIdx.x; i0 < total; i0 += 8 * blockDim.x) {
-        float z[8];
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int i = i0 + j * blockDim.x;
-          const int t = i / DP, c = i % DP;
-          z[j] = i < total && c < dim
-                     ? decay[static_cast<size_t>(q0 + t0 + t) * decay_stride + decay_col + h * dim + c] + dec_bias[h * dim + c]
-                     : 0.f;
-        }
-#pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int i = i0 + j * blockDim.x;
-          // (channels past dim decay to nothing: their rows of S are zeros anyway)
-          if (i < total) as[(i / DP) * DS + i % DP] = i % DP < dim ? channel_decay(z[j], decay_mode, tau, dec_rate) : 0.f;
-        }
+#pragma unroll 1
+      for (int i = threadIdx.x; i < nt * DP; i += blockDim.x) {
+        const int t = i / DP, c = i % DP;
+        // (channels past dim decay to nothing: their rows of S are zeros anyway)
+        as[t * DS + c] = c < dim ? channel_decay(decay[static_cast<size_t>(q0 + t0 + t) * decay_stride + decay_col + h * dim + c] + dec_bias[h * dim + c],
+                                                 decay_mode, tau, dec_rate)
+                                 : 0.f;
       }
     }
     for (int i = threadIdx.x; i < nt * cols_per_block; i += blockDim.x) {
@@ -298,7 +194,6 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       float b = write_mode == 2 ? step : 1.f;
       if (delta) b = 1.f / (1.f + expf(-(beta_rows != nullptr ? to_f32<T>(beta_rows[n * beta_stride + beta_col + h]) : beta[n * beta_stride + beta_col + h])));
       bs[t] = b;
-    }
     }
     __syncthreads();
     // eight lanes a token: unit norms (the rows scaled where they lie) and k . q, which the read-out needs;
@@ -411,12 +306,296 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
   }
 }
 
+// The form for aligned rows (what the engine's own tensors are).  Its loop over tokens is all that most of its time goes to, a
+// wave alone on its SIMD with nothing to hide behind, so what a token costs in instructions is what counts: the kind of decay,
+// write and read-out are template parameters (KIND, a sum of the flags below) and leave no branch in it; the next token's
+// vectors are read from LDS into a second register set by turns, without moves; its scalars come as one 16-byte read.  The
+// chunk after this one is on its way from memory while this one is walked.  Decays per channel are made by a kernel of
+// their own first (GIVEN: `decay` holds them), or, for steps of few tokens, here while they are staged.
+constexpr int kScanChannel = 1;    // a decay per key channel (else one for the head)
+constexpr int kScanDelta = 2;      // the delta rule (else plain writes, or writes by the step)
+constexpr int kScanReadFirst = 4;  // the read-out sees the memory as it was, plus the bonus
+
+template <typename T>
+struct Raw8;  // eight elements as they lie in memory
+template <>
+struct Raw8<bf16_t> {
+  uint4 w;
+  __device__ __forceinline__ void load(const bf16_t* p) { w = *reinterpret_cast<const uint4*>(p); }
+  __device__ __forceinline__ void clear() { w = make_uint4(0u, 0u, 0u, 0u); }
+  __device__ __forceinline__ void store(float* dst, float mul) const {
+    *reinterpret_cast<float4*>(dst) = make_float4(__uint_as_float(w.x << 16) * mul, __uint_as_float(w.x & 0xffff0000u) * mul,
+                                                  __uint_as_float(w.y << 16) * mul, __uint_as_float(w.y & 0xffff0000u) * mul);
+    *reinterpret_cast<float4*>(dst + 4) = make_float4(__uint_as_float(w.z << 16) * mul, __uint_as_float(w.z & 0xffff0000u) * mul,
+                                                      __uint_as_float(w.w << 16) * mul, __uint_as_float(w.w & 0xffff0000u) * mul);
+  }
+};
+template <>
+struct Raw8<float> {
+  float4 a, b;
+  __device__ __forceinline__ void load(const float* p) { a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4); }
+  __device__ __forceinline__ void clear() { a = b = make_float4(0.f, 0.f, 0.f, 0.f); }
+  __device__ __forceinline__ void store(float* dst, float mul) const {
+    *reinterpret_cast<float4*>(dst) = make_float4(a.x * mul, a.y * mul, a.z * mul, a.w * mul);
+    *reinterpret_cast<float4*>(dst + 4) = make_float4(b.x * mul, b.y * mul, b.z * mul, b.w * mul);
+  }
+};
+
+struct ScanArgs {
+  const int32_t *seq_qstart, *seq_qlen, *state_slots;
+  int qkv_stride, n_heads, n_kv, dim, vdim, q_col, k_col, v_col;
+  float q_scale, unit_eps;
+  int decay_mode, given;  // given: `decay` holds the channels' decays themselves
+  const float* decay;
+  int decay_stride, decay_col;
+  const float *decay_p0, *decay_p1;
+  float tau;
+  const float* beta;
+  int beta_stride, beta_col, by_step;
+  const float *skip, *bonus;
+  int chunk;
+};
+
+template <typename T, int TPC, int ROWS, int KIND>
+__global__ __launch_bounds__(256) void linear_state_scan_fast_kernel(const T* __restrict__ qkv, float* __restrict__ state, float* __restrict__ out,
+                                                                     const T* __restrict__ beta_rows, ScanArgs g) {
+  constexpr bool CH = KIND & kScanChannel, DELTA = KIND & kScanDelta, FIRST = KIND & kScanReadFirst;
+  constexpr int DP = TPC * ROWS;  // padded key channels
+  constexpr int DS = DP + 4;      // a staged row's stride: rows of different tokens then start in different banks
+  constexpr int COLS = 256 / TPC;
+  constexpr int P8 = DP / 8, P4 = DP / 4;
+  constexpr int NQ = DP / 32 < 1 ? 1 : (DP / 32 > 8 ? 8 : DP / 32);  // 16-byte pieces of q and k a thread stages (and of decays)
+  constexpr int NV = kScanTokens / TPC < 1 ? 1 : kScanTokens / TPC;  // values a thread stages
+  extern __shared__ float lds[];
+  const int chunk = g.chunk, rows_staged = chunk + 2;  // (the walk reads up to two tokens ahead; what it finds there is not used)
+  float* ks = lds;                                  // [chunk + 2][DS]
+  float* qs = ks + rows_staged * DS;                // [chunk + 2][DS]
+  float* as = qs + rows_staged * DS;                // [chunk + 2][DS] where decays are per channel
+  float* sc = as + (CH ? rows_staged * DS : 0);     // [chunk + 2][4]: the head's decay, the write's strength, k . q (with the bonus)
+  float* vs = sc + rows_staged * 4;                 // [chunk + 2][COLS]
+  float* us = vs + rows_staged * COLS;              // [DP]: the head's bonus
+
+  const int seq = blockIdx.x, h = blockIdx.y, kvh = h / (g.n_heads / g.n_kv);
+  const int col0 = blockIdx.z * COLS;
+  const int sub = threadIdx.x % TPC, col_local = threadIdx.x / TPC, col = col0 + col_local;
+  const int dim = g.dim, vdim = g.vdim;
+  const bool has_col = col < vdim;
+  const int q0 = g.seq_qstart[seq], ql = g.seq_qlen[seq];
+  float* S_head = state + (static_cast<size_t>(g.state_slots[seq]) * g.n_heads + h) * dim * vdim;
+  const float skip_h = g.skip != nullptr ? g.skip[h] : 0.f;
+  if (FIRST)
+    for (int i = threadIdx.x; i < DP; i += 256) us[i] = i < dim ? g.bonus[h * dim + i] : 0.f;
+  const float* dec_bias = g.decay_mode == 2 ? g.decay_p1 : g.decay_p0;
+  const float dec_rate = CH && g.decay_mode == 2 && !g.given ? expf(g.decay_p0[h]) : 1.f;
+
+  float S[ROWS];
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    const int i = sub * ROWS + r;
+    S[r] = has_col && i < dim ? S_head[static_cast<size_t>(i) * vdim + col] : 0.f;
+  }
+
+  // a chunk's operands, on their way in registers
+  Raw8<T> qk[NQ];
+  float4 dz[CH ? NQ : 1];
+  T vv[NV];
+  float s_dec = 0.f, s_beta = 0.f;
+  auto ask = [&](int t0) {
+    const int nt = min(chunk, ql - t0);
+    const size_t n0 = static_cast<size_t>(q0 + t0);
+#pragma unroll
+    for (int j = 0; j < NQ; ++j) {
+      const int v = threadIdx.x + j * 256;
+      const int item = v / P8, c = 8 * (v % P8), t = item >> 1, is_k = item & 1;
+      if (v < 2 * nt * P8 && c < dim)
+        qk[j].load(qkv + (n0 + t) * g.qkv_stride + (is_k ? g.k_col : g.q_col) + kvh * dim + c);
+      else
+        qk[j].clear();
+    }
+    if (CH && g.given) {
+#pragma unroll
+      for (int j = 0; j < NQ; ++j) {
+        const int v = threadIdx.x + j * 256, t = v / P4, c = 4 * (v % P4);
+        // (channels past dim decay to nothing: their rows of S are zeros anyway)
+        dz[CH ? j : 0] = v < nt * P4 && c < dim ? *reinterpret_cast<const float4*>(g.decay + (n0 + t) * g.decay_stride + g.decay_col + h * dim + c)
+                                                : make_float4(0.f, 0.f, 0.f, 0.f);
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = threadIdx.x + j * 256, t = i / COLS, c = col0 + i % COLS;
+      vv[j] = i < nt * COLS && c < vdim ? qkv[(n0 + t) * g.qkv_stride + g.v_col + h * vdim + c] : T(0);
+    }
+    if (threadIdx.x < nt) {
+      const size_t n = n0 + threadIdx.x;
+      if (!CH) s_dec = g.decay[n * g.decay_stride + g.decay_col + h];
+      if (DELTA) s_beta = beta_rows != nullptr ? to_f32<T>(beta_rows[n * g.beta_stride + g.beta_col + h]) : g.beta[n * g.beta_stride + g.beta_col + h];
+    }
+  };
+
+  ask(0);
+  for (int t0 = 0; t0 < ql; t0 += chunk) {
+    const int nt = min(chunk, ql - t0);
+    __syncthreads();  // the chunk before has been read
+    {
+      const float q_mul = g.unit_eps >= 0.f ? 1.f : g.q_scale;
+#pragma unroll
+      for (int j = 0; j < NQ; ++j) {
+        const int v = threadIdx.x + j * 256;
+        const int item = v / P8, c = 8 * (v % P8), t = item >> 1, is_k = item & 1;
+        if (v < 2 * nt * P8) qk[j].store((is_k ? ks : qs) + t * DS + c, is_k ? 1.f : q_mul);
+      }
+      if (CH && g.given) {
+#pragma unroll
+        for (int j = 0; j < NQ; ++j) {
+          const int v = threadIdx.x + j * 256;
+          if (v < nt * P4) *reinterpret_cast<float4*>(as + (v / P4) * DS + 4 * (v % P4)) = dz[CH ? j : 0];
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int i = threadIdx.x + j * 256;
+        if (i < nt * COLS) vs[i] = to_f32<T>(vv[j]);
+      }
+      if (threadIdx.x < nt) {
+        const float step = CH ? 1.f : scan_softplus(s_dec + g.decay_p1[h]);
+        if (!CH) sc[4 * threadIdx.x] = expf(-expf(g.decay_p0[h]) * step);
+        sc[4 * threadIdx.x + 1] = DELTA ? 1.f / (1.f + expf(-s_beta)) : (g.by_step ? step : 1.f);
+      }
+      if (CH && !g.given) {
+#pragma unroll 1
+        for (int i = threadIdx.x; i < nt * DP; i += 256) {
+          const int t = i / DP, c = i % DP;
+          as[t * DS + c] = c < dim ? channel_decay(g.decay[static_cast<size_t>(q0 + t0 + t) * g.decay_stride + g.decay_col + h * dim + c] + dec_bias[h * dim + c],
+                                                   g.decay_mode, g.tau, dec_rate)
+                                   : 0.f;
+        }
+      }
+    }
+    __syncthreads();
+    // eight lanes a token: unit norms (the rows scaled where they lie) and k . q, which the read-out needs
+    for (int t = threadIdx.x / 8; t < nt; t += 32) {
+      const int s8 = threadIdx.x % 8;
+      float* qrow = qs + t * DS;
+      float* krow = ks + t * DS;
+      float ssq = 0.f, ssk = 0.f, dot = 0.f;
+      for (int c = 4 * s8; c < DP; c += 32) {
+        const float4 a = *reinterpret_cast<const float4*>(qrow + c), b = *reinterpret_cast<const float4*>(krow + c);
+        ssq = fmaf(a.x, a.x, fmaf(a.y, a.y, fmaf(a.z, a.z, fmaf(a.w, a.w, ssq))));
+        ssk = fmaf(b.x, b.x, fmaf(b.y, b.y, fmaf(b.z, b.z, fmaf(b.w, b.w, ssk))));
+        if (FIRST) {
+          const float4 u = *reinterpret_cast<const float4*>(us + c);
+          dot = fmaf(a.x * u.x, b.x, fmaf(a.y * u.y, b.y, fmaf(a.z * u.z, b.z, fmaf(a.w * u.w, b.w, dot))));
+        } else {
+          dot = fmaf(a.x, b.x, fmaf(a.y, b.y, fmaf(a.z, b.z, fmaf(a.w, b.w, dot))));
+        }
+      }
+      dot = column_sum<8>(dot);
+      if (g.unit_eps >= 0.f) {
+        const float mq = g.q_scale / sqrtf(column_sum<8>(ssq) + g.unit_eps), mk = 1.f / sqrtf(column_sum<8>(ssk) + g.unit_eps);
+        for (int c = 4 * s8; c < DP; c += 32) {
+          float4 a = *reinterpret_cast<const float4*>(qrow + c), b = *reinterpret_cast<const float4*>(krow + c);
+          a.x *= mq; a.y *= mq; a.z *= mq; a.w *= mq;
+          b.x *= mk; b.y *= mk; b.z *= mk; b.w *= mk;
+          *reinterpret_cast<float4*>(qrow + c) = a;
+          *reinterpret_cast<float4*>(krow + c) = b;
+        }
+        dot *= mq * mk;
+      }
+      if (s8 == 0) sc[4 * t + 2] = dot;
+    }
+    __syncthreads();
+    if (t0 + chunk < ql) ask(t0 + chunk);
+    // the walk: two register sets by turns
+    struct Token {
+      float4 k[ROWS / 4], q[ROWS / 4], a[CH ? ROWS / 4 : 1], s;
+      float v;
+    } one, two;
+    const float *kp = ks + sub * ROWS, *qp = qs + sub * ROWS, *ap = as + sub * ROWS, *vp = vs + col_local, *sp = sc;
+    auto fetch = [&](Token& x, int ahead) {
+#pragma unroll
+      for (int r = 0; r < ROWS / 4; ++r) {
+        x.k[r] = *reinterpret_cast<const float4*>(kp + ahead * DS + 4 * r);
+        x.q[r] = *reinterpret_cast<const float4*>(qp + ahead * DS + 4 * r);
+        if (CH) x.a[r] = *reinterpret_cast<const float4*>(ap + ahead * DS + 4 * r);
+      }
+      x.s = *reinterpret_cast<const float4*>(sp + ahead * 4);
+      x.v = vp[ahead * COLS];
+    };
+    float* op = out + (static_cast<size_t>(q0 + t0) * g.n_heads + h) * vdim + col;
+    const size_t o_stride = static_cast<size_t>(g.n_heads) * vdim;
+    const bool stores = has_col && sub == 0;
+    auto walk = [&](const Token& x) {
+      // both sums over S at once: S^T k for the write, S^T q for the read-out, which sees the token's own write through
+      // q . (k u^T) = u (k . q)
+      float pk[4] = {0.f, 0.f, 0.f, 0.f}, pq[4] = {0.f, 0.f, 0.f, 0.f};
+      const float* k = reinterpret_cast<const float*>(x.k);
+      const float* q = reinterpret_cast<const float*>(x.q);
+      const float* a = reinterpret_cast<const float*>(x.a);
+      if (FIRST) {
+#pragma unroll
+        for (int r = 0; r < ROWS; ++r) pq[r % 4] = fmaf(S[r], q[r], pq[r % 4]);
+      }
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) S[r] *= CH ? a[CH ? r : 0] : x.s.x;
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) {
+        if (DELTA) pk[r % 4] = fmaf(S[r], k[r], pk[r % 4]);
+        if (!FIRST) pq[r % 4] = fmaf(S[r], q[r], pq[r % 4]);
+      }
+      float u = x.v;
+      if (DELTA) u = x.s.y * (u - column_sum<TPC>((pk[0] + pk[1]) + (pk[2] + pk[3])));
+      else if (!CH) u *= x.s.y;
+      const float sq = column_sum<TPC>((pq[0] + pq[1]) + (pq[2] + pq[3]));
+#pragma unroll
+      for (int r = 0; r < ROWS; ++r) S[r] = fmaf(k[r], u, S[r]);
+      float so = fmaf(u, x.s.z, sq);
+      if (!CH && !DELTA) so = fmaf(skip_h, x.v, so);
+      if (stores) *op = so;
+      op += o_stride;
+    };
+    fetch(one, 0);
+    int t = 0;
+    for (; t + 1 < nt; t += 2) {
+      fetch(two, 1);
+      walk(one);
+      fetch(one, 2);
+      walk(two);
+      kp += 2 * DS, qp += 2 * DS, ap += 2 * DS, vp += 2 * COLS, sp += 8;
+    }
+    if (t < nt) walk(one);
+  }
+#pragma unroll
+  for (int r = 0; r < ROWS; ++r) {
+    const int i = sub * ROWS + r;
+    if (has_col && i < dim) S_head[static_cast<size_t>(i) * vdim + col] = S[r];
+  }
+}
+
+// decays per key channel, made once for all the columns that will read them: out[n][h * dim + i], four a thread
+__global__ __launch_bounds__(256) void channel_decay_kernel(const float* __restrict__ z, int stride, int col, const float* __restrict__ p0,
+                                                            const float* __restrict__ p1, int mode, float tau, int dim, int channels,
+                                                            float* __restrict__ out, size_t total4) {
+  for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < total4; i += static_cast<size_t>(gridDim.x) * blockDim.x) {
+    const size_t n = i / (channels / 4);
+    const int c = 4 * static_cast<int>(i % (channels / 4));
+    const float4 x = *reinterpret_cast<const float4*>(z + n * stride + col + c);
+    const float4 b = *reinterpret_cast<const float4*>((mode == 2 ? p1 : p0) + c);
+    const float rate = mode == 2 ? expf(p0[c / dim]) : 1.f;  // (a head's channels are a multiple of four)
+    float v[4] = {x.x + b.x, x.y + b.y, x.z + b.z, x.w + b.w};
+#pragma unroll 1
+    for (int e = 0; e < 4; ++e) v[e] = channel_decay(v[e], mode, tau, rate);
+    *reinterpret_cast<float4*>(out + n * channels + c) = make_float4(v[0], v[1], v[2], v[3]);
+  }
+}
+
 // decay_mode 0: one decay per head from decay[n, decay_col + h], p0 = A_log [heads], p1 = dt_bias [heads];
 // decay_mode 1, 2, 3: one per key channel from z = decay[n, decay_col + h * dim + i]: 1, sigmoid(z + p0)^(1 / tau), p0 =
 // bias [heads * dim]; 2, exp(-exp(p0[h]) softplus(z + p1)), p0 = A_log [heads], p1 = dt_bias [heads * dim]; 3,
 // exp(-exp(z + p0)), p0 = bias [heads * dim].
 // beta (float32) or, in its place, beta_rows (of qkv's dtype), both read at [n, beta_col + h].  bonus [heads * dim]
 // float32 or null: the read-out comes before the write, with the token's own write weighed by the bonus (plain writes).
+// decays [n_tokens][heads * dim] float32 or null: room for the decays per channel, made first where tokens are many.
 // write_mode 0: plain writes; 1: the delta rule with beta = sigmoid(beta[n, beta_col + h]); 2: u = dt v with the
 // step dt = softplus(decay[n, decay_col + h] + p1[h]) that the head's decay is made of (decay_mode 0 only).
 // unit_eps < 0: q and k are taken as they are.  q_col, k_col, v_col: where the kv_heads' queries and keys and the
@@ -427,7 +606,7 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
                                     const float* decay, int decay_stride, int decay_col, const float* decay_p0,
                                     const float* decay_p1, float tau, const float* beta, int beta_stride, int beta_col,
                                     float* out, int q_col, int k_col, int v_col, int write_mode, const float* skip,
-                                    const void* beta_rows, const float* bonus, hipStream_t stream) {
+                                    const void* beta_rows, const float* bonus, float* decays, hipStream_t stream) {
   YK_REQUIRE(n_seqs >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0 && dim > 0 && vdim > 0, "linear_state_scan: bad sizes");
   YK_REQUIRE(q_col >= 0 && k_col >= 0 && v_col >= 0 && qkv_stride >= std::max(std::max(q_col, k_col) + n_kv * dim, v_col + n_heads * vdim),
              "linear_state_scan: rows shorter than q, k and v");
@@ -457,12 +636,61 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
   const size_t lds = chunk * per_token + (bonus != nullptr ? (dp + 4) * sizeof(float) : 0);
   YK_REQUIRE(lds <= 128 * 1024, "linear_state_scan: the staged tokens do not fit in LDS");
   auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
-  const bool vec = dim % 8 == 0 && qkv_stride % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 && al16(qkv) && chunk * dp <= 8192 &&
-                   (decay_mode == 0 || (decay_stride % 4 == 0 && decay_col % 4 == 0 && al16(decay) && al16(decay_mode == 2 ? decay_p1 : decay_p0)));
+  const int kind = (decay_mode != 0 ? kScanChannel : 0) + (write_mode == 1 ? kScanDelta : 0) + (bonus != nullptr ? kScanReadFirst : 0);
+  const bool fast = dim % 8 == 0 && qkv_stride % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 && al16(qkv) && chunk * dp <= 8192 && kind != kScanReadFirst &&
+                    (skip == nullptr || kind == 0);
+  if (fast) {
+    // many tokens: their decays per channel first, where the caller gave room for them
+    const bool given = decay_mode != 0 && decays != nullptr && decay_stride % 4 == 0 && decay_col % 4 == 0 && al16(decay) && al16(decays) &&
+                       al16(decay_mode == 2 ? decay_p1 : decay_p0);
+    if (given) {
+      const size_t total4 = static_cast<size_t>(n_tokens) * n_heads * dim / 4;
+      const int dgrid = static_cast<int>(std::min<size_t>((total4 + 255) / 256, 1 << 20));
+      channel_decay_kernel<<<dgrid, 256, 0, stream>>>(decay, decay_stride, decay_col, decay_p0, decay_p1, decay_mode, tau, dim, n_heads * dim, decays, total4);
+      if (yk_check_launch("channel_decay")) return -1;
+    }
+    const ScanArgs g{seq_qstart, seq_qlen, state_slots, qkv_stride, n_heads, n_kv, dim, vdim, q_col, k_col, v_col, q_scale, unit_eps,
+                     decay_mode, given, given ? decays : decay, given ? n_heads * dim : decay_stride, given ? 0 : decay_col, decay_p0, decay_p1, tau,
+                     beta, beta_stride, beta_col, write_mode == 2, skip, bonus, chunk};
+    const size_t fast_lds = sizeof(float) * ((chunk + 2) * ((decay_mode != 0 ? 3 : 2) * (dp + 4) + 4 + cols) + dp);
+    YK_REQUIRE(fast_lds <= 128 * 1024, "linear_state_scan: the staged tokens do not fit in LDS");
+#define YK_FAST(T, TPC, KIND)                                                                                                   \
+  {                                                                                                                             \
+    auto kern = rows == 8 ? linear_state_scan_fast_kernel<T, TPC, 8, KIND> : linear_state_scan_fast_kernel<T, TPC, 16, KIND>;   \
+    if (fast_lds > 64 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, \
+                                                    static_cast<int>(fast_lds)) != hipSuccess)                                  \
+      return yk_fail("linear_state_scan: the staged tokens do not fit in LDS");                                                 \
+    kern<<<grid, threads, fast_lds, stream>>>(static_cast<const T*>(qkv), state, out, static_cast<const T*>(beta_rows), g);     \
+    return yk_check_launch("linear_state_scan");                                                                                \
+  }
+#define YK_FAST_KIND(T, TPC)             \
+  switch (kind) {                        \
+    case 0: YK_FAST(T, TPC, 0)           \
+    case 1: YK_FAST(T, TPC, 1)           \
+    case 2: YK_FAST(T, TPC, 2)           \
+    case 3: YK_FAST(T, TPC, 3)           \
+    default: YK_FAST(T, TPC, 5)          \
+  }
+#define YK_FAST_TPC(T)                   \
+  switch (tpc) {                         \
+    case 1: YK_FAST_KIND(T, 1)           \
+    case 2: YK_FAST_KIND(T, 2)           \
+    case 4: YK_FAST_KIND(T, 4)           \
+    case 8: YK_FAST_KIND(T, 8)           \
+    case 16: YK_FAST_KIND(T, 16)         \
+    case 32: YK_FAST_KIND(T, 32)         \
+    default: YK_FAST_KIND(T, 64)         \
+  }
+    if (dtype == YK_F32) YK_FAST_TPC(float)
+    if (dtype == YK_BF16) YK_FAST_TPC(bf16_t)
+#undef YK_FAST_TPC
+#undef YK_FAST_KIND
+#undef YK_FAST
+    return yk_fail("linear_state_scan: unsupported dtype");
+  }
 #define YK_LAUNCH(T, TPC)                                                                                                       \
   {                                                                                                                             \
-    auto kern = rows == 8 ? (vec ? linear_state_scan_kernel<T, TPC, 8, true> : linear_state_scan_kernel<T, TPC, 8, false>)      \
-                          : (vec ? linear_state_scan_kernel<T, TPC, 16, true> : linear_state_scan_kernel<T, TPC, 16, false>);   \
+    auto kern = rows == 8 ? linear_state_scan_kernel<T, TPC, 8> : linear_state_scan_kernel<T, TPC, 16>;                         \
     if (lds > 64 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, \
                                                static_cast<int>(lds)) != hipSuccess)                                            \
       return yk_fail("linear_state_scan: the staged tokens do not fit in LDS");                                                 \

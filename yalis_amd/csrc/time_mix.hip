@@ -95,8 +95,10 @@ __device__ __forceinline__ float low_rank_act(float v, int act) { return act == 
 
 constexpr int kLowRankTokens = 8;  // tokens a workgroup takes at a time
 
-// a workgroup: up to eight tokens (their rows of y in LDS, padded with zeros to a multiple of eight), 256 columns, a thread
-// a column with its row of w read once for all of them
+// a workgroup: up to eight tokens, their rows of y in LDS (padded with zeros to a multiple of eight).  VEC (a rank that is a
+// multiple of eight): eight lanes a column, each taking pieces of eight of its row of w for all the tokens, so that a column's
+// row is read in one round trip and in consecutive bytes; the sums meet by exchanges and lane t stores token t's.  Otherwise a
+// thread a column.
 template <typename T, typename TW, bool VEC>
 __global__ __launch_bounds__(256) void low_rank_kernel(const T* __restrict__ y, int y_stride, const TW* __restrict__ w, int act,
                                                        float* __restrict__ out, int n_tokens, int cols, int rank) {
@@ -108,27 +110,37 @@ __global__ __launch_bounds__(256) void low_rank_kernel(const T* __restrict__ y, 
     rows[i] = t < live && j < rank ? low_rank_act(to_f32<T>(y[static_cast<size_t>(n0 + t) * y_stride + j]), act) : 0.f;
   }
   __syncthreads();
-  const int c = blockIdx.x * blockDim.x + threadIdx.x;
-  if (c >= cols) return;
-  const TW* wr = w + static_cast<size_t>(c) * rank;
   float acc[kLowRankTokens];
 #pragma unroll
   for (int t = 0; t < kLowRankTokens; ++t) acc[t] = 0.f;
   if (VEC) {
-    for (int j = 0; j < rank; j += 4) {
-      const float4 a = tm_load4<TW>(wr + j);
+    const int sub = threadIdx.x % 8, c = blockIdx.x * (blockDim.x / 8) + threadIdx.x / 8;
+    const TW* wr = w + static_cast<size_t>(min(c, cols - 1)) * rank;  // (a column beyond the last works on it and stores nothing)
+    for (int j = 8 * sub; j < rank; j += 64) {
+      const float4 a = tm_load4<TW>(wr + j), b = tm_load4<TW>(wr + j + 4);
 #pragma unroll
       for (int t = 0; t < kLowRankTokens; ++t) {
-        const float4 b = *reinterpret_cast<const float4*>(rows + t * rp + j);
-        acc[t] = fmaf(a.x, b.x, fmaf(a.y, b.y, fmaf(a.z, b.z, fmaf(a.w, b.w, acc[t]))));
+        const float4 p = *reinterpret_cast<const float4*>(rows + t * rp + j), q = *reinterpret_cast<const float4*>(rows + t * rp + j + 4);
+        acc[t] = fmaf(a.x, p.x, fmaf(a.y, p.y, fmaf(a.z, p.z, fmaf(a.w, p.w, fmaf(b.x, q.x, fmaf(b.y, q.y, fmaf(b.z, q.z, fmaf(b.w, q.w, acc[t]))))))));
       }
     }
-  } else {
-    for (int j = 0; j < rank; ++j) {
-      const float a = to_f32<TW>(wr[j]);
+    float mine = 0.f;
 #pragma unroll
-      for (int t = 0; t < kLowRankTokens; ++t) acc[t] = fmaf(a, rows[t * rp + j], acc[t]);
+    for (int t = 0; t < kLowRankTokens; ++t) {
+#pragma unroll
+      for (int o = 4; o > 0; o >>= 1) acc[t] += __shfl_xor(acc[t], o, 8);
+      if (t == sub) mine = acc[t];
     }
+    if (c < cols && sub < live) out[static_cast<size_t>(n0 + sub) * cols + c] = mine;
+    return;
+  }
+  const int c = blockIdx.x * blockDim.x + threadIdx.x;
+  if (c >= cols) return;
+  const TW* wr = w + static_cast<size_t>(c) * rank;
+  for (int j = 0; j < rank; ++j) {
+    const float a = to_f32<TW>(wr[j]);
+#pragma unroll
+    for (int t = 0; t < kLowRankTokens; ++t) acc[t] = fmaf(a, rows[t * rp + j], acc[t]);
   }
 #pragma unroll
   for (int t = 0; t < kLowRankTokens; ++t)
@@ -142,8 +154,9 @@ extern "C" int yk_low_rank(const void* y, int y_stride, int y_dtype, const void*
   YK_REQUIRE(rank <= 1536, "low_rank: ranks of more than 1,536 do not fit the row buffer");
   YK_REQUIRE((n_tokens + kLowRankTokens - 1) / kLowRankTokens <= 65535, "low_rank: too many tokens for one launch");
   if (n_tokens == 0) return 0;
-  const bool vec = rank % 4 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
-  dim3 grid((cols + 255) / 256, (n_tokens + kLowRankTokens - 1) / kLowRankTokens);
+  const bool vec = rank % 8 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0;
+  const int columns = vec ? 32 : 256;  // of a workgroup
+  dim3 grid((cols + columns - 1) / columns, (n_tokens + kLowRankTokens - 1) / kLowRankTokens);
   const size_t lds = static_cast<size_t>(kLowRankTokens) * ((rank + 7) / 8 * 8) * sizeof(float);
 #define YK_CASE(YD, T, WD, TW, V)                                                                                    \
   if (y_dtype == YD && w_dtype == WD && vec == V) {                                                                  \

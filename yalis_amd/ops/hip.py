@@ -138,7 +138,7 @@ _SIGNATURES = {
     "yk_latent_attention": ([_vp, _vp, _c_int, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _vp, _vp, _vp], _c_int),
     "yk_linear_state_scan": (
         [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _c_int, _c_int, _c_float, _c_float, _c_int, _vp, _c_int,
-         _c_int, _vp, _vp, _c_float, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp],
+         _c_int, _vp, _vp, _c_float, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _vp],
         _c_int,
     ),
     "yk_gated_head_norm": (
@@ -230,7 +230,7 @@ _LATER_SIGNATURES = {
         "yk_probe_mfma_bf16": ([_c_int, _c_int, _vp, _vp], _c_int),
     },
 }
-_ABI = 22
+_ABI = 23
 
 # Rows of x up to which the hand-written matrix-core kernel runs a bfloat16 product;
 # above it the vendor library does.
@@ -1727,6 +1727,9 @@ class HipOps:
         a = ctx.arrays
         mode = {"head": 0, "channel": 1, "channel_softplus": 2, "channel_exp": 3}[kind]
         beta_f32 = beta is not None and beta[0].dtype == torch.float32
+        # where tokens are many their decays per channel are made first, once for all the columns that read them
+        many = mode != 0 and n > 4 * a["seq_qstart"].numel()
+        decays = torch.empty((n, n_heads * dim), dtype=torch.float32, device=qkv.device) if many else None
         out = torch.empty((n, n_heads * vdim), dtype=torch.float32, device=qkv.device)
         self._check(self.lib.yk_linear_state_scan(
             qkv.data_ptr(), qkv.stride(0), _code(qkv.dtype), n_heads, n_kv, dim, vdim, state.data_ptr(), a["seq_qstart"].data_ptr(),
@@ -1734,7 +1737,7 @@ class HipOps:
             -1.0 if unit_eps is None else float(unit_eps), mode, src.data_ptr(), src.stride(0), col,
             p0.data_ptr(), _ptr(p1), tau, beta[0].data_ptr() if beta_f32 else None, 0 if beta is None else beta[0].stride(0),
             0 if beta is None else int(beta[1]), out.data_ptr(), int(q_col), int(k_col), int(v_col), write_mode, _ptr(skip),
-            beta[0].data_ptr() if beta is not None and not beta_f32 else None, _ptr(bonus), self._stream()))
+            beta[0].data_ptr() if beta is not None and not beta_f32 else None, _ptr(bonus), _ptr(decays), self._stream()))
         return out
 
     def gated_head_norm(self, o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first: bool = False,
