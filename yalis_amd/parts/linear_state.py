@@ -7,7 +7,7 @@ outer product k u^T into it and reads q out of it:
     u  = beta (v - S^T k)           the delta rule        ("delta_rule")
     S <- S + k u^T,   o = S^T q     (the read-out sees the token's own write)
 
-and each head's o is divided by its root mean square, multiplied by a weight (shared by the heads, or one per
+and o is scaled per head to a root mean square of one, multiplied by a weight (shared by the heads, or one per
 element) and by silu or the sigmoid of a projection of the mixer's input, and projected back.  Decays, write strengths, unit
 norms, S and the read-out norm are float32 in both engines; one kernel (``ops.linear_state_scan``)
 walks every request's span with S in registers, one column of S to a group of lanes.

@@ -1,5 +1,5 @@
 """Two mixers side by side: both read the same input, and the result is a multiple of the sum of their outputs,
-each first divided by its root mean square over the model's width and multiplied by a weight of its own.
+each scaled to a root mean square of one (over the model's width) and multiplied by a weight of its own.
 
 params: left, right (PartSpecs of the two mixers), left_norm, right_norm (names of the weights [hidden]), hidden_size,
 eps, scale (0.5).  At most one of the two keeps pages; their states lie one after the other among this mixer's.
