@@ -327,7 +327,7 @@ def qk_row_scales(proj, n_q_cols, n_k_cols, positions, bias=None, eps=None, temp
 
 def qkv_prepare(qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q_norm=None, k_norm=None, qk_eps=0.0,
                 rotation=None, value_norm_eps=None, value_rotation=None, k_cache=None, v_cache=None, slots=None, page_size=0,
-                bias=None, row_scales=None, norm_over_projection=False, values_from_keys=False, unweighted_norm=False):
+                bias=None, row_scales=None, norm_over_projection=False, values_from_keys=False, unweighted_norm=False, query_maps=1):
     n = qkv.shape[0]
     x = qkv.to(torch.float32)
     if bias is not None:
@@ -365,13 +365,31 @@ def qkv_prepare(qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q
         page, off = (slots // page_size).long(), (slots % page_size).long()
         k_cache[page, :, off, :] = k.to(k_cache.dtype)
         v_cache[page, :, :, off] = v.to(v_cache.dtype)
+    if query_maps > 1:  # a row per map, zeros where the other maps' elements are
+        part = head_dim // query_maps
+        rows = torch.zeros((n, n_heads, query_maps, head_dim), dtype=q.dtype, device=q.device)
+        for m in range(query_maps):
+            rows[:, :, m, m * part: (m + 1) * part] = q[:, :, m * part: (m + 1) * part]
+        return rows.reshape(n, query_maps * hd).to(act_dtype)
     return q.reshape(n, hd).to(act_dtype)
 
 
 def attention_masked(q, n_heads, n_kv, head_dim, value_dim, k_cache, v_cache, page_size, scale, ctx, group, window=0,
                      keep_first=0, softcap=0.0, value_rotation=None, gate=None, gate_col=0, gate_elems=1, distance_bias=None, sink=None,
-                     chunked=False):
+                     chunked=False, differential=None):
+    """``differential`` (lambda, eps, gain): a head's queries and keys are two maps side by side, each with a softmax of its
+    own; the output is (a1 - lambda a2) divided by its root mean square and times gain."""
     n = q.shape[0]
+    if differential is not None:
+        lam, eps, gain = differential
+        part = head_dim // 2
+        a = []
+        for m in range(2):
+            qm = q.view(n, n_heads, head_dim)[..., m * part: (m + 1) * part].float().reshape(n, -1)
+            a.append(attention_masked(qm, n_heads, n_kv, part, value_dim, k_cache[..., m * part: (m + 1) * part], v_cache, page_size, scale, ctx,
+                                      group, window, keep_first, softcap, chunked=chunked).view(n, n_heads, value_dim))
+        o = a[0] - lam * a[1]
+        return (o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps) * gain).reshape(n, -1).to(q.dtype)
     positions, token_seq = ctx.arrays["positions"], ctx.arrays["token_seq"]
     bt = ctx.arrays[f"block_table_g{group}"]
     qh = q.view(n, n_heads, head_dim).to(torch.float32)
@@ -554,8 +572,10 @@ def activation(x, kind, out_dtype):
     return y.to(out_dtype)
 
 
-def scale_rows(x, s):
+def scale_rows(x, s, softcap=0.0):
     x *= s
+    if softcap:
+        x.copy_(softcap * torch.tanh(x / softcap))
     return x
 
 
@@ -645,7 +665,9 @@ def linear_state_scan(qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, un
         q = q / torch.sqrt((q * q).sum(-1, keepdim=True) + unit_eps)
         k = k / torch.sqrt((k * k).sum(-1, keepdim=True) + unit_eps)
     q = q * q_scale
-    if decay[0] == "head":
+    if decay[0] == "fixed":
+        g = decay[1].float()[None, :, None].expand(n, n_heads, dim)
+    elif decay[0] == "head":
         _, src, col, a_log, dt_bias = decay
         step = torch.nn.functional.softplus(src[:, col: col + n_heads].float() + dt_bias.float())
         g = torch.exp(-torch.exp(a_log.float()) * step)
@@ -690,6 +712,8 @@ def linear_state_scan(qkv, n_heads, n_kv, dim, vdim, state, ctx, q_scale=1.0, un
 
 def gated_head_norm(o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first=False, gate_act="silu"):
     n = o.shape[0]
+    if weight is None:
+        weight = torch.ones(vdim, dtype=torch.float32, device=o.device)
     g = gate[:, gate_col: gate_col + n_heads * vdim].float()
     if gate_act == "sigmoid":
         w = weight.float() if weight.numel() == vdim else weight.float().view(n_heads, vdim)
@@ -778,6 +802,85 @@ def low_rank(y, w, act=None):
     return linear(torch.tanh(y.float()) if act == "tanh" else y, w, torch.float32)
 
 
+# ------------------------------------ a stream kept as copies, a normed embedding, fixed decays, experts in groups
+def embed_norm(token_ids, table, weight, eps, copies):
+    x = _rmsnorm(table[token_ids.long()].to(torch.float32), weight, eps, False)
+    return x[:, None, :].repeat(1, copies, 1)
+
+
+def streams_norm(residual, y, experts, mix, out, read, rows, weight, eps, unit_offset, out_dtype):
+    """residual [N, streams, width] float32: x_t <- sum_s mix[s, t] x_s + out[t] y (in place unless ``rows`` picks some;
+    mix None: nothing is pending), y = ``y`` + the sum of a token's expert rows; returns norm(sum_s read[s] x_s)."""
+    x = residual
+    if mix is not None:
+        n, _, width = residual.shape
+        branch = torch.zeros((n, width), dtype=torch.float32, device=residual.device)
+        if y is not None:
+            branch = branch + y.float()
+        if experts is not None:
+            branch = moe_combine(branch, *experts)
+        x = torch.einsum("st,nsc->ntc", mix, residual) + out[None, :, None] * branch[:, None, :]
+        if rows is None:
+            residual.copy_(x)
+    if rows is not None:
+        x = x[rows.long()]
+    u = x.sum(1) if read is None else torch.einsum("s,nsc->nc", read, x)
+    return _rmsnorm(u, weight, eps, unit_offset).to(out_dtype)
+
+
+def scan_inputs(proj, n_heads, dim, vdim, k_scale=1.0, rotation=None, positions=None, act=None):
+    """float32 rows [q | k | v] as they enter the recurrence: an activation of all three, or q and k rotated; k scaled."""
+    n, kd = proj.shape[0], n_heads * dim
+    x = proj[:, : 2 * kd + n_heads * vdim].float()
+    if act is not None:
+        x = plain_act(x, act)
+    q, k, v = x[:, :kd].reshape(n, n_heads, dim), x[:, kd: 2 * kd].reshape(n, n_heads, dim), x[:, 2 * kd:]
+    if rotation is not None:
+        c, s = rotation.cos[positions.long()][:, None, :], rotation.sin[positions.long()][:, None, :]
+        q, k = (_turn(t, c, s, rotation.rotary_dim, rotation.interleaved) for t in (q, k))
+    return torch.cat([q.reshape(n, kd), k.reshape(n, kd) * k_scale, v], dim=1)
+
+
+def fixed_decay_scan(proj, n_heads, dim, vdim, state, ctx, decay, k_scale=1.0, rotation=None, act=None, chunks=None, seq_chunk0=None):
+    rows = scan_inputs(proj, n_heads, dim, vdim, k_scale, rotation, ctx.arrays["positions"], act)
+    return linear_state_scan(rows, n_heads, n_heads, dim, vdim, state, ctx, decay=("fixed", decay))
+
+
+def moe_router_share(logits, top, experts=None, bias=None, correction=None, groups=None):
+    """(choice int32 [N, top], weights float32 [N, top]): sigmoid scores, chosen by score + ``correction`` among the experts
+    of the ``groups`` = (count, keep) best groups, weighed by the scores' shares."""
+    experts = logits.shape[1] if experts is None else experts
+    z = logits[:, :experts].float()
+    s = torch.sigmoid(z if bias is None else z + bias)
+    c = s if correction is None else s + correction
+    n = z.shape[0]
+    choice = torch.empty((n, top), dtype=torch.int32, device=logits.device)
+    for t in range(n):
+        left = c[t].clone()
+        if groups is not None:
+            count, keep = groups
+            per = left.view(count, experts // count)
+            score = torch.topk(per, min(2, per.shape[1]), dim=1).values.sum(1)
+            allowed = set()
+            for _ in range(keep):
+                g = int(torch.argmax(score))
+                allowed.add(g)
+                score[g] = -math.inf
+            for g in range(count):
+                if g not in allowed:
+                    per[g] = -math.inf
+        for k in range(top):
+            e = int(torch.argmax(left))
+            choice[t, k] = e
+            left[e] = -math.inf
+    chosen = torch.gather(s, 1, choice.long())
+    return choice, chosen / (chosen.sum(1, keepdim=True) + 1e-20)
+
+
+RefOps.embed_norm = staticmethod(embed_norm)
+RefOps.streams_norm = staticmethod(streams_norm)
+RefOps.fixed_decay_scan = staticmethod(fixed_decay_scan)
+RefOps.moe_router_share = staticmethod(moe_router_share)
 RefOps.sum_norm = staticmethod(sum_norm)
 RefOps.embed_pairs = staticmethod(embed_pairs)
 RefOps.token_shift_mix = staticmethod(token_shift_mix)

@@ -160,6 +160,19 @@ __device__ __forceinline__ float ext_bias(const float* __restrict__ col, int n, 
   return col[static_cast<size_t>(min(max(n, 0), rows - 1)) * n_heads];
 }
 
+// Differential attention on the same kernels: a head's keys are [map 1 | map 2] and every head brings two query rows, one per
+// map with zeros in the other's half (n_heads counts these rows, neighbours are a head's two maps).  Both rows' columns lie
+// in neighbouring lanes of one wave, so the epilogue exchanges them there: o = (a1 - lambda a2) / sqrt(mean(o^2) + eps) * gain,
+// float32 until it is stored, in rows of n_heads / 2 heads.
+struct MapArgs {
+  int on;
+  float lambda, eps, gain;
+};
+// the other map's value of the same element (lane r ^ 1)
+__device__ __forceinline__ float other_map(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), 0xB1, 0xf, 0xf, false));  // quad_perm [1,0,3,2]
+}
+
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
 typedef float f32x4_t __attribute__((ext_vector_type(4)));
 typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
@@ -262,7 +275,7 @@ __global__ __launch_bounds__(64 * W, 2) void attn_mfma_kernel(
     int page_size, int n_heads, int n_kv, int hpt, int chunks, float scale_log2, int window,
     int n_splits, float* __restrict__ ws_o, float* __restrict__ ws_ml, RopeSrc rs, int keep_first_arg = 0,
     float cap_over_scale = 0.f, float scale_over_cap_2log2e = 0.f, const float* __restrict__ dist_bias = nullptr,
-    int bias_rows = 0, float inv_scale = 0.f, const float* __restrict__ sink = nullptr, int chunked_arg = 0) {
+    int bias_rows = 0, float inv_scale = 0.f, const float* __restrict__ sink = nullptr, int chunked_arg = 0, MapArgs maps = MapArgs{}) {
   const int keep_first = EXT ? keep_first_arg : 0, chunked = EXT ? chunked_arg : 0;
   constexpr int KS = D / 32;  // matrix-core steps over the head dimension
   constexpr int DT = D / 16;  // output tiles over the head dimension
@@ -675,7 +688,30 @@ __global__ __launch_bounds__(64 * W, 2) void attn_mfma_kernel(
     m = m_all;
   }
 
-  if (n_splits == 1) {
+  if (EXT && maps.on && n_splits == 1) {
+    // (every lane takes part in the exchanges; columns that stand for nothing are not stored)
+    const float inv = 1.f / l;
+    float ss = 0.f;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float a = acc[dt][i] * inv;
+        acc[dt][i] = fmaf(-maps.lambda, other_map(a), a);
+        ss = fmaf(acc[dt][i], acc[dt][i], ss);
+      }
+    const float to_unit = maps.gain / sqrtf(column_lanes_sum(ss) / static_cast<float>(D) + maps.eps);
+    if (col_ok && hh % 2 == 0) {
+      bf16_t* op = out + (static_cast<size_t>(tok0 + tt) * (n_heads / 2) + (h_base + hh) / 2) * D + 4 * gq;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt) {
+        u32x2_t w;
+        w[0] = pack_bf16x2(acc[dt][0] * to_unit, acc[dt][1] * to_unit);
+        w[1] = pack_bf16x2(acc[dt][2] * to_unit, acc[dt][3] * to_unit);
+        *reinterpret_cast<u32x2_t*>(op + 16 * dt) = w;
+      }
+    }
+  } else if (n_splits == 1) {
     if (col_ok) {
       // (m and l are in powers of two: the sink's share is 2^(sink log2(e) - m))
       if (EXT && sink != nullptr) l += fast_exp2(fmaf(sink[h_base + hh], 1.4426950408889634f, -m));
@@ -723,7 +759,7 @@ __global__ __launch_bounds__(256, CT == 1 ? 3 : 2) void attn_mfma_prefill_kernel
     int page_size, int n_heads, int n_kv, int hpt, int chunks, float scale_log2, int window,
     int n_splits, float* __restrict__ ws_o, float* __restrict__ ws_ml, int pages_lds_limit, int keep_first_arg,
     float cap_over_scale, float scale_over_cap_2log2e, const float* __restrict__ dist_bias, int bias_rows, float inv_scale,
-    const float* __restrict__ sink, int chunked_arg) {
+    const float* __restrict__ sink, int chunked_arg, MapArgs maps) {
   constexpr int KS = D / 32, DT = D / 16;
   const int keep_first = EXT ? keep_first_arg : 0, chunked = EXT ? chunked_arg : 0;
   constexpr int KROW = D + 8;   // bf16 elements per parked key row
@@ -1034,6 +1070,30 @@ __global__ __launch_bounds__(256, CT == 1 ? 3 : 2) void attn_mfma_prefill_kernel
       }
       continue;
     }
+    if (EXT && maps.on) {
+      const float inv = 1.f / lc;
+      float ss = 0.f;
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float a = acc[c][dt][i] * inv;
+          acc[c][dt][i] = fmaf(-maps.lambda, other_map(a), a);
+          ss = fmaf(acc[c][dt][i], acc[c][dt][i], ss);
+        }
+      const float to_unit = maps.gain / sqrtf(column_lanes_sum(ss) / static_cast<float>(D) + maps.eps);
+      if (col_ok[c] && hh % 2 == 0) {
+        bf16_t* op = out + (static_cast<size_t>(tile_tok0 + tok_c[c]) * (n_heads / 2) + (h_base + hh) / 2) * D + 4 * gq;
+#pragma unroll
+        for (int dt = 0; dt < DT; ++dt) {
+          u32x2_t w;
+          w[0] = pack_bf16x2(acc[c][dt][0] * to_unit, acc[c][dt][1] * to_unit);
+          w[1] = pack_bf16x2(acc[c][dt][2] * to_unit, acc[c][dt][3] * to_unit);
+          *reinterpret_cast<u32x2_t*>(op + 16 * dt) = w;
+        }
+      }
+      continue;
+    }
     if (col_ok[c]) {
       if (EXT && sink != nullptr) lc += fast_exp2(fmaf(sink[h_base + hh], 1.4426950408889634f, -m[c]));
       const float inv = 1.f / lc;
@@ -1082,6 +1142,48 @@ __global__ __launch_bounds__(256) void attn_combine_kernel(
   }
 }
 
+// The same where neighbouring columns are a head's two maps: a thread merges four elements of both, the D / 4 threads of
+// a head take its root mean square together.
+template <int D>
+__global__ __launch_bounds__(256) void attn_combine_maps_kernel(
+    bf16_t* __restrict__ out, const int32_t* __restrict__ tiles, int n_heads, int n_kv, int hpt,
+    int chunks, int n_splits, const float* __restrict__ ws_o, const float* __restrict__ ws_ml, int parts, MapArgs maps) {
+  const int t = blockIdx.x / parts, part = blockIdx.x % parts;
+  const int tpt_ = 16 / hpt;
+  const int tok0 = tiles[4 * t + 1] + part * tpt_, ntok = tiles[4 * t + 2] - part * tpt_;
+  const int g = blockIdx.y / chunks, chunk = blockIdx.y % chunks;
+  const int qpk = n_heads / n_kv;
+  const int h_base = g * qpk + chunk * hpt;
+  const int heads_here = min(hpt, qpk - chunk * hpt);
+  const size_t w0 = (static_cast<size_t>(blockIdx.x) * gridDim.y + blockIdx.y) * n_splits;
+  constexpr int PIECES = D / 4;  // a multiple of 16: a head's threads lie in one wave
+  for (int e = threadIdx.x; e < 8 * PIECES; e += blockDim.x) {
+    const int c = 2 * (e / PIECES), d = (e % PIECES) * 4;
+    const int tt = c / hpt, hh = c % hpt;
+    const bool live = tt < min(ntok, tpt_) && hh < heads_here;
+    float a1[4] = {0.f, 0.f, 0.f, 0.f}, a2[4] = {0.f, 0.f, 0.f, 0.f};
+    if (live) {
+      attn_merge_splits(ws_o, ws_ml, w0 * 16 + c, n_splits, D, d, a1);
+      attn_merge_splits(ws_o, ws_ml, w0 * 16 + c + 1, n_splits, D, d, a2);
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      a1[i] = fmaf(-maps.lambda, a2[i], a1[i]);
+      ss = fmaf(a1[i], a1[i], ss);
+    }
+#pragma unroll
+    for (int o = PIECES / 2; o > 0; o /= 2) ss += __shfl_xor(ss, o, kWave);
+    const float to_unit = maps.gain / sqrtf(ss / static_cast<float>(D) + maps.eps);
+    if (live) {
+      u32x2_t o;
+      o[0] = pack_bf16x2(a1[0] * to_unit, a1[1] * to_unit);
+      o[1] = pack_bf16x2(a1[2] * to_unit, a1[3] * to_unit);
+      *reinterpret_cast<u32x2_t*>(out + (static_cast<size_t>(tok0 + tt) * (n_heads / 2) + (h_base + hh) / 2) * D + d) = o;
+    }
+  }
+}
+
 extern "C" int yk_attn_mfma_supported(int head_dim) { return head_dim == 64 || head_dim == 128; }
 
 // Heads of one kv head that share a wave, and tokens per tile, for a head layout.
@@ -1114,8 +1216,12 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
                                     int head_dim, int n_heads, int n_kv, float scale, int window,
                                     int n_splits, int col_tiles, float* workspace, size_t workspace_floats,
                                     int pages_lds_limit, int keep_first, float softcap, const float* dist_bias, int bias_rows,
-                                    const float* sink, int chunked, hipStream_t stream) {
+                                    const float* sink, int chunked, int maps, float map_lambda, float map_eps, float map_gain,
+                                    hipStream_t stream) {
   YK_REQUIRE(n_tiles >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attn_mfma_prefill: bad head counts");
+  YK_REQUIRE(maps == 1 || (maps == 2 && (n_heads / n_kv) % 2 == 0 && sink == nullptr && dist_bias == nullptr),
+             "attn_mfma_prefill: one map, or two query rows a head without sinks and biases per distance");
+  const MapArgs map_args{maps == 2, map_lambda, map_eps, map_gain};
   YK_REQUIRE(!chunked || (window > 0 && keep_first == 0), "attn_mfma_prefill: chunks need their size and keep no first keys");
   YK_REQUIRE(col_tiles == 1 || col_tiles == 2, "attn_mfma_prefill: a wave has 1 or 2 column tiles");
   YK_REQUIRE(yk_attn_mfma_supported(head_dim), "attn_mfma_prefill: head_dim must be 64 or 128");
@@ -1129,7 +1235,7 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
   YK_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attn_mfma_prefill: keep_first and softcap must not be negative");
   YK_REQUIRE(dist_bias == nullptr || bias_rows >= 1, "attn_mfma_prefill: an empty table of biases");
   if (n_tiles == 0) return 0;
-  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr || chunked;
+  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr || chunked || maps == 2;
   const float inv_scale = 1.f / scale;
   const float cap_over_scale = softcap > 0.f ? softcap / scale : 0.f;
   const float scale_over_cap = softcap > 0.f ? scale / softcap * 2.f * 1.4426950408889634f : 0.f;
@@ -1147,7 +1253,7 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
   static_cast<const bf16_t*>(q), q_stride, static_cast<bf16_t*>(out), static_cast<const bf16_t*>(k_cache),     \
       static_cast<const bf16_t*>(v_cache), tiles, block_table, table_width, page_size, n_heads, n_kv, hpt,     \
       chunks, scale_log2, window, n_splits, ws_o, ws_ml, pages_lds_limit, keep_first, cap_over_scale, scale_over_cap, \
-      dist_bias, bias_rows, inv_scale, sink, chunked
+      dist_bias, bias_rows, inv_scale, sink, chunked, map_args
 #define YK_PF(DD, BIP)                                                                                       \
   if (ext && col_tiles == 2)                                                                                 \
     attn_mfma_prefill_kernel<DD, BIP, 2, true><<<grid, block, 0, stream>>>(YK_PF_ARGS);                      \
@@ -1168,7 +1274,11 @@ extern "C" int yk_attn_mfma_prefill(const void* q, int q_stride, void* out, cons
   if (yk_check_launch("attn_mfma_prefill")) return -1;
   if (n_splits > 1) {
     dim3 cgrid(4 * col_tiles * n_tiles, n_kv * chunks);
-    if (head_dim == 64)
+    if (maps == 2 && head_dim == 64)
+      attn_combine_maps_kernel<64><<<cgrid, 256, 0, stream>>>(static_cast<bf16_t*>(out), tiles, n_heads, n_kv, hpt, chunks, n_splits, ws_o, ws_ml, 4 * col_tiles, map_args);
+    else if (maps == 2)
+      attn_combine_maps_kernel<128><<<cgrid, 256, 0, stream>>>(static_cast<bf16_t*>(out), tiles, n_heads, n_kv, hpt, chunks, n_splits, ws_o, ws_ml, 4 * col_tiles, map_args);
+    else if (head_dim == 64)
       attn_combine_kernel<64><<<cgrid, 256, 0, stream>>>(static_cast<bf16_t*>(out), tiles, n_heads, n_kv, hpt, chunks, n_splits, ws_o, ws_ml, 4 * col_tiles, sink);
     else
       attn_combine_kernel<128><<<cgrid, 256, 0, stream>>>(static_cast<bf16_t*>(out), tiles, n_heads, n_kv, hpt, chunks, n_splits, ws_o, ws_ml, 4 * col_tiles, sink);
@@ -1187,13 +1297,15 @@ static int launch_attn_mfma(const void* q, int q_stride, void* out, const void* 
                             int n_waves, int n_splits, float* workspace, size_t workspace_floats,
                             int leave_splits, const RopeSrc* rope, bool rope_f32, hipStream_t stream, int keep_first = 0,
                             float softcap = 0.f, const float* dist_bias = nullptr, int bias_rows = 0, const float* sink = nullptr,
-                            int chunked = 0) {
+                            int chunked = 0, MapArgs maps = MapArgs{}) {
+  YK_REQUIRE(!maps.on || ((n_heads / n_kv) % 2 == 0 && sink == nullptr && dist_bias == nullptr && !leave_splits),
+             "attn_mfma: two maps are two query rows a head, without sinks and biases per distance, merged here");
   YK_REQUIRE(!chunked || (window > 0 && keep_first == 0), "attn_mfma: chunks need their size and keep no first keys");
   YK_REQUIRE(n_tiles >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attn_mfma: bad head counts");
   YK_REQUIRE(sink == nullptr || !leave_splits, "attn_mfma: splits that another kernel merges cannot carry a sink");
   YK_REQUIRE(keep_first >= 0 && softcap >= 0.f, "attn_mfma: keep_first and softcap must not be negative");
   YK_REQUIRE(dist_bias == nullptr || bias_rows >= 1, "attn_mfma: an empty table of biases");
-  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr || chunked;
+  const bool ext = (keep_first > 0 && window > 0) || softcap > 0.f || dist_bias != nullptr || sink != nullptr || chunked || maps.on;
   const float inv_scale = scale > 0.f ? 1.f / scale : 0.f;
   YK_REQUIRE(!(ext && rope), "attn_mfma: kept first keys and squashed scores are not offered with rotary inside the launch");
   const float cap_over_scale = softcap > 0.f ? softcap / scale : 0.f;
@@ -1234,17 +1346,21 @@ static int launch_attn_mfma(const void* q, int q_stride, void* out, const void* 
   }
 #define YK_LAUNCH_EXT(DD)                                                                          \
   if (tiled) {                                                                                     \
-    if (n_waves == 1) attn_mfma_kernel<DD, 1, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
-    else attn_mfma_kernel<DD, 4, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
+    if (n_waves == 1) attn_mfma_kernel<DD, 1, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked, maps); \
+    else attn_mfma_kernel<DD, 4, true, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked, maps); \
   } else {                                                                                         \
-    if (n_waves == 1) attn_mfma_kernel<DD, 1, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
-    else attn_mfma_kernel<DD, 4, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked); \
+    if (n_waves == 1) attn_mfma_kernel<DD, 1, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked, maps); \
+    else attn_mfma_kernel<DD, 4, false, 0, true><<<grid, block, 0, stream>>>(YK_ARGS, keep_first, cap_over_scale, scale_over_cap, dist_bias, bias_rows, inv_scale, sink, chunked, maps); \
   }
 #define YK_LAUNCH(DD)                                                                              \
   if (ext) { YK_LAUNCH_EXT(DD) } else                                                              \
   if (!rope) { YK_LAUNCH_R(DD, 0) } else if (rope_f32) { YK_LAUNCH_R(DD, 2) } else { YK_LAUNCH_R(DD, 1) } \
   if (yk_check_launch("attn_mfma")) return -1;                                                     \
-  if (n_splits > 1 && !leave_splits) {                                                             \
+  if (n_splits > 1 && maps.on) {                                                                   \
+    attn_combine_maps_kernel<DD><<<dim3(n_tiles, n_kv * chunks), 256, 0, stream>>>(                \
+        static_cast<bf16_t*>(out), tiles, n_heads, n_kv, hpt, chunks, n_splits, ws_o, ws_ml, 1, maps); \
+    if (yk_check_launch("attn_combine")) return -1;                                                \
+  } else if (n_splits > 1 && !leave_splits) {                                                      \
     attn_combine_kernel<DD><<<dim3(n_tiles, n_kv * chunks), 256, 0, stream>>>(                     \
         static_cast<bf16_t*>(out), tiles, n_heads, n_kv, hpt, chunks, n_splits, ws_o, ws_ml, 1, sink); \
     if (yk_check_launch("attn_combine")) return -1;                                                \
@@ -1267,10 +1383,13 @@ extern "C" int yk_attn_mfma(const void* q, int q_stride, void* out, const void* 
                             int head_dim, int n_heads, int n_kv, float scale, int window,
                             int n_waves, int n_splits, float* workspace, size_t workspace_floats,
                             int leave_splits, int keep_first, float softcap, const float* dist_bias, int bias_rows,
-                            const float* sink, int chunked, hipStream_t stream) {
+                            const float* sink, int chunked, int maps, float map_lambda, float map_eps, float map_gain,
+                            hipStream_t stream) {
+  YK_REQUIRE(maps == 1 || maps == 2, "attn_mfma: one map or two");
   return launch_attn_mfma(q, q_stride, out, k_cache, v_cache, tiles, n_tiles, block_table, table_width, page_size,
                           head_dim, n_heads, n_kv, scale, window, n_waves, n_splits, workspace, workspace_floats,
-                          leave_splits, nullptr, false, stream, keep_first, softcap, dist_bias, bias_rows, sink, chunked);
+                          leave_splits, nullptr, false, stream, keep_first, softcap, dist_bias, bias_rows, sink, chunked,
+                          MapArgs{maps == 2, map_lambda, map_eps, map_gain});
 }
 
 // yk_attn_mfma for a step of single tokens (every tile holds ONE token), with rotary + append

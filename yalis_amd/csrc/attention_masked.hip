@@ -11,10 +11,14 @@
 //    its key heads), with weights as wide as the projections, whose inverse root mean square comes from
 //  * yk_qk_row_scales: per token, what its queries and its keys are multiplied with as wholes after the weights:
 //    that inverse root mean square and / or the queries' temperature 1 + coef ln(floor((p + 1) / every) + 1).
+//    With q_maps > 1 a head's elements are that many maps side by side and every map's queries are written as a row of
+//    their own, zeros where the other maps' elements are: its products with whole key rows are the map's scores.
 //  * yk_attn_masked: scores q . k * scale, optionally squashed s <- cap * tanh(s / cap); key j
 //    is visible to the query at position p iff j <= p and (p - j < window or j < keep_first)
 //    (window 0: no window), or, chunked, floor(j / window) = floor(p / window); softmax over the visible keys; keys of head_dim, values of
 //    value_dim elements.  One wave per (token, head), float32 arithmetic, any sizes up to 256.
+//    With two maps (differential attention) a head's queries and keys are [map 1 | map 2]; each map has a softmax of its own
+//    over its half's scores, and the head's output is (a1 - lambda a2) divided by its root mean square, times a gain.
 //    Its epilogue can turn the output back by the query's own position (the inverse of the
 //    values' rotation) and multiply a head's output by the sigmoid of a gate column of the
 //    projection.
@@ -57,7 +61,7 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(
     int interleaved, int max_pos, int v_norm, float v_eps, const float* __restrict__ v_cos,
     const float* __restrict__ v_sin, int v_interleaved, int v_max_pos, T* __restrict__ k_cache,
     T* __restrict__ v_cache, const int32_t* __restrict__ slots, int page_size, int tiled,
-    const float* __restrict__ bias, const float* __restrict__ row_scales, int v_from_k) {
+    const float* __restrict__ bias, const float* __restrict__ row_scales, int v_from_k, int q_maps) {
   __shared__ float bufs[4][kMaxHead];
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   float* buf = bufs[wave];
@@ -166,7 +170,8 @@ __global__ __launch_bounds__(256) void qkv_prepare_kernel(
         v = d < rot / 2 ? rot_first(buf[d], buf[d + rot / 2], cv[i], sv[i]) : rot_second(buf[d - rot / 2], buf[d], cv[i], sv[i]);
     }
     if (kind == 0)
-      q_out[static_cast<size_t>(n) * q_stride + col0 + d] = from_f32<T>(v);
+      for (int mp = 0; mp < q_maps; ++mp)  // a row per map, zeros where the other maps' elements are
+        q_out[static_cast<size_t>(n) * q_stride + static_cast<size_t>(col0) * q_maps + mp * head_dim + d] = from_f32<T>(d / (head_dim / q_maps) == mp ? v : 0.f);
     else if (kind == 1)
       k_cache[base + cache_k_offset(tiled, page_size, head_dim, off, d)] = from_f32<T>(v);
     else
@@ -189,7 +194,7 @@ __global__ __launch_bounds__(512) void qkv_prepare8_kernel(
     int interleaved, int max_pos, int v_norm, float v_eps, const float* __restrict__ v_cos,
     const float* __restrict__ v_sin, int v_interleaved, int v_max_pos, bf16_t* __restrict__ k_cache,
     bf16_t* __restrict__ v_cache, const int32_t* __restrict__ slots, int page_size, int tiled, int n_tokens,
-    const float* __restrict__ bias, const float* __restrict__ row_scales, int v_from_k) {
+    const float* __restrict__ bias, const float* __restrict__ row_scales, int v_from_k, int q_maps) {
   __shared__ float bufs[8][kMaxHead];
   __shared__ __attribute__((aligned(16))) bf16_t outs[8][kMaxHead];
   __shared__ int slot_s[8];
@@ -297,8 +302,9 @@ __global__ __launch_bounds__(512) void qkv_prepare8_kernel(
   if (kind == 0) {
     for (int idx = threadIdx.x; idx < n_live * pieces; idx += blockDim.x) {
       const int t = idx / pieces, p = idx % pieces;
-      *reinterpret_cast<uint4*>(q_out + static_cast<size_t>(n0 + t) * q_stride + col0 + 8 * p) =
-          *reinterpret_cast<const uint4*>(&outs[t][8 * p]);
+      for (int mp = 0; mp < q_maps; ++mp)  // a row per map, zeros where the other maps' elements are
+        *reinterpret_cast<uint4*>(q_out + static_cast<size_t>(n0 + t) * q_stride + static_cast<size_t>(col0) * q_maps + mp * head_dim + 8 * p) =
+            p / (pieces / q_maps) == mp ? *reinterpret_cast<const uint4*>(&outs[t][8 * p]) : make_uint4(0u, 0u, 0u, 0u);
     }
     return;
   }
@@ -345,8 +351,9 @@ extern "C" int yk_qkv_prepare(const void* src, int src_dtype, int n_splits, int 
                               int interleaved, int max_pos, int v_norm, float v_eps, const float* v_cos,
                               const float* v_sin, int v_interleaved, int v_max_pos, void* k_cache, void* v_cache,
                               const int32_t* slots, int page_size, int tiled, const float* bias, const float* row_scales,
-                              int v_from_k, hipStream_t stream) {
+                              int v_from_k, int q_maps, hipStream_t stream) {
   YK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv >= 0, "qkv_prepare: bad sizes");
+  YK_REQUIRE(q_maps >= 1 && head_dim % q_maps == 0 && q_stride >= n_heads * q_maps * head_dim, "qkv_prepare: a head's elements divide into its maps");
   YK_REQUIRE(qk_norm >= 0 && qk_norm <= 2 && (qk_norm != 2 || (row_scales != nullptr && q_norm_w != nullptr && (n_kv == 0 || k_norm_w != nullptr))),
              "qkv_prepare: a norm over the whole projection takes its weights and the rows' scales");
   YK_REQUIRE(!v_from_k || v_dim == head_dim, "qkv_prepare: values that are the keys are as wide as the keys");
@@ -361,7 +368,7 @@ extern "C" int yk_qkv_prepare(const void* src, int src_dtype, int n_splits, int 
   if (n_tokens == 0) return 0;
   const size_t stride = static_cast<size_t>(n_tokens) * src_stride;
   auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
-  if (act_dtype == YK_BF16 && n_tokens >= 16 && head_dim % 8 == 0 && v_dim % 8 == 0 && q_stride % 8 == 0 && page_size % 8 == 0 &&
+  if (act_dtype == YK_BF16 && n_tokens >= 16 && head_dim % (8 * q_maps) == 0 && v_dim % 8 == 0 && q_stride % 8 == 0 && page_size % 8 == 0 &&
       al16(q_out) && al16(k_cache) && al16(v_cache) && (norm_w_dtype == YK_BF16 || norm_w_dtype == YK_F32)) {
     dim3 grid8((n_tokens + 7) / 8, n_heads + 2 * n_kv);
 #define YK_CASE8(SD, TS, WD, TW)                                                                              \
@@ -371,7 +378,7 @@ extern "C" int yk_qkv_prepare(const void* src, int src_dtype, int n_splits, int 
         n_heads, n_kv, head_dim, v_dim, positions, static_cast<const TW*>(q_norm_w),                           \
         static_cast<const TW*>(k_norm_w), qk_norm, qk_eps, cos_t, sin_t, rotary_dim, interleaved, max_pos,      \
         v_norm, v_eps, v_cos, v_sin, v_interleaved, v_max_pos, static_cast<bf16_t*>(k_cache),                  \
-        static_cast<bf16_t*>(v_cache), slots, page_size, tiled, n_tokens, bias, row_scales, v_from_k);         \
+        static_cast<bf16_t*>(v_cache), slots, page_size, tiled, n_tokens, bias, row_scales, v_from_k, q_maps);         \
     return yk_check_launch("qkv_prepare (8 tokens)");                                                          \
   }
     YK_CASE8(YK_F32, float, YK_F32, float)
@@ -388,7 +395,7 @@ extern "C" int yk_qkv_prepare(const void* src, int src_dtype, int n_splits, int 
         n_heads, n_kv, head_dim, v_dim, positions, static_cast<const TW*>(q_norm_w),                          \
         static_cast<const TW*>(k_norm_w), qk_norm, qk_eps, cos_t, sin_t, rotary_dim, interleaved, max_pos,     \
         v_norm, v_eps, v_cos, v_sin, v_interleaved, v_max_pos, static_cast<T*>(k_cache), static_cast<T*>(v_cache), \
-        slots, page_size, tiled, bias, row_scales, v_from_k);                                                 \
+        slots, page_size, tiled, bias, row_scales, v_from_k, q_maps);                                                 \
     return yk_check_launch("qkv_prepare");                                                                    \
   }
   YK_CASE(YK_F32, float, YK_F32, float, YK_F32, float)
@@ -511,7 +518,8 @@ __global__ __launch_bounds__(64) void attn_masked_kernel(
     int n_kv, float scale, float softcap, int window, int keep_first, int tiled, const float* __restrict__ v_cos,
     const float* __restrict__ v_sin, int v_interleaved, int v_max_pos, const TG* __restrict__ gate_src,
     int gate_splits, size_t gate_split_stride, int gate_round, int gate_stride, int gate_col0, int gate_elems,
-    const float* __restrict__ dist_bias, int bias_rows, const float* __restrict__ sink, int chunked) {
+    const float* __restrict__ dist_bias, int bias_rows, const float* __restrict__ sink, int chunked, int maps, float map_lambda,
+    float map_eps, float map_gain) {
   const size_t slab_k = static_cast<size_t>(page_size) * head_dim, slab_v = static_cast<size_t>(page_size) * v_dim;
   __shared__ float qs[kMaxHead];
   __shared__ float os[kMaxHead];
@@ -528,57 +536,71 @@ __global__ __launch_bounds__(64) void attn_masked_kernel(
   for (int d = lane; d < head_dim; d += 64) qs[d] = to_f32<T>(qrow[d]);
   __syncthreads();
   const int32_t* bt = block_table + static_cast<size_t>(seq) * table_width;
-  // a sink starts the running maximum and counts once in the sum: exp(sink) in the denominator, with no value
-  float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.f : 0.f;
-  float acc[4] = {0.f, 0.f, 0.f, 0.f};
-  for (int t0 = 0; t0 < total; t0 += 64) {
-    const int idx = t0 + lane;
-    const bool valid = idx < total;
-    float s = -INFINITY;
-    int base = 0, off = 0;
-    if (valid) {
-      const int key = idx < n_first ? idx : lo + (idx - n_first);
-      const int page = bt[key / page_size];
-      off = key % page_size;
-      base = page * n_kv + g;
-      const T* kp = k_cache + static_cast<size_t>(base) * slab_k;
-      float dot = 0.f;
-      for (int d = 0; d < head_dim; ++d)
-        dot = fmaf(qs[d], to_f32<T>(kp[cache_k_offset(tiled, page_size, head_dim, off, d)]), dot);
-      s = dot * scale;
-      if (softcap > 0.f) s = softcap * tanhf(s / softcap);
-      // a learned number per (distance, head), added to the scaled score as it is
-      if (dist_bias != nullptr) s += dist_bias[static_cast<size_t>(min(pos - key, bias_rows - 1)) * n_heads + h];
-    }
-    const float m_new = fmaxf(m, wave_max(s));  // finite: the tile holds at least one key
-    const float p = valid ? expf(s - m_new) : 0.f;
-    const float alpha = expf(m - m_new);  // 0 on the first tile
-    l = l * alpha + wave_sum(p);
-    m = m_new;
-    __syncthreads();  // the previous tile's ps/pbase are no longer read
-    ps[lane] = p;
-    pbase[lane] = base;
-    poff[lane] = off;
-    __syncthreads();
-    const int count = min(64, total - t0);
+  const int part = head_dim / maps;  // elements of a map
+  float combined[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int mp = 0; mp < maps; ++mp) {
+    // a sink starts the running maximum and counts once in the sum: exp(sink) in the denominator, with no value
+    float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.f : 0.f;
+    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int t0 = 0; t0 < total; t0 += 64) {
+      const int idx = t0 + lane;
+      const bool valid = idx < total;
+      float s = -INFINITY;
+      int base = 0, off = 0;
+      if (valid) {
+        const int key = idx < n_first ? idx : lo + (idx - n_first);
+        const int page = bt[key / page_size];
+        off = key % page_size;
+        base = page * n_kv + g;
+        const T* kp = k_cache + static_cast<size_t>(base) * slab_k;
+        float dot = 0.f;
+        for (int d = mp * part; d < (mp + 1) * part; ++d)
+          dot = fmaf(qs[d], to_f32<T>(kp[cache_k_offset(tiled, page_size, head_dim, off, d)]), dot);
+        s = dot * scale;
+        if (softcap > 0.f) s = softcap * tanhf(s / softcap);
+        // a learned number per (distance, head), added to the scaled score as it is
+        if (dist_bias != nullptr) s += dist_bias[static_cast<size_t>(min(pos - key, bias_rows - 1)) * n_heads + h];
+      }
+      const float m_new = fmaxf(m, wave_max(s));  // finite: the tile holds at least one key
+      const float p = valid ? expf(s - m_new) : 0.f;
+      const float alpha = expf(m - m_new);  // 0 on the first tile
+      l = l * alpha + wave_sum(p);
+      m = m_new;
+      __syncthreads();  // the previous tile's ps/pbase are no longer read
+      ps[lane] = p;
+      pbase[lane] = base;
+      poff[lane] = off;
+      __syncthreads();
+      const int count = min(64, total - t0);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = lane + 64 * i;
-      if (d < v_dim) {
-        float a = acc[i] * alpha;
-        for (int j = 0; j < count; ++j) {
-          const T* vp = v_cache + static_cast<size_t>(pbase[j]) * slab_v + cache_v_offset(tiled, page_size, v_dim, poff[j], d);
-          a = fmaf(ps[j], to_f32<T>(*vp), a);
+      for (int i = 0; i < 4; ++i) {
+        const int d = lane + 64 * i;
+        if (d < v_dim) {
+          float a = acc[i] * alpha;
+          for (int j = 0; j < count; ++j) {
+            const T* vp = v_cache + static_cast<size_t>(pbase[j]) * slab_v + cache_v_offset(tiled, page_size, v_dim, poff[j], d);
+            a = fmaf(ps[j], to_f32<T>(*vp), a);
+          }
+          acc[i] = a;
         }
-        acc[i] = a;
       }
     }
+    const float inv = 1.f / l, share = mp == 0 ? 1.f : -map_lambda;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) combined[i] = fmaf(share, acc[i] * inv, combined[i]);
   }
-  const float inv = 1.f / l;
+  if (maps > 1) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ss = fmaf(combined[i], combined[i], ss);  // (nothing beyond v_dim)
+    const float to_unit = map_gain / sqrtf(wave_sum(ss) / static_cast<float>(v_dim) + map_eps);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) combined[i] *= to_unit;
+  }
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int d = lane + 64 * i;
-    if (d < v_dim) os[d] = acc[i] * inv;
+    if (d < v_dim) os[d] = combined[i];
   }
   __syncthreads();
   float gate = 1.f;
@@ -605,13 +627,16 @@ __global__ __launch_bounds__(64) void attn_masked_kernel(
 // gate_elems: 1, a gate per head in column gate_col0 + h, or v_dim, one per output element in column gate_col0 + h *
 // v_dim + d.  dist_bias [bias_rows][n_heads] float32 or null: what is added to the score of a key at distance n (the
 // last row for every larger distance).  sink [n_heads] float32 or null: exp(sink[h]) joins head h's denominator once.
+// maps 2: see above, with lambda, the eps under the root and the gain (without maps they are not read).
 extern "C" int yk_attn_masked(const void* q, int q_stride, void* out, const void* k_cache, const void* v_cache, int dtype,
                               const int32_t* positions, const int32_t* token_seq, const int32_t* block_table,
                               int table_width, int n_tokens, int page_size, int head_dim, int v_dim, int n_heads, int n_kv,
                               float scale, float softcap, int window, int keep_first, int tiled, const float* v_cos,
                               const float* v_sin, int v_interleaved, int v_max_pos, const void* gate_src, int gate_dtype,
                               int gate_splits, int gate_round, int gate_stride, int gate_col0, int gate_elems,
-                              const float* dist_bias, int bias_rows, const float* sink, int chunked, hipStream_t stream) {
+                              const float* dist_bias, int bias_rows, const float* sink, int chunked, int maps, float map_lambda,
+                              float map_eps, float map_gain, hipStream_t stream) {
+  YK_REQUIRE(maps == 1 || (maps == 2 && head_dim % 2 == 0 && sink == nullptr && dist_bias == nullptr), "attn_masked: one map, or two without sinks and biases per distance");
   YK_REQUIRE(!chunked || (window > 0 && keep_first == 0), "attn_masked: chunks need their size and keep no first keys");
   YK_REQUIRE(n_tokens >= 0 && n_heads > 0 && n_kv > 0 && n_heads % n_kv == 0, "attn_masked: bad head counts");
   YK_REQUIRE(gate_src == nullptr || gate_elems == 1 || gate_elems == v_dim, "attn_masked: a gate per head or per output element");
@@ -633,7 +658,7 @@ extern "C" int yk_attn_masked(const void* q, int q_stride, void* out, const void
         static_cast<const T*>(v_cache), positions, token_seq, block_table, table_width, page_size, head_dim,   \
         v_dim, n_heads, n_kv, scale, softcap, window, keep_first, tiled, v_cos, v_sin, v_interleaved, v_max_pos, \
         static_cast<const TG*>(gate_src), gate_splits, gstride, gate_round, gate_stride, gate_col0, gate_elems, \
-        dist_bias, bias_rows, sink, chunked);                                                                  \
+        dist_bias, bias_rows, sink, chunked, maps, map_lambda, map_eps, map_gain);                             \
     return yk_check_launch("attn_masked");                                                                     \
   }
   YK_CASE(YK_F32, float, YK_F32, float)

@@ -181,6 +181,95 @@ extern "C" int yk_moe_router_topk(const float* logits, int logits_stride, int n_
   return yk_check_launch("moe_router_topk");
 }
 
+// The same choice with other weights: scores s = sigmoid(logit [+ bias]), choice scores c = s + correction (null: c = s).  With
+// `groups` > 0 the experts form that many equal groups of neighbours; a group's score is the sum of its two largest c, and
+// only experts of the `keep` best groups can be chosen.  The `top` largest c win (ties: the lower number, of groups too), their
+// weights are s / (sum of the chosen s + 1e-20).  A wave a token, four tokens a workgroup; scores and choice scores live in LDS.
+__global__ __launch_bounds__(256) void moe_router_share_kernel(const float* __restrict__ logits, int logits_stride, int n_experts, int top,
+                                                               const float* __restrict__ bias, const float* __restrict__ correction,
+                                                               int groups, int keep, int32_t* __restrict__ choice,
+                                                               float* __restrict__ weights, int n_tokens) {
+  extern __shared__ float share_lds[];  // per wave: scores and choice scores [n_experts] each, groups' scores and marks [groups] each
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  float* sc = share_lds + static_cast<size_t>(wave) * 2 * (n_experts + groups);
+  float* ch = sc + n_experts;
+  float* gs = ch + n_experts;
+  float* kept = gs + groups;
+  const int n = min(static_cast<int>(blockIdx.x) * 4 + wave, n_tokens - 1);  // (a wave beyond the tokens repeats the last one)
+  const float* row = logits + static_cast<size_t>(n) * logits_stride;
+  for (int e = lane; e < n_experts; e += kWave) {
+    const float s = 1.f / (1.f + expf(-(bias != nullptr ? row[e] + bias[e] : row[e])));
+    sc[e] = s;
+    ch[e] = correction != nullptr ? s + correction[e] : s;
+  }
+  __syncthreads();
+  // the place of the largest of v[0 .. count), the same in every lane (ties: the lowest; a NaN counts as minus infinity);
+  // it is struck out
+  auto take = [&](float* v, int count) {
+    float best = -INFINITY;
+    int at = 0x7fffffff;
+    for (int e = lane; e < count; e += kWave) {
+      const float x = v[e] == v[e] ? v[e] : -INFINITY;
+      if (at == 0x7fffffff || x > best) best = x, at = e;
+    }
+    for (int off = kWave / 2; off > 0; off /= 2) {
+      const float ov = __shfl_xor(best, off, kWave);
+      const int oe = __shfl_xor(at, off, kWave);
+      if (oe != 0x7fffffff && (at == 0x7fffffff || ov > best || (ov == best && oe < at))) best = ov, at = oe;
+    }
+    __syncthreads();
+    if (lane == 0) v[at] = -INFINITY;
+    __syncthreads();
+    return at;
+  };
+  if (groups > 0) {
+    const int size = n_experts / groups;
+    for (int g = lane; g < groups; g += kWave) {
+      float first = -INFINITY, second = -INFINITY;
+      for (int i = 0; i < size; ++i) {
+        const float v = ch[g * size + i];
+        if (v > first) second = first, first = v;
+        else if (v > second) second = v;
+      }
+      gs[g] = size > 1 ? first + second : first;
+      kept[g] = 0.f;
+    }
+    __syncthreads();
+    for (int k = 0; k < keep; ++k) {
+      const int g = take(gs, groups);
+      if (lane == 0) kept[g] = 1.f;
+    }
+    __syncthreads();
+    for (int e = lane; e < n_experts; e += kWave)
+      if (kept[e / size] == 0.f) ch[e] = -INFINITY;
+    __syncthreads();
+  }
+  float sum = 0.f;
+  int mine = 0;  // (lane k keeps the k-th choice: top is at most a wave's lanes)
+  for (int k = 0; k < top; ++k) {
+    const int e = take(ch, n_experts);
+    sum += sc[e];
+    if (lane == k) mine = e;
+  }
+  if (lane < top && static_cast<int>(blockIdx.x) * 4 + wave < n_tokens) {
+    choice[static_cast<size_t>(n) * top + lane] = mine;
+    weights[static_cast<size_t>(n) * top + lane] = sc[mine] / (sum + 1e-20f);
+  }
+}
+
+extern "C" int yk_moe_router_share(const float* logits, int logits_stride, int n_experts, int top, const float* bias, const float* correction,
+                                   int groups, int keep, int32_t* choice, float* weights, int n_tokens, hipStream_t stream) {
+  YK_REQUIRE(n_tokens >= 0 && n_experts >= 1 && n_experts <= 1024 && top >= 1 && top <= n_experts && top <= 64 && logits_stride >= n_experts,
+             "moe_router_share: bad sizes (up to 1,024 experts, 64 a token)");
+  YK_REQUIRE(groups >= 0 && (groups == 0 || (n_experts % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (n_experts / groups))),
+             "moe_router_share: the kept groups cannot give that many experts");
+  if (n_tokens == 0) return 0;
+  const size_t lds = 4 * 2 * static_cast<size_t>(n_experts + groups) * sizeof(float);
+  moe_router_share_kernel<<<(n_tokens + 3) / 4, 256, lds, stream>>>(logits, logits_stride, n_experts, top, bias, correction, groups, keep, choice,
+                                                                    weights, n_tokens);
+  return yk_check_launch("moe_router_share");
+}
+
 // out[n, :] = dense[n, :] (a tensor, a product's unreduced slices, or nothing) + weight * the sum of the token's `top`
 // rows of rows [tokens * top][width] (each times its own entry of row_weights [tokens * top] where given): what a mixture adds to
 // the stream, as one float32 tensor

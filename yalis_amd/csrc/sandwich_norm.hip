@@ -16,7 +16,7 @@
 // the rows whose logits are wanted.
 //
 // Beside it: an elementwise activation of a product's output (relu squared, silu, gelu) and the
-// multiplication of float32 rows by a constant.
+// multiplication of float32 rows by a constant, with an optional soft cap.
 #include <algorithm>
 
 #include "common.h"
@@ -288,15 +288,19 @@ extern "C" int yk_activation(const void* src, int src_dtype, int n_splits, int r
   return yk_fail("activation: unsupported dtype combination");
 }
 
-__global__ void scale_rows_kernel(float* __restrict__ x, float s, size_t total) {
+// x *= s; with a cap, x = cap tanh(x s / cap)
+__global__ void scale_rows_kernel(float* __restrict__ x, float s, float cap, size_t total) {
   for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < total;
-       i += static_cast<size_t>(gridDim.x) * blockDim.x)
-    x[i] *= s;
+       i += static_cast<size_t>(gridDim.x) * blockDim.x) {
+    const float v = x[i] * s;
+    x[i] = cap > 0.f ? cap * tanhf(v / cap) : v;
+  }
 }
 
-extern "C" int yk_scale_rows(float* x, float s, size_t total, hipStream_t stream) {
+extern "C" int yk_scale_rows(float* x, float s, float cap, size_t total, hipStream_t stream) {
+  YK_REQUIRE(cap >= 0.f, "scale_rows: a cap is positive, 0 for none");
   if (total == 0) return 0;
   const int grid = static_cast<int>(std::min<size_t>((total + 255) / 256, 1 << 20));
-  scale_rows_kernel<<<grid, 256, 0, stream>>>(x, s, total);
+  scale_rows_kernel<<<grid, 256, 0, stream>>>(x, s, cap, total);
   return yk_check_launch("scale_rows");
 }

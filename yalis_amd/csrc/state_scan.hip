@@ -18,6 +18,7 @@
 //   decay per head:     exp(-exp(A_log[h]) * softplus(x[n, h] + dt_bias[h]))
 //   decay per channel:  sigmoid(z[n, h, i] + bias[h, i]) ^ (1 / tau)  =  exp(logsigmoid(.) / tau), or
 //                       exp(-exp(A_log[h]) * softplus(z[n, h, i] + dt_bias[h, i])), or exp(-exp(z[n, h, i] + bias[h, i]))
+//  fixed decay:        a constant of the model per head
 //   beta:               sigmoid(x[n, h])
 //   unit vectors:       q / sqrt(sum q^2 + eps), k likewise (with unit_eps >= 0), then q * q_scale
 // A span cut anywhere gives the same S bit for bit: every token's step is made alone.
@@ -117,7 +118,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
   float* ks = lds;                                        // [chunk][DS]
   float* qs = ks + chunk * DS;                            // [chunk][DS]
   float* as = qs + chunk * DS;                            // [chunk][DS] (per channel) or [chunk]
-  const bool per_channel = decay_mode != 0;
+  const bool per_channel = decay_mode != 0 && decay_mode != 4;
   float* vs = as + chunk * (per_channel ? DS : 1);        // [chunk][cols_per_block]
   float* bs = vs + chunk * cols_per_block;                // [chunk]
   float* kqs = bs + chunk;                                // [chunk]: k . q (times the bonus) of every token, as they enter the recurrence
@@ -191,6 +192,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_kernel(
       const size_t n = static_cast<size_t>(q0 + t0 + t);
       const float step = decay_mode == 0 ? scan_softplus(decay[n * decay_stride + decay_col + h] + decay_p1[h]) : 1.f;
       if (decay_mode == 0) as[t] = expf(-expf(decay_p0[h]) * step);
+      if (decay_mode == 4) as[t] = decay_p0[h];
       float b = write_mode == 2 ? step : 1.f;
       if (delta) b = 1.f / (1.f + expf(-(beta_rows != nullptr ? to_f32<T>(beta_rows[n * beta_stride + beta_col + h]) : beta[n * beta_stride + beta_col + h])));
       bs[t] = b;
@@ -428,7 +430,7 @@ __global__ __launch_bounds__(256) void linear_state_scan_fast_kernel(const T* __
     }
     if (threadIdx.x < nt) {
       const size_t n = n0 + threadIdx.x;
-      if (!CH) s_dec = g.decay[n * g.decay_stride + g.decay_col + h];
+      if (!CH && g.decay_mode == 0) s_dec = g.decay[n * g.decay_stride + g.decay_col + h];
       if (DELTA) s_beta = beta_rows != nullptr ? to_f32<T>(beta_rows[n * g.beta_stride + g.beta_col + h]) : g.beta[n * g.beta_stride + g.beta_col + h];
     }
   };
@@ -458,8 +460,8 @@ __global__ __launch_bounds__(256) void linear_state_scan_fast_kernel(const T* __
         if (i < nt * COLS) vs[i] = to_f32<T>(vv[j]);
       }
       if (threadIdx.x < nt) {
-        const float step = CH ? 1.f : scan_softplus(s_dec + g.decay_p1[h]);
-        if (!CH) sc[4 * threadIdx.x] = expf(-expf(g.decay_p0[h]) * step);
+        const float step = CH || g.decay_mode != 0 ? 1.f : scan_softplus(s_dec + g.decay_p1[h]);
+        if (!CH) sc[4 * threadIdx.x] = g.decay_mode == 4 ? g.decay_p0[h] : expf(-expf(g.decay_p0[h]) * step);
         sc[4 * threadIdx.x + 1] = DELTA ? 1.f / (1.f + expf(-s_beta)) : (g.by_step ? step : 1.f);
       }
       if (CH && !g.given) {
@@ -592,7 +594,7 @@ __global__ __launch_bounds__(256) void channel_decay_kernel(const float* __restr
 // decay_mode 0: one decay per head from decay[n, decay_col + h], p0 = A_log [heads], p1 = dt_bias [heads];
 // decay_mode 1, 2, 3: one per key channel from z = decay[n, decay_col + h * dim + i]: 1, sigmoid(z + p0)^(1 / tau), p0 =
 // bias [heads * dim]; 2, exp(-exp(p0[h]) softplus(z + p1)), p0 = A_log [heads], p1 = dt_bias [heads * dim]; 3,
-// exp(-exp(z + p0)), p0 = bias [heads * dim].
+// exp(-exp(z + p0)), p0 = bias [heads * dim]; decay_mode 4: p0[h] itself, a constant per head (nothing is read per token).
 // beta (float32) or, in its place, beta_rows (of qkv's dtype), both read at [n, beta_col + h].  bonus [heads * dim]
 // float32 or null: the read-out comes before the write, with the token's own write weighed by the bonus (plain writes).
 // decays [n_tokens][heads * dim] float32 or null: room for the decays per channel, made first where tokens are many.
@@ -612,12 +614,13 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
              "linear_state_scan: rows shorter than q, k and v");
   YK_REQUIRE(write_mode == 0 || (write_mode == 1 && (beta != nullptr || beta_rows != nullptr)) || (write_mode == 2 && decay_mode == 0),
              "linear_state_scan: the delta rule needs beta, a write by the step the decay per head");
-  YK_REQUIRE(decay_mode >= 0 && decay_mode <= 3, "linear_state_scan: unknown kind of decay");
+  YK_REQUIRE(decay_mode >= 0 && decay_mode <= 4, "linear_state_scan: unknown kind of decay");
   YK_REQUIRE(bonus == nullptr || (write_mode == 0 && skip == nullptr), "linear_state_scan: a bonus goes with plain writes and no skip");
-  YK_REQUIRE(decay != nullptr && decay_p0 != nullptr && (decay_mode == 1 || decay_mode == 3 || decay_p1 != nullptr), "linear_state_scan: the decay's inputs are missing");
+  YK_REQUIRE(decay_p0 != nullptr && (decay_mode == 4 || (decay != nullptr && (decay_mode == 1 || decay_mode == 3 || decay_p1 != nullptr))), "linear_state_scan: the decay's inputs are missing");
   YK_REQUIRE(decay_mode != 1 || tau > 0.f, "linear_state_scan: tau must be positive");
   YK_REQUIRE(dim <= kScanRowsMax * kWave, "linear_state_scan: heads of more than 1,024 key channels are not offered");
   if (n_seqs == 0) return 0;
+  const bool per_channel = decay_mode != 0 && decay_mode != 4;
   // eight rows a lane while that leaves a column inside a wave (a wave's instructions per token are what
   // the walk costs: fewer rows a lane, more lanes a column), sixteen beyond
   // (steps of single tokens are all staging and no walk: there the fewer, larger workgroups of sixteen rows
@@ -631,17 +634,17 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
   dim3 grid(n_seqs, n_heads, (vdim + cols - 1) / cols);
   const size_t dp = static_cast<size_t>(tpc) * rows;
   int chunk = kScanTokens;
-  const size_t per_token = sizeof(float) * (2 * (dp + 4) + (decay_mode != 0 ? dp + 4 : 1) + cols + 2);
+  const size_t per_token = sizeof(float) * (2 * (dp + 4) + (per_channel ? dp + 4 : 1) + cols + 2);
   while (chunk > 4 && (chunk * per_token > 110 * 1024 || chunk * dp > 8192)) chunk /= 2;
   const size_t lds = chunk * per_token + (bonus != nullptr ? (dp + 4) * sizeof(float) : 0);
   YK_REQUIRE(lds <= 128 * 1024, "linear_state_scan: the staged tokens do not fit in LDS");
   auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
-  const int kind = (decay_mode != 0 ? kScanChannel : 0) + (write_mode == 1 ? kScanDelta : 0) + (bonus != nullptr ? kScanReadFirst : 0);
+  const int kind = (per_channel ? kScanChannel : 0) + (write_mode == 1 ? kScanDelta : 0) + (bonus != nullptr ? kScanReadFirst : 0);
   const bool fast = dim % 8 == 0 && qkv_stride % 8 == 0 && q_col % 8 == 0 && k_col % 8 == 0 && al16(qkv) && chunk * dp <= 8192 && kind != kScanReadFirst &&
                     (skip == nullptr || kind == 0);
   if (fast) {
     // many tokens: their decays per channel first, where the caller gave room for them
-    const bool given = decay_mode != 0 && decays != nullptr && decay_stride % 4 == 0 && decay_col % 4 == 0 && al16(decay) && al16(decays) &&
+    const bool given = per_channel && decays != nullptr && decay_stride % 4 == 0 && decay_col % 4 == 0 && al16(decay) && al16(decays) &&
                        al16(decay_mode == 2 ? decay_p1 : decay_p0);
     if (given) {
       const size_t total4 = static_cast<size_t>(n_tokens) * n_heads * dim / 4;
@@ -652,7 +655,7 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
     const ScanArgs g{seq_qstart, seq_qlen, state_slots, qkv_stride, n_heads, n_kv, dim, vdim, q_col, k_col, v_col, q_scale, unit_eps,
                      decay_mode, given, given ? decays : decay, given ? n_heads * dim : decay_stride, given ? 0 : decay_col, decay_p0, decay_p1, tau,
                      beta, beta_stride, beta_col, write_mode == 2, skip, bonus, chunk};
-    const size_t fast_lds = sizeof(float) * ((chunk + 2) * ((decay_mode != 0 ? 3 : 2) * (dp + 4) + 4 + cols) + dp);
+    const size_t fast_lds = sizeof(float) * ((chunk + 2) * ((per_channel ? 3 : 2) * (dp + 4) + 4 + cols) + dp);
     YK_REQUIRE(fast_lds <= 128 * 1024, "linear_state_scan: the staged tokens do not fit in LDS");
 #define YK_FAST(T, TPC, KIND)                                                                                                   \
   {                                                                                                                             \
@@ -717,10 +720,60 @@ extern "C" int yk_linear_state_scan(const void* qkv, int qkv_stride, int dtype, 
   return yk_fail("linear_state_scan: unsupported dtype");
 }
 
+// ------------------------------------------------------------------------ what enters a recurrence
+// float32 rows [q | k | v] from a projection's rows [q | k | v | ...]: with silu, the activation of all three; with tables,
+// q and k rotated by their positions (the first `rot` elements of every head); k times k_scale.  A thread an element.
+template <typename T>
+__global__ __launch_bounds__(256) void scan_inputs_kernel(const T* __restrict__ src, int src_stride, int n_heads, int dim, int vdim,
+                                                          const int32_t* __restrict__ positions, const float* __restrict__ cos_t,
+                                                          const float* __restrict__ sin_t, int rot, int interleaved, int max_pos,
+                                                          float k_scale, int silu, float* __restrict__ out, size_t total) {
+  const int kd = n_heads * dim, cols = 2 * kd + n_heads * vdim;
+  for (size_t i = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; i < total; i += static_cast<size_t>(gridDim.x) * blockDim.x) {
+    const size_t n = i / cols;
+    const int c = static_cast<int>(i % cols);
+    const T* row = src + n * src_stride;
+    auto at = [&](int col) { const float x = to_f32<T>(row[col]); return silu ? act_silu(x) : x; };
+    float v = at(c);
+    if (c < 2 * kd) {
+      const int d = c % dim;
+      if (d < rot) {
+        const int half = rot / 2, m = interleaved ? d / 2 : (d < half ? d : d - half);
+        const size_t a = static_cast<size_t>(min(positions[n], max_pos - 1)) * half + m;
+        const bool first = interleaved ? d % 2 == 0 : d < half;
+        const float other = at(interleaved ? (first ? c + 1 : c - 1) : (first ? c + half : c - half));
+        v = first ? rot_first(v, other, cos_t[a], sin_t[a]) : rot_second(other, v, cos_t[a], sin_t[a]);
+      }
+      if (c >= kd) v *= k_scale;
+    }
+    out[i] = v;
+  }
+}
+
+extern "C" int yk_scan_inputs(const void* src, int src_stride, int dtype, int n_heads, int dim, int vdim, const int32_t* positions,
+                              const float* cos_t, const float* sin_t, int rot, int interleaved, int max_pos, float k_scale, int silu,
+                              float* out, int n_tokens, hipStream_t stream) {
+  YK_REQUIRE(n_tokens >= 0 && n_heads > 0 && dim > 0 && vdim > 0 && src_stride >= n_heads * (2 * dim + vdim), "scan_inputs: bad sizes");
+  YK_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dim && (rot == 0 || (cos_t != nullptr && sin_t != nullptr && positions != nullptr && max_pos > 0)),
+             "scan_inputs: rotary tables missing, or more elements than a head has");
+  if (n_tokens == 0) return 0;
+  const size_t total = static_cast<size_t>(n_tokens) * n_heads * (2 * dim + vdim);
+  const int grid = static_cast<int>(std::min<size_t>((total + 255) / 256, 1 << 20));
+  if (dtype == YK_F32)
+    scan_inputs_kernel<float><<<grid, 256, 0, stream>>>(static_cast<const float*>(src), src_stride, n_heads, dim, vdim, positions, cos_t, sin_t, rot,
+                                                        interleaved, max_pos, k_scale, silu, out, total);
+  else if (dtype == YK_BF16)
+    scan_inputs_kernel<bf16_t><<<grid, 256, 0, stream>>>(static_cast<const bf16_t*>(src), src_stride, n_heads, dim, vdim, positions, cos_t, sin_t, rot,
+                                                         interleaved, max_pos, k_scale, silu, out, total);
+  else
+    return yk_fail("scan_inputs: unsupported dtype");
+  return yk_check_launch("scan_inputs");
+}
+
 // --------------------------------------------------------------- the read-out's norm and gate
 // a wave per (token, part of vdim elements): y = o / sqrt(mean(o^2) + eps) * w * silu(gate), or, gate_first, the gate
 // before the norm: y = g / sqrt(mean(g^2) + eps) * w with g = o * silu(gate).  gate_act 1: the sigmoid in silu's place.  w_stride 0: one weight of vdim elements
-// for every part; vdim: a weight of n_heads * vdim elements.
+// for every part; vdim: a weight of n_heads * vdim elements; w null: no weight.
 __device__ __forceinline__ float head_gate_act(float g, int act) { return act == 1 ? 1.f / (1.f + expf(-g)) : act_silu(g); }
 template <typename TW, typename TG, typename TO>
 __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __restrict__ o, const TW* __restrict__ w, float eps,
@@ -734,7 +787,8 @@ __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __res
   const int h = static_cast<int>(item % n_heads);
   const float* row = o + item * vdim;
   const TG* g = gate + n * gate_stride + gate_col + h * vdim;
-  const TW* wp = w + static_cast<size_t>(h) * w_stride;
+  const TW* wp = w != nullptr ? w + static_cast<size_t>(h) * w_stride : nullptr;
+  auto weight = [&](int c) { return wp != nullptr ? to_f32<TW>(wp[c]) : 1.f; };
   float ss = 0.f;
   if (gate_first) {
     for (int c = lane; c < vdim; c += kWave) {
@@ -743,13 +797,13 @@ __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __res
     }
     const float inv = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(vdim) + eps);
     for (int c = lane; c < vdim; c += kWave)
-      out[item * vdim + c] = from_f32<TO>(row[c] * head_gate_act(to_f32<TG>(g[c]), gate_act) * inv * to_f32<TW>(wp[c]));
+      out[item * vdim + c] = from_f32<TO>(row[c] * head_gate_act(to_f32<TG>(g[c]), gate_act) * inv * weight(c));
     return;
   }
   for (int c = lane; c < vdim; c += kWave) ss = fmaf(row[c], row[c], ss);
   const float inv = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(vdim) + eps);
   for (int c = lane; c < vdim; c += kWave)
-    out[item * vdim + c] = from_f32<TO>(row[c] * inv * to_f32<TW>(wp[c]) * head_gate_act(to_f32<TG>(g[c]), gate_act));
+    out[item * vdim + c] = from_f32<TO>(row[c] * inv * weight(c) * head_gate_act(to_f32<TG>(g[c]), gate_act));
 }
 
 extern "C" int yk_gated_head_norm(const float* o, const void* w, int w_dtype, float eps, const void* gate, int gate_dtype,

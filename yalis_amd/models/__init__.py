@@ -1,2 +1,2 @@
 """Architectures.  Importing the package registers the ones it ships."""
-from . import bekedra, llama, mesolix, nutavik, rafusun, suranex  # noqa: F401
+from . import bekedra, llama, mesolix, nutavik, rafusun, suranex, zimupel  # noqa: F401

@@ -85,7 +85,7 @@ _SIGNATURES = {
     "yk_qkv_prepare": (
         [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _c_int,
          _c_int, _c_float, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_float, _vp, _vp, _c_int, _c_int, _vp, _vp, _vp, _c_int,
-         _c_int, _vp, _vp, _c_int, _vp],
+         _c_int, _vp, _vp, _c_int, _c_int, _vp],
         _c_int,
     ),
     "yk_qk_row_scales": (
@@ -95,7 +95,7 @@ _SIGNATURES = {
     "yk_attn_masked": (
         [_vp, _c_int, _vp, _vp, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
          _c_float, _c_int, _c_int, _c_int, _vp, _vp, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _vp,
-         _c_int, _vp, _c_int, _vp],
+         _c_int, _vp, _c_int, _c_int, _c_float, _c_float, _c_float, _vp],
         _c_int,
     ),
     "yk_attn_finish": (
@@ -110,7 +110,18 @@ _SIGNATURES = {
         _c_int,
     ),
     "yk_activation": ([_vp, _c_int, _c_int, _c_int, _c_int, _vp, _c_int, _c_size_t, _vp], _c_int),
-    "yk_scale_rows": ([_vp, _c_float, _c_size_t, _vp], _c_int),
+    "yk_scale_rows": ([_vp, _c_float, _c_float, _c_size_t, _vp], _c_int),
+    "yk_embed_norm": ([_vp, _vp, _c_int, _c_int, _vp, _c_float, _vp, _c_int, _c_int, _c_int, _vp], _c_int),
+    "yk_streams_norm": (
+        [_vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_float, _vp, _vp, _vp, _vp, _vp, _vp, _c_int, _c_float,
+         _c_int, _vp, _c_int, _c_int, _vp],
+        _c_int,
+    ),
+    "yk_scan_inputs": (
+        [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_float, _c_int, _vp, _c_int, _vp],
+        _c_int,
+    ),
+    "yk_moe_router_share": ([_vp, _c_int, _c_int, _c_int, _vp, _vp, _c_int, _c_int, _vp, _vp, _c_int, _vp], _c_int),
     "yk_latent_prepare": (
         [_vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_float, _vp, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp, _vp,
          _c_int, _vp, _c_int, _vp],
@@ -197,11 +208,13 @@ _SIGNATURES = {
     "yk_attn_tokens_per_tile": ([_c_int, _c_int], _c_int),
     "yk_attn_mfma_workspace": ([_c_int, _c_int, _c_int, _c_int, _c_int], _c_size_t),
     "yk_attn_mfma_prefill": (
-        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _c_int, _vp],
+        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _c_int,
+         _c_int, _c_float, _c_float, _c_float, _vp],
         _c_int,
     ),
     "yk_attn_mfma": (
-        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _c_int, _vp],
+        [_vp, _c_int, _vp, _vp, _vp, _vp, _c_int, _vp, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_int, _c_int, _vp, _c_size_t, _c_int, _c_int, _c_float, _vp, _c_int, _vp, _c_int,
+         _c_int, _c_float, _c_float, _c_float, _vp],
         _c_int,
     ),
     "yk_attn_mfma_rope": (
@@ -230,7 +243,7 @@ _LATER_SIGNATURES = {
         "yk_probe_mfma_bf16": ([_c_int, _c_int, _vp, _vp], _c_int),
     },
 }
-_ABI = 23
+_ABI = 24
 
 # Rows of x up to which the hand-written matrix-core kernel runs a bfloat16 product;
 # above it the vendor library does.
@@ -958,10 +971,15 @@ class HipOps:
         ``attention_masked``'s)."""
         return self.attention_can_rotate(act_dtype, head_dim)
 
+    def attention_takes_maps(self, act_dtype: torch.dtype, head_dim: int) -> bool:
+        """Whether ``attention`` takes ``differential=`` where both maps of a head together are ``head_dim`` wide."""
+        return self.attention_can_rotate(act_dtype, head_dim)
+
     def attention(self, qkv, n_heads, n_kv, head_dim, k_cache, v_cache, page_size,
                   scale, window, ctx, group, tiles, long_tiles=None, plan=None, long_plan=None,
                   long_col_tiles: int = 1, token_cols=None, rope: Optional["RopeInLaunch"] = None,
-                  keep_first: int = 0, softcap: float = 0.0, distance_bias=None, sink=None, chunked: bool = False):
+                  keep_first: int = 0, softcap: float = 0.0, distance_bias=None, sink=None, chunked: bool = False,
+                  differential=None):
         """Queries are the first n_heads heads of each row of ``qkv`` (whatever follows
         them in the row is skipped); keys and values come from the cache through the
         block table of ``group``.  ``long_tiles`` hold up to
@@ -976,6 +994,10 @@ class HipOps:
         are squashed to softcap * tanh(s / softcap); ``distance_bias`` (float32 [distances, n_heads]): row
         min(p - j, distances - 1) is added to head h's scaled (and squashed) score of key j for the query at p;
         ``chunked``: the window begins anew at every multiple of its size instead of sliding.
+
+        ``differential`` (lambda, eps, gain; matrix-core kernels only): every head brings two query rows, one per map with
+        zeros where the other map's keys are (``qkv_prepare(query_maps=2)``; ``n_heads`` counts these rows), and the result
+        [N, n_heads / 2 * head_dim] is (a1 - lambda a2) divided by its root mean square per head and times gain.
 
         ``rope`` (only where ``attention_can_rotate``, and only for steps whose spans are single
         tokens): ``qkv`` is then the projection's raw output (a tensor or a ``SplitSum``) and
@@ -992,14 +1014,18 @@ class HipOps:
             raise KernelError(f"cache pages have shapes {tuple(k_cache.shape)}, {tuple(v_cache.shape)}")
         if k_cache.dtype != qkv.dtype:
             raise KernelError("cache and activations differ in dtype")
-        out = torch.empty((n, n_heads * head_dim), dtype=qkv.dtype, device=qkv.device)
+        maps = 1 if differential is None else 2
+        lam, map_eps, gain = (0.0, 0.0, 1.0) if differential is None else (float(v) for v in differential)
+        if maps == 2 and (n_heads % (2 * n_kv) or sink is not None or distance_bias is not None):
+            raise KernelError("attention: two maps are two query rows a head, without sinks and biases per distance")
+        out = torch.empty((n, n_heads // maps * head_dim), dtype=qkv.dtype, device=qkv.device)
         use_mfma = (
             qkv.dtype == torch.bfloat16
             and self._ask("yk_attn_mfma_supported", head_dim)
             and qkv.stride(0) % 8 == 0
             and qkv.data_ptr() % 16 == 0
         )
-        if (keep_first or softcap or distance_bias is not None or sink is not None or chunked) and not use_mfma:
+        if (keep_first or softcap or distance_bias is not None or sink is not None or chunked or maps == 2) and not use_mfma:
             raise KernelError("attention: kept first keys, chunks, squashed scores, biases per distance and sinks outside the matrix-core kernels' sizes are attention_masked's")
         # keys any query of the step reads at most (a chunk's queries read no other chunk's)
         reach = min(ctx.max_ctx, int(window)) if chunked else ctx.max_ctx
@@ -1022,7 +1048,7 @@ class HipOps:
                     long_tiles.data_ptr(), n_long, bt.data_ptr(), bt.shape[1], page_size, head_dim,
                     n_heads, n_kv, float(scale), int(window), long_splits, int(long_col_tiles), _ptr(ws),
                     0 if ws is None else ws.numel(), int(self.long_span_pages_in_lds), int(keep_first), float(softcap),
-                    _ptr(distance_bias), bias_rows, _ptr(sink), int(bool(chunked)), self._stream(),
+                    _ptr(distance_bias), bias_rows, _ptr(sink), int(bool(chunked)), maps, lam, map_eps, gain, self._stream(),
                 )
             )
         if use_mfma and tiles.shape[0] == 0:
@@ -1036,13 +1062,14 @@ class HipOps:
             ws_floats = self._ask("yk_attn_mfma_workspace", n_tiles, n_heads, n_kv, head_dim, splits)
             ws = self._ws(ws_floats) if ws_floats else None
             leave = bool(token_cols is not None and splits > 1 and n <= MERGE_IN_PRODUCT_MAX_TOKENS and (long_tiles is None or long_tiles.shape[0] == 0)
-                         and sink is None)  # (a sink joins in the merge kernel)
+                         and sink is None and maps == 1)  # (a sink joins, and maps meet, in the merge kernel)
             self._check(
                 self.lib.yk_attn_mfma(
                     qkv.data_ptr(), qkv.stride(0), out.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                     tiles.data_ptr(), n_tiles, bt.data_ptr(), bt.shape[1], page_size, head_dim, n_heads, n_kv,
                     float(scale), int(window), waves, splits, _ptr(ws), 0 if ws is None else ws.numel(), int(leave),
-                    int(keep_first), float(softcap), _ptr(distance_bias), bias_rows, _ptr(sink), int(bool(chunked)), self._stream(),
+                    int(keep_first), float(softcap), _ptr(distance_bias), bias_rows, _ptr(sink), int(bool(chunked)),
+                    maps, lam, map_eps, gain, self._stream(),
                 )
             )
             if leave:
@@ -1245,7 +1272,8 @@ class HipOps:
     def qkv_prepare(self, qkv, n_heads, n_kv, head_dim, value_dim, positions, act_dtype, q_norm=None, k_norm=None,
                     qk_eps: float = 0.0, rotation=None, value_norm_eps=None, value_rotation=None,
                     k_cache=None, v_cache=None, slots=None, page_size: int = 0, bias=None, row_scales=None,
-                    norm_over_projection: bool = False, values_from_keys: bool = False, unweighted_norm: bool = False) -> torch.Tensor:
+                    norm_over_projection: bool = False, values_from_keys: bool = False, unweighted_norm: bool = False,
+                    query_maps: int = 1) -> torch.Tensor:
         """From a projection's rows [q | k | v | ...] (a tensor or a ``SplitSum``): normed (weights
         ``q_norm`` / ``k_norm`` of head_dim elements, or none) and rotated queries [N, n_heads * head_dim];
         normed, rotated keys and unit-normed (``value_norm_eps``), rotated (``value_rotation``) values
@@ -1254,7 +1282,9 @@ class HipOps:
         projected (biased, before the norm).  ``norm_over_projection``: the weights are as wide as the q (k)
         projection and no root mean square is taken here: it comes with ``row_scales`` (float32 [N, 2], from
         ``qk_row_scales``), which multiply a token's queries (column 0) and keys (column 1) after the weights.
-        ``unweighted_norm``: every head is divided by its root mean square (``qk_eps`` under the root) and that is all."""
+        ``unweighted_norm``: every head is divided by its root mean square (``qk_eps`` under the root) and that is all.
+        ``query_maps`` = m > 1: a head's elements are m maps side by side, and the queries come as [N, n_heads * m * head_dim],
+        a row per head and map with zeros where the other maps' elements are."""
         n_splits, round_sum, src = 1, 0, qkv
         if isinstance(qkv, SplitSum):
             qkv.check_live()
@@ -1277,7 +1307,9 @@ class HipOps:
             raise KernelError("qkv_prepare: a norm over the whole projection takes its weights and the rows' scales")
         if positions.numel() != n or (n_kv > 0 and slots.numel() != n):
             raise KernelError("positions/slots do not match the number of tokens")
-        q_out = torch.empty((n, n_heads * head_dim), dtype=act_dtype, device=src.device)
+        if query_maps < 1 or head_dim % query_maps:
+            raise KernelError(f"qkv_prepare: heads of {head_dim} do not divide into {query_maps} maps")
+        q_out = torch.empty((n, n_heads * query_maps * head_dim), dtype=act_dtype, device=src.device)
         tiled = False
         if n_kv > 0:
             if k_cache.dtype != act_dtype or v_cache.dtype != act_dtype:
@@ -1318,7 +1350,7 @@ class HipOps:
                 int(bool(value_rotation is not None and value_rotation.interleaved)),
                 0 if value_rotation is None else value_rotation.cos.shape[0],
                 _ptr(k_cache) if n_kv else None, _ptr(v_cache) if n_kv else None, _ptr(slots) if n_kv else None,
-                int(page_size), int(tiled), _ptr(bias), _ptr(row_scales), int(bool(values_from_keys)), self._stream(),
+                int(page_size), int(tiled), _ptr(bias), _ptr(row_scales), int(bool(values_from_keys)), int(query_maps), self._stream(),
             )
         )
         return q_out
@@ -1362,7 +1394,7 @@ class HipOps:
     def attention_masked(self, q, n_heads, n_kv, head_dim, value_dim, k_cache, v_cache, page_size, scale, ctx, group,
                          window: int = 0, keep_first: int = 0, softcap: float = 0.0, value_rotation=None,
                          gate=None, gate_col: int = 0, gate_elems: int = 1, distance_bias=None, sink=None,
-                         chunked: bool = False) -> torch.Tensor:
+                         chunked: bool = False, differential=None) -> torch.Tensor:
         """softmax over the keys j <= p with (p - j < window or j < keep_first) of q . k * scale
         (squashed by ``softcap`` * tanh(s / ``softcap``) when set), times the values [N, n_heads *
         value_dim]; then, with ``value_rotation``, every head's output turned back by its token's
@@ -1371,7 +1403,12 @@ class HipOps:
         a gate per output element, in the columns ``gate_col`` + h * value_dim + d).  ``distance_bias`` (float32
         [distances, n_heads]): row min(p - j, distances - 1) is added to the scaled scores of head h.  ``sink`` (float32
         [n_heads]): exp(sink[h]) joins head h's denominator once; it has no key and no value.  ``chunked``: the window
-        begins anew at every multiple of its size (keys j with floor(j / window) = floor(p / window))."""
+        begins anew at every multiple of its size (keys j with floor(j / window) = floor(p / window)).  ``differential``
+        (lambda, eps, gain): a head's queries and keys are two maps side by side, each with a softmax of its own over its
+        half's scores; the head's output is (a1 - lambda a2) divided by its root mean square and times gain."""
+        if differential is not None and (head_dim % 2 or sink is not None or distance_bias is not None):
+            raise KernelError("attention_masked: two maps divide a head in halves and go without sinks and biases per distance")
+        lam, map_eps, gain = (0.0, 0.0, 1.0) if differential is None else (float(v) for v in differential)
         self._rows(q, "queries")
         if sink is not None and (sink.dtype != torch.float32 or sink.numel() != n_heads or not sink.is_contiguous()):
             raise KernelError("attention_masked: the sinks are contiguous float32 [heads]")
@@ -1396,7 +1433,8 @@ class HipOps:
                 None if vr is None else vr.cos.data_ptr(), None if vr is None else vr.sin.data_ptr(),
                 int(bool(vr is not None and vr.interleaved)), 0 if vr is None else vr.cos.shape[0],
                 _ptr(gsrc), 0 if gsrc is None else _code(gsrc.dtype), gsplits, ground, gstride, int(gate_col), int(gate_elems),
-                _ptr(distance_bias), 0 if distance_bias is None else distance_bias.shape[0], _ptr(sink), int(bool(chunked)), self._stream(),
+                _ptr(distance_bias), 0 if distance_bias is None else distance_bias.shape[0], _ptr(sink), int(bool(chunked)),
+                1 if differential is None else 2, lam, map_eps, gain, self._stream(),
             )
         )
         return out
@@ -1514,12 +1552,62 @@ class HipOps:
                                            out.data_ptr(), _code(out_dtype), out.numel(), self._stream()))
         return out
 
-    def scale_rows(self, x: torch.Tensor, s: float) -> torch.Tensor:
-        """x (contiguous float32) *= s, in place."""
+    def scale_rows(self, x: torch.Tensor, s: float, softcap: float = 0.0) -> torch.Tensor:
+        """x (contiguous float32) *= s, in place; with ``softcap`` c, x = c tanh(s x / c)."""
         if x.dtype != torch.float32 or not x.is_contiguous():
             raise KernelError("scale_rows takes a contiguous float32 tensor")
-        self._check(self.lib.yk_scale_rows(x.data_ptr(), float(s), x.numel(), self._stream()))
+        self._check(self.lib.yk_scale_rows(x.data_ptr(), float(s), float(softcap), x.numel(), self._stream()))
         return x
+
+    # ------------------------------------------------------------- a stream kept as several copies
+    def embed_norm(self, token_ids, table, weight, eps, copies: int) -> torch.Tensor:
+        """float32 [N, copies, width]: table[id] divided by its root mean square and times ``weight``, the same in every copy."""
+        if table.dim() != 2 or not table.is_contiguous() or weight.dtype != table.dtype or weight.numel() != table.shape[1] or not weight.is_contiguous():
+            raise KernelError("embed_norm: a contiguous table and a weight as wide as its rows, of one dtype")
+        if token_ids.dtype != torch.int32:
+            raise KernelError("embed_norm: token ids are int32")
+        n, width = token_ids.numel(), table.shape[1]
+        out = torch.empty((n, int(copies), width), dtype=torch.float32, device=table.device)
+        self._check(self.lib.yk_embed_norm(token_ids.data_ptr(), table.data_ptr(), _code(table.dtype), table.shape[0], weight.data_ptr(), float(eps),
+                                           out.data_ptr(), n, width, int(copies), self._stream()))
+        return out
+
+    def streams_norm(self, residual, y, experts, mix, out, read, rows, weight, eps, unit_offset, out_dtype) -> torch.Tensor:
+        """``residual`` float32 [N, streams, width], in place: x_t <- sum_s mix[s, t] x_s + out[t] b, where b is ``y`` (a tensor, a
+        ``SplitSum`` or None) plus, with ``experts`` = (rows, top, weight, row weights or None), a mixture's uncombined rows as
+        ``moe_combine`` sums them; ``mix`` [streams, streams] and ``out`` [streams] float32, None: nothing is pending.  Returns
+        norm(sum_s read[s] x_s) * weight in ``out_dtype`` (``read`` None: the plain sum).  With ``rows`` (int32) those
+        tokens' rows only, and the residual is left as it is."""
+        if residual.dim() != 3 or residual.dtype != torch.float32 or not residual.is_contiguous():
+            raise KernelError("streams_norm: the copies are contiguous float32 [N, streams, width]")
+        n, streams, width = residual.shape
+        for t, count in ((mix, streams * streams), (out, streams), (read, streams)):
+            if t is not None and (t.dtype != torch.float32 or t.numel() != count or not t.is_contiguous()):
+                raise KernelError("streams_norm: the tables are contiguous float32 [streams, streams] and [streams]")
+        if weight.numel() != width or not weight.is_contiguous() or (mix is None) != (out is None):
+            raise KernelError(f"streams_norm: the norm's weight has {weight.numel()} elements, rows have {width}")
+        if isinstance(y, SplitAttention):
+            y = y.merge()
+        n_splits, round_sum, src = 1, 0, y
+        if isinstance(y, SplitSum):
+            y.check_live()
+            n_splits, round_sum, src = y.n_splits, y.round_sum, y.tensor
+        if y is not None and (tuple(y.shape) != (n, width) or not src.is_contiguous()):
+            raise KernelError(f"streams_norm: the branch {tuple(y.shape)} does not match the stream {(n, width)}")
+        erows, top, eweight, rweights = experts if experts is not None else (None, 0, 1.0, None)
+        if erows is not None and (erows.dtype != torch.float32 or not erows.is_contiguous() or tuple(erows.shape) != (n * top, width)):
+            raise KernelError(f"streams_norm: expert rows {tuple(erows.shape)} do not match the stream {(n, width)}")
+        if rweights is not None and (rweights.dtype != torch.float32 or rweights.numel() != n * top or not rweights.is_contiguous()):
+            raise KernelError("streams_norm: the rows' weights are contiguous float32, one per row")
+        if rows is not None and rows.dtype != torch.int32:
+            raise KernelError("streams_norm: picked rows are int32")
+        n_out = n if rows is None else rows.numel()
+        h = torch.empty((n_out, width), dtype=out_dtype, device=residual.device)
+        self._check(self.lib.yk_streams_norm(
+            residual.data_ptr(), n, streams, width, _ptr(src), 0 if src is None else _code(src.dtype), n_splits, round_sum, _ptr(erows), int(top),
+            float(eweight), _ptr(rweights), _ptr(mix), _ptr(out), _ptr(read), _ptr(rows), weight.data_ptr(), _code(weight.dtype), float(eps),
+            int(bool(unit_offset)), h.data_ptr(), _code(out_dtype), n_out, self._stream()))
+        return h
 
     # ------------------------------------------------------------- attention over one latent per token
     def latent_prepare(self, proj, q_rank, q_norm, eps, act_dtype, kv_col=0, kv_rank=0, rot_dim=0, kv_norm=None, rotation=None,
@@ -1683,7 +1771,7 @@ class HipOps:
         exp(-exp(A_log) softplus(x[:, col + h] + dt_bias)); ("channel", z, col, bias, tau): a_i = sigmoid(z[:,
         col + h * dim + i] + bias)^(1 / tau); ("channel_softplus", z, col, A_log, dt_bias): a_i = exp(-exp(A_log_h)
         softplus(z[:, col + h * dim + i] + dt_bias)); ("channel_exp", z, col, bias): a_i = exp(-exp(z[:, col + h * dim + i] +
-        bias)); x, z float32.  ``beta``: (x, col) -> sigmoid(x[:, col + h]), x float32 or of ``qkv``'s dtype, or
+        bias)); x, z float32; ("fixed", a): a constant per head, a float32 [heads].  ``beta``: (x, col) -> sigmoid(x[:, col + h]), x float32 or of ``qkv``'s dtype, or
         None for plain writes, or "step": u = dt v with the step dt = softplus(x[:, col + h] + dt_bias) of the head's
         decay.  ``columns`` = (q, k, v): where the kv heads' queries and keys and the heads' values start in a row
         (default 0, n_kv * dim, 2 * n_kv * dim).  ``skip`` (float32 [heads]): o += skip_h v.  ``bonus`` (float32
@@ -1693,6 +1781,8 @@ class HipOps:
         n = qkv.shape[0]
         if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (n_heads, dim, vdim):
             raise KernelError(f"linear_state_scan: state {tuple(state.shape)} does not hold {n_heads} matrices of {dim} x {vdim}")
+        if decay[0] == "fixed":
+            decay = ("fixed", None, 0, decay[1])
         kind, src, col = decay[0], decay[1], int(decay[2])
         need = n_heads if kind == "head" else n_heads * dim
         write_mode = 0 if beta is None else (2 if isinstance(beta, str) else 1)
@@ -1705,7 +1795,7 @@ class HipOps:
             raise KernelError("linear_state_scan: the skip is contiguous float32, one number per head")
         if bonus is not None and (bonus.dtype != torch.float32 or bonus.numel() != n_heads * dim or not bonus.is_contiguous() or write_mode or skip is not None):
             raise KernelError("linear_state_scan: the bonus is contiguous float32 [heads, dim] and goes with plain writes and no skip")
-        for t, what, cols in ((src, "decay", col + need),) + (((beta[0], "beta", int(beta[1]) + n_heads),) if beta is not None else ()):
+        for t, what, cols in (((src, "decay", col + need),) if src is not None else ()) + (((beta[0], "beta", int(beta[1]) + n_heads),) if beta is not None else ()):
             if (t.dtype != torch.float32 and not (what == "beta" and t.dtype == qkv.dtype)) or t.dim() != 2 or t.stride(1) != 1 or t.shape[0] != n or t.shape[1] < cols:
                 raise KernelError(f"linear_state_scan: the {what}'s input must be float32 rows of at least {cols} columns")
         if kind == "head":
@@ -1720,30 +1810,62 @@ class HipOps:
         elif kind == "channel_exp":
             p0, p1, tau = decay[3], None, 1.0
             ok = p0.dtype == torch.float32 and p0.numel() == n_heads * dim and p0.is_contiguous()
+        elif kind == "fixed":
+            p0, p1, tau = decay[3], None, 1.0
+            ok = p0.dtype == torch.float32 and p0.numel() == n_heads and p0.is_contiguous()
         else:
             raise KernelError(f"linear_state_scan: unknown kind of decay {kind!r}")
         if not ok:
             raise KernelError("linear_state_scan: the decay's constants must be contiguous float32 of the heads' size")
         a = ctx.arrays
-        mode = {"head": 0, "channel": 1, "channel_softplus": 2, "channel_exp": 3}[kind]
+        mode = {"head": 0, "channel": 1, "channel_softplus": 2, "channel_exp": 3, "fixed": 4}[kind]
         beta_f32 = beta is not None and beta[0].dtype == torch.float32
         # where tokens are many their decays per channel are made first, once for all the columns that read them
-        many = mode != 0 and n > 4 * a["seq_qstart"].numel()
+        many = mode not in (0, 4) and n > 4 * a["seq_qstart"].numel()
         decays = torch.empty((n, n_heads * dim), dtype=torch.float32, device=qkv.device) if many else None
         out = torch.empty((n, n_heads * vdim), dtype=torch.float32, device=qkv.device)
         self._check(self.lib.yk_linear_state_scan(
             qkv.data_ptr(), qkv.stride(0), _code(qkv.dtype), n_heads, n_kv, dim, vdim, state.data_ptr(), a["seq_qstart"].data_ptr(),
             a["seq_qlen"].data_ptr(), a["state_slots"].data_ptr(), a["seq_qstart"].numel(), n, float(q_scale),
-            -1.0 if unit_eps is None else float(unit_eps), mode, src.data_ptr(), src.stride(0), col,
+            -1.0 if unit_eps is None else float(unit_eps), mode, _ptr(src), 0 if src is None else src.stride(0), col,
             p0.data_ptr(), _ptr(p1), tau, beta[0].data_ptr() if beta_f32 else None, 0 if beta is None else beta[0].stride(0),
             0 if beta is None else int(beta[1]), out.data_ptr(), int(q_col), int(k_col), int(v_col), write_mode, _ptr(skip),
             beta[0].data_ptr() if beta is not None and not beta_f32 else None, _ptr(bonus), _ptr(decays), self._stream()))
         return out
 
+    FIXED_DECAY_CHUNK = 64  # tokens of a span that meet in products
+
+    def scan_inputs(self, proj, n_heads, dim, vdim, k_scale=1.0, rotation=None, positions=None, act=None) -> torch.Tensor:
+        """float32 rows [q | k | v] as they enter a recurrence, from a projection's rows [q | k | v | ...]: ``act`` ("silu") on all
+        three, ``rotation`` on q and k by the tokens' positions, k times ``k_scale``."""
+        self._rows(proj, "scan_inputs input")
+        if act not in (None, "silu"):
+            raise KernelError(f"scan_inputs: activation {act!r} is not offered")
+        n = proj.shape[0]
+        if proj.shape[1] < n_heads * (2 * dim + vdim):
+            raise KernelError(f"scan_inputs: rows of {proj.shape[1]} elements, fewer than the heads need")
+        r = rotation
+        if r is not None and (r.cos.dtype != torch.float32 or r.cos.shape != r.sin.shape or r.cos.shape[1] != r.rotary_dim // 2 or positions.numel() != n):
+            raise KernelError("scan_inputs: rotary tables are float32 [positions, rotary_dim/2], and every token has a position")
+        out = torch.empty((n, n_heads * (2 * dim + vdim)), dtype=torch.float32, device=proj.device)
+        self._check(self.lib.yk_scan_inputs(
+            proj.data_ptr(), proj.stride(0), _code(proj.dtype), n_heads, dim, vdim, _ptr(positions) if r is not None else None,
+            None if r is None else r.cos.data_ptr(), None if r is None else r.sin.data_ptr(), 0 if r is None else r.rotary_dim,
+            int(bool(r is not None and r.interleaved)), 0 if r is None else r.cos.shape[0], float(k_scale), int(act == "silu"), out.data_ptr(), n,
+            self._stream()))
+        return out
+
+    def fixed_decay_scan(self, proj, n_heads, dim, vdim, state, ctx, decay, k_scale=1.0, rotation=None, act=None, chunks=None, seq_chunk0=None):
+        """The recurrence S <- a_h S + k v^T, o = S^T q with a constant decay per head (``decay`` float32 [heads]) over each
+        request's span, S [slots, heads, dim, vdim] float32 updated in place.  ``proj`` [N, >= heads * (2 * dim + vdim)]: columns
+        [q | k | v | ...] as projected; see ``scan_inputs`` for what is made of them first.  Returns o float32 [N, heads * vdim]."""
+        rows = self.scan_inputs(proj, n_heads, dim, vdim, k_scale, rotation, ctx.arrays["positions"], act)
+        return self.linear_state_scan(rows, n_heads, n_heads, dim, vdim, state, ctx, decay=("fixed", decay))
+
     def gated_head_norm(self, o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first: bool = False,
                         gate_act: str = "silu") -> torch.Tensor:
         """Per head, o / sqrt(mean(o^2) + eps) * weight * silu(gate[:, gate_col + h * vdim + .]); ``o`` float32
-        [N, heads * vdim], ``weight`` [vdim] shared by the heads, or [heads * vdim].  The "heads" are whatever equal
+        [N, heads * vdim], ``weight`` [vdim] shared by the heads, or [heads * vdim], or None.  The "heads" are whatever equal
         parts of a row are normed each by its own root mean square.  ``gate_first``: the gate comes before the
         norm, rms(o * silu(gate)) * weight.  ``gate_act`` "sigmoid": the sigmoid in silu's place.  The gate comes in
         ``out_dtype`` or float32."""
@@ -1751,15 +1873,15 @@ class HipOps:
             raise KernelError(f"gated_head_norm: gate {gate_act!r} is not offered")
         n = o.shape[0]
         self._rows(gate, "gated_head_norm gate")
-        if o.dtype != torch.float32 or not o.is_contiguous() or o.shape[1] != n_heads * vdim or weight.numel() not in (vdim, n_heads * vdim) \
-                or not weight.is_contiguous():
+        if o.dtype != torch.float32 or not o.is_contiguous() or o.shape[1] != n_heads * vdim or (weight is not None and (
+                weight.numel() not in (vdim, n_heads * vdim) or not weight.is_contiguous())):
             raise KernelError("gated_head_norm: o is contiguous float32 [N, heads * vdim], the weight [vdim] or [heads * vdim]")
         if gate.dtype not in (out_dtype, torch.float32) or gate.shape[0] != n or gate.shape[1] < gate_col + n_heads * vdim:
             raise KernelError("gated_head_norm: the gate does not fit")
         out = torch.empty((n, n_heads * vdim), dtype=out_dtype, device=o.device)
         self._check(self.lib.yk_gated_head_norm(
-            o.data_ptr(), weight.data_ptr(), _code(weight.dtype), float(eps), gate.data_ptr(), _code(gate.dtype), gate.stride(0),
-            gate_col, n_heads, vdim, out.data_ptr(), _code(out_dtype), n, int(weight.numel() != vdim or n_heads == 1),
+            o.data_ptr(), _ptr(weight), _F32 if weight is None else _code(weight.dtype), float(eps), gate.data_ptr(), _code(gate.dtype), gate.stride(0),
+            gate_col, n_heads, vdim, out.data_ptr(), _code(out_dtype), n, int(weight is not None and (weight.numel() != vdim or n_heads == 1)),
             int(bool(gate_first)), int(gate_act == "sigmoid"), self._stream()))
         return out
 
@@ -2010,6 +2132,27 @@ class HipOps:
         self._check(self.lib.yk_moe_router_topk(logits.data_ptr(), logits.stride(0), experts, int(top), x.data_ptr(), x.stride(0), _code(x.dtype),
                                                 x.shape[1], choice.data_ptr(), xs.data_ptr(), n, _ptr(bias), None, self._stream()))
         return choice, xs
+
+    def moe_router_share(self, logits, top: int, experts: Optional[int] = None, bias=None, correction=None, groups=None):
+        """(choice int32 [N, top], weights float32 [N, top]) from a router's float32 ``logits`` [N, >= experts]: scores are their
+        sigmoids (``bias`` float32 [experts] joins the logits), the choice is by score + ``correction`` (float32 [experts]); with
+        ``groups`` = (count, keep) among the experts of the ``keep`` best of ``count`` equal groups of neighbours, a group's score
+        the sum of its two largest; a chosen expert's weight is its score over the sum of the chosen scores + 1e-20.  Among
+        equals the lower number wins."""
+        self._rows(logits, "router logits")
+        n = logits.shape[0]
+        experts = logits.shape[1] if experts is None else int(experts)
+        if logits.dtype != torch.float32 or experts > logits.shape[1]:
+            raise KernelError("moe_router_share: logits are float32 [N, >= experts]")
+        for t in (bias, correction):
+            if t is not None and (t.dtype != torch.float32 or t.numel() != experts or not t.is_contiguous()):
+                raise KernelError("moe_router_share: the bias and the correction are contiguous float32 [experts]")
+        count, keep = (0, 0) if groups is None else (int(groups[0]), int(groups[1]))
+        choice = torch.empty((n, top), dtype=torch.int32, device=logits.device)
+        weights = torch.empty((n, top), dtype=torch.float32, device=logits.device)
+        self._check(self.lib.yk_moe_router_share(logits.data_ptr(), logits.stride(0), experts, int(top), _ptr(bias), _ptr(correction), count, keep,
+                                                 choice.data_ptr(), weights.data_ptr(), n, self._stream()))
+        return choice, weights
 
     def moe_combine(self, dense, rows, top: int, weight: float = 1.0, row_weights=None) -> torch.Tensor:
         """float32 [N, width]: ``dense`` (a tensor, a ``SplitSum`` or None) + weight * the sum of each token's ``top``

@@ -42,7 +42,12 @@ query_temperature ({"coef": c, "every": e}: the query at position p is multiplie
 position p sees the keys from floor(p / window) * window on, counted from the sequence's start), sink_score (a
 number: a sink of that score for every head, without a tensor), qk_norm without "q" and "k" (queries and keys are
 divided by their root mean square per head and multiplied by no weight; since a rotation changes no pair's length
-this is the same before the rotation as after it).  A layer may have no position encoding at all (``position``
+this is the same before the rotation as after it), projection_bias["v"] (a bias of the v projection too), differential
+({"q1", "k1", "q2", "k2": tensor names below the prefix, [head_dim] each; "offset": d; "eps": e}: differential attention (Ye
+et al., "Differential Transformer").  Every query and key head is two of head_dim elements side by side, [map 1 | map 2];
+each map has a softmax of its own over its scores, both weigh the same values, and a head's output is
+a1 - lambda a2, divided by its root mean square (e under the root) and multiplied by 1 - d, with one number for
+the layer, lambda = exp(sum(q1 k1)) - exp(sum(q2 k2)) + d).  A layer may have no position encoding at all (``position``
 None).
 """
 from __future__ import annotations
@@ -69,7 +74,12 @@ class Attention(Mixer):
         self.hidden = int(params["hidden_size"])
         self.n_heads = int(params["num_heads"])
         self.n_kv = int(params["num_kv_heads"])
-        self.head_dim = int(params["head_dim"])
+        self.differential = params.get("differential")
+        # with two maps a head's queries and keys are both maps' side by side
+        self.maps = 2 if self.differential else 1
+        self.head_dim = int(params["head_dim"]) * self.maps
+        self.score_heads = self.n_heads * self.maps  # softmaxes a token has
+        self.map_constants = None  # (lambda, eps, 1 - offset), from the tensors
         self.scale = float(params["scale"])
         self.window = params.get("window")
         if self.n_heads % self.n_kv:
@@ -89,6 +99,9 @@ class Attention(Mixer):
         if self.rotation is not None and self.rotation.rotary_dim > self.head_dim:
             raise ValueError("rotary_dim exceeds head_dim")
         self.value_dim = int(params.get("value_dim") or self.head_dim)
+        if self.differential and (params.get("qk_norm") or params.get("value_position") or params.get("gate") or params.get("sink")
+                                  or params.get("sink_score") is not None or params.get("distance_bias") or pos is not None):
+            raise ValueError(f"{self.prefix}: two maps are not offered together with norms, rotations, gates, sinks or biases per distance")
         self.qk_norm = params.get("qk_norm")
         self.value_norm_eps = params.get("value_norm_eps")
         vpos: PartSpec = params.get("value_position")
@@ -117,8 +130,8 @@ class Attention(Mixer):
         if self.values_from_keys and self.value_dim != self.head_dim:
             raise ValueError(f"{self.prefix}: values that are the keys are as wide as the keys")
         self.projection_bias = dict(params.get("projection_bias") or {})
-        if set(self.projection_bias) - {"q", "k"}:
-            raise ValueError(f"{self.prefix}: projection_bias names the biases of q and k")
+        if set(self.projection_bias) - {"q", "k", "v"} or (self.values_from_keys and "v" in self.projection_bias):
+            raise ValueError(f"{self.prefix}: projection_bias names the biases of q, k and (where there is such a projection) v")
         # (a norm without weights divides each head by its own root mean square)
         self.qk_norm_weights = bool(self.qk_norm) and self.qk_norm.get("q") is not None
         if self.qk_norm and self.qk_norm_weights != (self.qk_norm.get("k") is not None):
@@ -135,13 +148,13 @@ class Attention(Mixer):
         self.masked = bool(
             self.value_dim != self.head_dim or self.qk_norm or self.value_norm_eps is not None or self.value_rotation is not None
             or self.softcap or self.keep_first or self.gate_name or self.distance_bias or self.sink_name or self.values_from_keys
-            or self.projection_bias or self.query_temperature or self.chunked or self.sink_score is not None
+            or self.projection_bias or self.query_temperature or self.chunked or self.sink_score is not None or self.differential
         )
         self.w_qn = self.w_kn = None
         if self.masked:
             if self.bias:
                 raise ValueError(f"{self.prefix}: the four biases are not offered together with the masked attention's options "
-                                 "(projection_bias gives q and k theirs)")
+                                 "(projection_bias gives q, k and v theirs)")
             self.group = None
             self.w_qkv = self.w_q = self.w_o = None
             self.b_qkv = self.b_q = self.b_o = None
@@ -153,6 +166,9 @@ class Attention(Mixer):
             if self.on_matrix_cores and (self.sink_name or self.sink_score is not None):
                 with_sink = getattr(rt.ops, "attention_takes_sink", None)
                 self.on_matrix_cores = bool(with_sink is not None and with_sink(rt.act_dtype, self.head_dim) is True)
+            if self.on_matrix_cores and self.differential:
+                with_maps = getattr(rt.ops, "attention_takes_maps", None)
+                self.on_matrix_cores = bool(with_maps is not None and with_maps(rt.act_dtype, self.head_dim) is True)
             if self.on_matrix_cores:
                 self._tile_sizes(rt)
             return
@@ -170,12 +186,12 @@ class Attention(Mixer):
         self.b_qkv = self.b_q = self.b_o = None
 
     def _tile_sizes(self, rt) -> None:
-        self.tokens_per_tile = rt.ops.attention_tokens_per_tile(self.n_heads, self.n_kv)
+        self.tokens_per_tile = rt.ops.attention_tokens_per_tile(self.score_heads, self.n_kv)
         # spans longer than `long_tile` go to the kernel for long spans, in tiles of that many
         # tokens or twice as many (`long_tiles_of`: the step's choice)
-        self.long_tile = rt.ops.attention_long_span_tile(self.n_heads, self.n_kv)
-        self.long_tile_2 = rt.ops.attention_long_span_tile(self.n_heads, self.n_kv, 2)
-        self.layout = f"h{self.n_heads}g{self.n_kv}"
+        self.long_tile = rt.ops.attention_long_span_tile(self.score_heads, self.n_kv)
+        self.long_tile_2 = rt.ops.attention_long_span_tile(self.score_heads, self.n_kv, 2)
+        self.layout = f"h{self.score_heads}g{self.n_kv}"
 
     # ---- what it needs
     def tensor_specs(self) -> Dict[str, TensorSpec]:
@@ -198,6 +214,11 @@ class Attention(Mixer):
             specs[f"{self.prefix}.{self.projection_bias['q']}"] = TensorSpec((hd,), "float", ("normal", 0.1))
         if "k" in self.projection_bias and self.projects_kv:
             specs[f"{self.prefix}.{self.projection_bias['k']}"] = TensorSpec((kd,), "float", ("normal", 0.1))
+        if "v" in self.projection_bias and self.projects_kv:
+            specs[f"{self.prefix}.{self.projection_bias['v']}"] = TensorSpec((self.n_kv * self.value_dim,), "float", ("normal", 0.1))
+        if self.differential:
+            for which in ("q1", "k1", "q2", "k2"):
+                specs[f"{self.prefix}.{self.differential[which]}"] = TensorSpec((self.head_dim // self.maps,), "float", ("normal", 0.1))
         if self.sink_name:
             specs[f"{self.prefix}.{self.sink_name}"] = TensorSpec((self.n_heads,), "float", ("normal", 1.0))
         if self.gate_name:
@@ -250,7 +271,15 @@ class Attention(Mixer):
                 if "k" in self.projection_bias and self.projects_kv:
                     kd = self.n_kv * self.head_dim
                     b[q.shape[0]: q.shape[0] + kd] = tensors[f"{self.prefix}.{self.projection_bias['k']}"].to(torch.float32)
+                if "v" in self.projection_bias and self.projects_kv:
+                    v0 = q.shape[0] + self.n_kv * self.head_dim
+                    b[v0: v0 + self.n_kv * self.value_dim] = tensors[f"{self.prefix}.{self.projection_bias['v']}"].to(torch.float32)
                 self.b_proj = b
+            if self.differential:
+                d = self.differential
+                q1, k1, q2, k2 = (tensors[f"{self.prefix}.{d[n]}"].to(torch.float32) for n in ("q1", "k1", "q2", "k2"))
+                lam = torch.exp((q1 * k1).sum()) - torch.exp((q2 * k2).sum()) + float(d["offset"])
+                self.map_constants = (float(lam), float(d["eps"]), 1.0 - float(d["offset"]))
             return
         if self.projects_kv:
             self.w_qkv = torch.cat([q, tensors[self.names["k"]], tensors[self.names["v"]]], dim=0).contiguous()
@@ -310,8 +339,8 @@ class Attention(Mixer):
             return 1
         qlen = hb.seq_qlen[long_spans].astype(np.int64)
         tiles = int((-(-qlen // self.long_tile_2)).sum())
-        heads_per_tile = min(self.n_heads // self.n_kv, 16)
-        chunks = -(-(self.n_heads // self.n_kv) // heads_per_tile)
+        heads_per_tile = min(self.score_heads // self.n_kv, 16)
+        chunks = -(-(self.score_heads // self.n_kv) // heads_per_tile)
         fewest = int((hb.seq_ctx[long_spans] - hb.seq_qlen[long_spans]).min())
         return self.rt.ops.attention_long_col_tiles(tiles * self.n_kv * chunks, fewest)
 
@@ -359,6 +388,8 @@ class Attention(Mixer):
             more["values_from_keys"] = True
         if self.qk_norm and not self.qk_norm_weights:
             more["unweighted_norm"] = True
+        if self.differential and self.on_matrix_cores:
+            more["query_maps"] = self.maps  # each map's queries as a row of their own, zeros where the other's keys are
         q = ops.qkv_prepare(
             proj, self.n_heads, n_kv_rows, self.head_dim, self.value_dim, ctx.arrays["positions"], self.rt.act_dtype,
             q_norm=self.w_qn, k_norm=self.w_kn, qk_eps=float(self.qk_norm["eps"]) if self.qk_norm else 0.0,
@@ -370,13 +401,15 @@ class Attention(Mixer):
         sink = {} if self.sink is None else {"sink": self.sink}
         if self.chunked:
             sink["chunked"] = True
+        if self.differential:
+            sink["differential"] = self.map_constants
         if self.on_matrix_cores:
             memo_key = f"attention_long_col_tiles_{self.layout}"
             col_tiles = ctx.memo.get(memo_key)
             if col_tiles is None:
                 col_tiles = ctx.memo[memo_key] = self.long_col_tiles(ctx.host)
             out = ops.attention(
-                q, self.n_heads, self.n_kv, self.head_dim, k_cache, v_cache, self.rt.page_size, self.scale,
+                q, self.score_heads, self.n_kv, self.head_dim, k_cache, v_cache, self.rt.page_size, self.scale,
                 0 if self.window is None else int(self.window), ctx, site.group,
                 ctx.arrays[f"attention_tiles_{self.tokens_per_tile}_upto{self.long_tile}"],
                 ctx.arrays[f"attention_long_tiles_{self.long_tile_2 if col_tiles == 2 else self.long_tile}_{self.layout}"],

@@ -143,6 +143,16 @@ class NormedSum:
         return self.combine()
 
 
+class StreamMix:
+    """A pending contribution to a stream that is kept as several copies (residual [N, streams, width]): every copy
+    becomes a mix of all the old ones plus a share of the branch's output, x_t <- sum_s mix[s, t] x_s + out[t] y.  ``inner``
+    is y, whatever a part's ``forward`` returned; ``mix`` (float32 [streams, streams], indexed [from, to]) and ``out``
+    (float32 [streams]) are on the device.  ``Norm.streams_norm`` applies it in the pass that reads the copies next."""
+
+    def __init__(self, inner, mix: torch.Tensor, out: torch.Tensor):
+        self.inner, self.mix, self.out = inner, mix, out
+
+
 class Part:
     """Common to all parts."""
 
@@ -260,6 +270,13 @@ class Norm(Part):
         raise NotImplementedError
 
 
+    def streams_norm(self, residual: torch.Tensor, delta: Optional["StreamMix"], read: Optional[torch.Tensor], rows=None) -> torch.Tensor:
+        """For a stream kept as copies, ``residual`` float32 [N, streams, width]: apply ``delta`` to them in place, and
+        return norm(sum_s read[s] x_s) in the activation dtype (``read`` float32 [streams]; None: their plain sum).  With
+        ``rows`` (one index per output row) those rows only, and ``residual`` stays as it is."""
+        raise NotImplementedError
+
+
 class Position(Part):
     """A position encoding.  What a mixer may ask of it (a kind implements what it offers and
     leaves the rest at None; a mixer raises for a kind that offers nothing it can use):
@@ -276,11 +293,21 @@ class Position(Part):
         return None
 
 
+class Streams(Part):
+    """How one branch of a block hangs on a stream that is kept as several copies: what it reads of them (``read``,
+    float32 [streams]) and how its output goes back (``write(y)`` -> ``StreamMix``)."""
+
+    read: Optional[torch.Tensor] = None
+
+    def write(self, y) -> StreamMix:
+        raise NotImplementedError
+
+
 class Block:
     """The arrangement of norms, mixer and feed-forward around the residual.
 
     ``roles`` names the parts an arrangement is built from: role -> (family, required), the
-    family one of "mixer", "feed_forward", "norm".  The model builds every role a layer's
+    family one of "mixer", "feed_forward", "norm", "streams".  The model builds every role a layer's
     spec names through the family's registry and calls the arrangement with them as keyword
     arguments (roles the spec leaves out, where not required, come as None).  ``mixer`` (a role
     or None) is the part whose cache and state the model plans memory for."""
@@ -330,9 +357,10 @@ POSITIONS = _Registry("position encoding")
 BLOCKS = _Registry("block arrangement")
 EMBEDDINGS = _Registry("embedding")
 HEADS = _Registry("output head")
+STREAMS = _Registry("stream connection")
 
 # family name (``Block.roles``) -> registry
-FAMILIES = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS}
+FAMILIES = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS, "streams": STREAMS}
 
 register_mixer = MIXERS.register
 register_feed_forward = FEED_FORWARDS.register
@@ -341,3 +369,4 @@ register_position = POSITIONS.register
 register_block = BLOCKS.register
 register_embedding = EMBEDDINGS.register
 register_head = HEADS.register
+register_streams = STREAMS.register

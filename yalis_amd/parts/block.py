@@ -199,3 +199,37 @@ class SandwichBlock(Block):
             return pending
         h = self.feed_forward_norm.add_norm(residual, pending)
         return NormedBranch(self.feed_forward.forward(h, ctx), self.feed_forward_out_norm, self.branch_scale)
+
+
+@register_block("mixed_streams")
+class MixedStreamsBlock(Block):
+    """Pre-norm branches on a stream kept as several copies: u = sum_s in[s] x_s, y = branch(norm(u)),
+    x_t <- sum_s mix[s, t] x_s + out[t] y, first for the mixer, then for the feed-forward, each with weights of its own
+    (``parts/streams.py``).  A layer may leave the feed-forward, its norm and its connection out.
+
+    The residual is [N, streams, width].  Between two branches the copies are touched once: the norm that reads them next
+    mixes them and adds the pending branch in the same pass (``Norm.streams_norm``); the last one is handed on as a
+    ``StreamMix``."""
+
+    roles = {
+        "mixer_streams": ("streams", True),
+        "mixer_norm": ("norm", True),
+        "mixer": ("mixer", True),
+        "feed_forward_streams": ("streams", False),
+        "feed_forward_norm": ("norm", False),
+        "feed_forward": ("feed_forward", False),
+    }
+
+    def __init__(self, mixer_streams, mixer_norm, mixer, feed_forward_streams=None, feed_forward_norm=None, feed_forward=None):
+        if len({feed_forward is None, feed_forward_norm is None, feed_forward_streams is None}) != 1:
+            raise ValueError("a mixed_streams block has a feed-forward with its norm and its connection, or none of the three")
+        self.mixer_streams, self.mixer_norm, self.mixer = mixer_streams, mixer_norm, mixer
+        self.feed_forward_streams, self.feed_forward_norm, self.feed_forward = feed_forward_streams, feed_forward_norm, feed_forward
+
+    def forward(self, residual, delta, ctx, site):
+        h = self.mixer_norm.streams_norm(residual, delta, self.mixer_streams.read)
+        delta = self.mixer_streams.write(self.mixer.forward(h, ctx, site))
+        if self.feed_forward is None:
+            return delta
+        h = self.feed_forward_norm.streams_norm(residual, delta, self.feed_forward_streams.read)
+        return self.feed_forward_streams.write(self.feed_forward.forward(h, ctx))

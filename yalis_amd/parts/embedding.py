@@ -125,10 +125,43 @@ class TokenPairEmbedding(TokenEmbedding):
         return residual, Settled(rounded)
 
 
+@register_embedding("normed_token_embedding")
+class NormedTokenEmbedding(TokenEmbedding):
+    """The token's row through an RMS norm with a weight, float32: the stream starts normed.  ``streams`` (None: one
+    stream, [N, hidden]): the stream is kept as that many copies [N, streams, hidden], all equal at the start.
+
+    params: name, norm_name (the norm's weight), eps, vocab_size, hidden_size, streams."""
+
+    graph_capturable = True
+
+    def __init__(self, params, rt: Runtime):
+        super().__init__(params, rt)
+        self.norm_name = params["norm_name"]
+        self.eps = float(params["eps"])
+        self.streams = params.get("streams")
+        self.norm_weight = None
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return {self.name: TensorSpec((self.vocab, self.hidden)), self.norm_name: TensorSpec((self.hidden,), "float", ("one_plus_normal", 0.1))}
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        self.table, self.norm_weight = tensors[self.name].contiguous(), tensors[self.norm_name].contiguous()
+        if self.norm_weight.dtype != self.table.dtype:
+            self.table, self.norm_weight = self.table.float(), self.norm_weight.float()
+
+    def forward(self, token_ids: torch.Tensor) -> torch.Tensor:
+        x = self.rt.ops.embed_norm(token_ids, self.table, self.norm_weight, self.eps, 1 if self.streams is None else int(self.streams))
+        return x[:, 0] if self.streams is None else x
+
+    def begin(self, token_ids: torch.Tensor, lazily: bool):
+        return self.forward(token_ids), None
+
+
 @register_head("lm_head")
 class LMHead(Part):
     """params: name, tied_to (name of the embedding table, or None), vocab_size,
-    hidden_size, scale (1.0: what the logits are multiplied with)."""
+    hidden_size, scale (1.0: what the logits are multiplied with), softcap (None; c: logits are squashed to
+    c tanh(z / c), after the scale)."""
 
     graph_capturable = True
 
@@ -139,6 +172,7 @@ class LMHead(Part):
         self.vocab = int(params["vocab_size"])
         self.hidden = int(params["hidden_size"])
         self.scale = float(params.get("scale", 1.0))
+        self.softcap = float(params.get("softcap") or 0.0)
         self.weight = None
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
@@ -160,6 +194,8 @@ class LMHead(Part):
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         logits = self.rt.ops.linear(h, self.weight, torch.float32)
-        if self.scale != 1.0:
+        if self.softcap:
+            self.rt.ops.scale_rows(logits, self.scale, softcap=self.softcap)
+        elif self.scale != 1.0:
             self.rt.ops.scale_rows(logits, self.scale)
         return logits

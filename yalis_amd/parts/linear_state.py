@@ -35,6 +35,15 @@ decay exp(-exp(A_log) dt) and the strength of its write, S <- a S + dt B x^T (k 
 S^T C + D x (q = C, a skip per head); B and C are shared by groups of heads.  The read-out is gated first, by
 silu(z), and then normed in ``norm_groups`` equal parts, each by its own root mean square, with a weight as wide as
 the read-out.
+
+"retention" (Sun et al., "Retentive Network: A Successor to Transformer for Large Language Models"): a decay per head that is a constant
+of the model, plain writes; q and k rotate by their positions and k is multiplied by head_dim^-1/2 on top; the read-out is normed
+per head without a weight and gated by silu of W_g h.
+
+"lightning_attention" (Qin et al., "Lightning Attention-2: A Free Lunch for Handling Unlimited Sequence Lengths in Large Language
+Models"): the same recurrence on silu(W_q h), silu(W_k h), silu(W_v h); the heads' read-outs are normed together with one weight and
+gated by the sigmoid of W_g h.  These two run on a scan of their own (``ops.fixed_decay_scan``): with decays that do not depend
+on the tokens, the tokens of a chunk meet in products, and only the memory passes from chunk to chunk.
 """
 from __future__ import annotations
 
@@ -42,8 +51,10 @@ from typing import Dict, Mapping
 
 import torch
 
+from ..config.specs import PartSpec
+from ..engine.batch import chunk_starts, span_chunks
 from ..weights.loader import TensorSpec
-from .base import Mixer, Runtime, StateNeed, register_mixer
+from .base import POSITIONS, Mixer, Runtime, StateNeed, register_mixer
 from .latent_attention import _pad_rows
 
 
@@ -332,6 +343,96 @@ class GatedLinearAttention(_MatrixStateMixer):
             unit_eps=None, decay=("channel", z, 0, self.b_a2, self.tau), beta=None,
         )
         return self._finish(o, proj, self.gate_col)
+
+
+class _FixedDecayMixer(_MatrixStateMixer):
+    """params: prefix, hidden_size, num_heads, head_dim, value_dim, decay (one number per head), out_norm_eps, names."""
+
+    # what the scan makes of the projections as they enter it
+    input_act = None  # an activation of q, k and v
+    k_scale = 1.0
+    rotation = None
+
+    def __init__(self, params, rt: Runtime):
+        super().__init__(params, rt)
+        decay = [float(d) for d in params["decay"]]
+        if len(decay) != self.n_heads or not all(0.0 <= d <= 1.0 for d in decay):
+            raise ValueError(f"{self.prefix}: decay holds a number between 0 and 1 for each of the {self.n_heads} heads, got {decay}")
+        self.decay_list = decay
+        self.decay = None
+        self.qkv_cols = self.qk_cols + self.v_cols
+        self.gate_col = self.qkv_cols + (-self.qkv_cols % 8)
+        self.chunk = int(getattr(rt.ops, "FIXED_DECAY_CHUNK", 64))  # tokens that meet in products
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        specs = self._common_specs()
+        del specs[self._name("norm")]
+        return specs
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        t = lambda short: tensors[self._name(short)]
+        q = t("q")
+        pad = torch.zeros((self.gate_col - self.qkv_cols, self.hidden), dtype=q.dtype, device=q.device)
+        self.w_in = _pad_rows([p for p in (q, t("k"), t("v"), pad, t("g")) if p.shape[0]], 16)
+        self.w_o = t("o")
+        self.decay = torch.tensor(self.decay_list, dtype=torch.float32, device=q.device)
+
+    def state_need(self):
+        return self._state()
+
+    def products(self):
+        rows = self.gate_col + self.v_cols
+        return ((rows + (-rows % 16), self.hidden), (self.hidden, self.v_cols))
+
+    def step_inputs(self):
+        n = self.chunk
+        return {f"span_chunks_{n}": lambda hb: span_chunks(hb, n), f"chunk_starts_{n}": lambda hb: chunk_starts(hb, n)}
+
+    def forward(self, h: torch.Tensor, ctx, site) -> torch.Tensor:
+        ops = self.rt.ops
+        proj = ops.linear(h, self.w_in, self.rt.act_dtype)
+        o = ops.fixed_decay_scan(
+            proj, self.n_heads, self.head_dim, self.value_dim, site.state(0), ctx, self.decay, k_scale=self.k_scale,
+            rotation=self.rotation, act=self.input_act, chunks=ctx.arrays[f"span_chunks_{self.chunk}"],
+            seq_chunk0=ctx.arrays[f"chunk_starts_{self.chunk}"])
+        return self._out(o, proj)
+
+    def _out(self, o, proj):
+        raise NotImplementedError
+
+
+@register_mixer("retention")
+class Retention(_FixedDecayMixer):
+    """params: as above, and position (a rotary PartSpec, or None: nothing rotates), k_scale (head_dim^-1/2)."""
+
+    def __init__(self, params, rt: Runtime):
+        super().__init__(params, rt)
+        self.k_scale = float(params.get("k_scale", self.head_dim ** -0.5))
+        pos: PartSpec = params.get("position")
+        if pos is not None:
+            self.rotation = POSITIONS.get(pos.kind)(pos.params, rt).rotation()
+            if self.rotation is None or self.rotation.rotary_dim > self.head_dim:
+                raise ValueError(f"{self.prefix}: this mixer takes a rotation of at most head_dim={self.head_dim} elements")
+
+    def _out(self, o, proj):
+        return self._finish(o, proj, self.gate_col)  # (no weight)
+
+
+@register_mixer("lightning_attention")
+class LightningAttention(_FixedDecayMixer):
+    input_act = "silu"
+
+    def tensor_specs(self) -> Dict[str, TensorSpec]:
+        return dict(super().tensor_specs(), **{self._name("norm"): TensorSpec((self.v_cols,), "float", ("one_plus_normal", 0.1))})
+
+    def load(self, tensors: Mapping[str, torch.Tensor]) -> None:
+        super().load(tensors)
+        self.w_norm = tensors[self._name("norm")].contiguous()
+
+    def _out(self, o, proj):
+        ops, act = self.rt.ops, self.rt.act_dtype
+        y = ops.gated_head_norm(o, self.w_norm, self.out_eps, proj, self.gate_col, 1, self.v_cols, act, gate_act="sigmoid")
+        return ops.linear(y, self.w_o, act, partial_ok=True)
 
 
 @register_mixer("state_space_duality")

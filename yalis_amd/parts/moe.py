@@ -118,13 +118,18 @@ class RoutedMoE(FeedForward):
     Other forms of the same mixture: ``router_bias`` (a tensor name below the prefix, [experts], added to the
     float32 logits before the choice), ``scores`` "softmax_of_chosen" (the chosen experts' weights are the softmax
     over their own logits alone; the default "sigmoid" is as above), ``weighs`` "output" (an expert reads the
-    token's input as it is and its output is multiplied by the weight; the default "input" is as above),
+    token's input as it is and its output is multiplied by the weight; the default "input" is as above), ``scores``
+    "sigmoid_share" (weights on the outputs: the chosen experts' sigmoids, divided by their sum + 1e-20), with it
+    ``choice_correction`` (a tensor name below the prefix, [experts], added to the sigmoids for the choice alone) and
+    ``groups`` ({"count", "keep"}: the experts form ``count`` equal groups of neighbours, a group's score is the sum of its
+    two largest choice scores, and only experts of the ``keep`` best groups can be chosen),
     ``gated`` False (an expert is down(act(up x)) with ``activation`` one of the kernel library's plain ones,
     "relu2" the square of relu; no gate tensor).  With weights on the outputs ``forward`` returns the experts'
     uncombined rows beside their weights (``ExpertRows``) for whoever sums the branch into the stream.
 
     params: prefix, hidden_size, experts, top, intermediate_size, activation ("silu"), shared (None or
     {"intermediate_size", "activation"}), router_bias (None), scores ("sigmoid"), weighs ("input"), gated (True),
+    choice_correction (None), groups (None),
     names (optional: "router", "expert" with {e} for the expert's number, "shared", "gate", "up", "down")."""
 
     graph_capturable = True
@@ -148,9 +153,18 @@ class RoutedMoE(FeedForward):
         self.router_bias = None
         self.scores = params.get("scores", "sigmoid")
         self.weighs = params.get("weighs", "input")
-        if (self.scores, self.weighs) not in (("sigmoid", "input"), ("softmax_of_chosen", "output")):
+        if (self.scores, self.weighs) not in (("sigmoid", "input"), ("softmax_of_chosen", "output"), ("sigmoid_share", "output")):
             raise ValueError(f"{self.prefix}: scores={self.scores!r} with weighs={self.weighs!r} is not offered "
-                             "(sigmoid scores weigh the inputs, a softmax over the chosen weighs the outputs)")
+                             "(sigmoid scores weigh the inputs, a softmax over the chosen or their sigmoids' shares weigh the outputs)")
+        self.correction_name = params.get("choice_correction")
+        self.correction = None
+        self.groups = params.get("groups")
+        if self.scores != "sigmoid_share" and (self.correction_name or self.groups):
+            raise ValueError(f"{self.prefix}: a correction of the choice and groups go with scores 'sigmoid_share'")
+        if self.groups is not None:
+            count, keep = int(self.groups["count"]), int(self.groups["keep"])
+            if count < 1 or self.experts % count or not 1 <= keep <= count or self.top > keep * (self.experts // count):
+                raise ValueError(f"{self.prefix}: {count} groups of {self.experts} experts, {keep} kept, cannot give {self.top} a token")
         self.shared = params.get("shared")
         names = {"router": "router", "expert": "e{e}", "shared": "shared", "gate": "gate", "up": "up", "down": "down"}
         names.update(params.get("names", {}))
@@ -171,6 +185,8 @@ class RoutedMoE(FeedForward):
         specs = {f"{self.prefix}.{self.names['router']}": TensorSpec((self.experts, self.hidden), "float", ("normal", 0.5))}
         if self.router_bias_name:
             specs[f"{self.prefix}.{self.router_bias_name}"] = TensorSpec((self.experts,), "float", ("normal", 0.5))
+        if self.correction_name:
+            specs[f"{self.prefix}.{self.correction_name}"] = TensorSpec((self.experts,), "float", ("normal", 0.1))
         for e in range(self.experts):
             if self.gated:
                 specs[self._name(self._expert(e), "gate")] = TensorSpec((self.inter, self.hidden))
@@ -191,6 +207,8 @@ class RoutedMoE(FeedForward):
         self.w_router = router.contiguous()
         if self.router_bias_name:
             self.router_bias = tensors[f"{self.prefix}.{self.router_bias_name}"].to(torch.float32).contiguous()
+        if self.correction_name:
+            self.correction = tensors[f"{self.prefix}.{self.correction_name}"].to(torch.float32).contiguous()
         # [experts, 2, ff, hidden] (gate rows, then up rows), or [experts, 1, ff, hidden] without gates
         self.w_gate_up = torch.stack([
             torch.stack(([tensors[self._name(self._expert(e), "gate")]] if self.gated else []) + [tensors[self._name(self._expert(e), "up")]])
@@ -213,7 +231,12 @@ class RoutedMoE(FeedForward):
         ops = self.rt.ops
         logits = ops.linear(h, self.w_router, torch.float32)
         if self.weighs == "output":
-            choice, weights = ops.moe_router_topk(logits, None, self.top, experts=self.experts, bias=self.router_bias, scores=self.scores)
+            if self.scores == "sigmoid_share":
+                groups = None if self.groups is None else (int(self.groups["count"]), int(self.groups["keep"]))
+                choice, weights = ops.moe_router_share(logits, self.top, experts=self.experts, bias=self.router_bias, correction=self.correction,
+                                                       groups=groups)
+            else:
+                choice, weights = ops.moe_router_topk(logits, None, self.top, experts=self.experts, bias=self.router_bias, scores=self.scores)
             rows = ops.moe_experts(h, None, choice, self.w_gate_up, self.w_down, self.activation, input_per_token=True)
             dense = None
             if self.shared:

@@ -7,7 +7,8 @@ every norm of a pre-norm block: the float32 residual stream is updated in place
 and normalised in one pass.  ``norm_add`` is the other way round, for blocks that norm a
 branch's output instead of its input: residual += norm(branch), again one pass.  ``sum_norm`` is
 for blocks that norm the stream itself after the branch has joined it: residual = norm(a * residual +
-branch), with an optional weight per element on the branch (a layer scale), one pass too.
+branch), with an optional weight per element on the branch (a layer scale), one pass too.  ``streams_norm`` is for a
+stream kept as several copies: it mixes them, adds the branch, and norms the sum that the next branch reads, one pass again.
 """
 from __future__ import annotations
 
@@ -16,7 +17,7 @@ from typing import Dict, Mapping, Optional
 import torch
 
 from ..weights.loader import TensorSpec
-from .base import ExpertRows, Norm, NormedBranch, NormedSum, PlusRow, Runtime, Settled, register_norm
+from .base import ExpertRows, Norm, NormedBranch, NormedSum, PlusRow, Runtime, Settled, StreamMix, register_norm
 
 
 @register_norm("rmsnorm")
@@ -90,7 +91,20 @@ class RMSNorm(Norm):
         return self.rt.ops.sum_norm(residual, terms, scale, self.branch_weight, residual_scale, self.weight, self.eps,
                                     self.unit_offset, self.rt.act_dtype)
 
+    def streams_norm(self, residual, delta, read, rows=None):
+        if delta is not None and not isinstance(delta, StreamMix):
+            raise TypeError(f"a stream kept as copies takes contributions that say how they mix, got {type(delta).__name__}")
+        y, mix, out = (None, None, None) if delta is None else (delta.inner, delta.mix, delta.out)
+        experts = None
+        if isinstance(y, NormedSum):
+            y = y.combine()
+        if isinstance(y, ExpertRows):
+            y, experts = y.dense, (y.rows, y.top, y.weight, y.row_weights)
+        return self.rt.ops.streams_norm(residual, y, experts, mix, out, read, rows, self.weight, self.eps, self.unit_offset, self.rt.act_dtype)
+
     def gather_add_norm(self, residual, delta, rows):
+        if residual.dim() == 3:  # copies of the stream: the final norm reads their sum
+            return self.streams_norm(residual, delta, None, rows)
         if isinstance(delta, PlusRow):
             delta = delta.settle(residual)
         if isinstance(delta, NormedBranch):
