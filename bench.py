@@ -44,6 +44,10 @@ size.
 mixing, norms after the sums, dense feed-forwards) beside the Nutavik configuration of equal width, heads and
 feed-forward weights (the closest of the engine's models: the same scan of matrix states) and the Llama configuration of
 equal size.
+``--design zimupel`` measures the Zimupel design (differential attention, retention and lightning attention on a stream kept
+as several copies, dense and routed feed-forwards) beside the Mesolix configuration of equal width, heads, state sizes and
+feed-forwards (the closest of the engine's models: a matrix-state recurrence, attention and routed experts) and the Llama
+configuration of equal size.
 """
 import argparse
 import json
@@ -434,12 +438,13 @@ def _op_costs(ops, hb):
 
     def attention(a, kw, out):
         qkv, heads, kv, d = a[0], a[1], a[2], a[3]
+        maps = 2 if kw.get("differential") is not None else 1  # (query rows come per map: half of each is zeros)
         chunked = kw.get("chunked", False)
         keys = visible(a[8], 0, chunked)
         b = hb()
         # (chunks: a request's queries read from the first one's chunk on)
         cached = [c - (c - q) // a[8] * a[8] if chunked else c for c, q in zip(b.seq_ctx.tolist(), b.seq_qlen.tolist())]
-        return 4.0 * heads * d * keys, 4.0 * kv * d * sum(cached) + 4.0 * qkv.shape[0] * heads * d
+        return (2.0 / maps + 2.0) * heads * d * keys, 4.0 * kv * d * sum(cached) + 4.0 * qkv.shape[0] * heads // maps * d
 
     def rglru(a, kw, out):
         u, wa = a[0], a[3]
@@ -458,6 +463,25 @@ def _op_costs(ops, hb):
         qkv, heads, dim, vdim, state = a[0], a[1], a[3], a[4], a[5]
         b = hb()
         return 6.0 * qkv.shape[0] * heads * dim * vdim, float(nbytes(qkv, out) + 8.0 * b.n_seqs * heads * dim * vdim)
+
+    def fixed_decay_scan(a, kw, out):
+        # q, k and v of every token, the read-outs, and every request's matrices read and written
+        proj, heads, dim, vdim = a[0], a[1], a[2], a[3]
+        return (6.0 * proj.shape[0] * heads * dim * vdim,
+                float(proj.shape[0] * heads * (2 * dim + vdim) * proj.element_size() + nbytes(out) + 8.0 * hb().n_seqs * heads * dim * vdim))
+
+    def gated_head_norm(a, kw, out):
+        return 0.0, float(nbytes(a[0], out) + out.numel() * a[3].element_size())
+
+    def streams_norm(a, kw, out):
+        # the copies read and (where a branch joins and nothing is picked) written, the branch's parts, the normed rows
+        residual, y, experts, mix, rows = a[0], a[1], a[2], a[3], a[6]
+        picked = 1.0 if rows is None else rows.numel() / residual.shape[0]
+        branch = nbytes(getattr(y, "tensor", y)) + (nbytes(experts[0]) if experts is not None else 0)
+        return 0.0, float(picked * (nbytes(residual) * (2 if mix is not None and rows is None else 1) + branch) + nbytes(out))
+
+    def embed_norm(a, kw, out):
+        return 0.0, float(a[0].numel() * a[1].shape[1] * a[1].element_size() + nbytes(out))
 
     def grouped_linear(a, kw, out):
         x, w = a[0], a[1]
@@ -491,10 +515,11 @@ def _op_costs(ops, hb):
             "rglru": rglru, "norm_add": moved, "add_rmsnorm": moved, "gather_add_rmsnorm": moved, "qkv_prepare": moved,
             "rope_append": moved, "causal_conv": moved, "gated_act": moved, "round_rows": moved, "embed": embed,
             "sandwich_norm": moved, "activation": moved, "latent_prepare": moved, "head_linear": head_linear,
-            "latent_attention": latent_attention, "linear_state_scan": state_scan, "gated_head_norm": moved, "conv_state_push": moved, "moe_router_topk": moved,
+            "latent_attention": latent_attention, "linear_state_scan": state_scan, "gated_head_norm": gated_head_norm, "conv_state_push": moved, "moe_router_topk": moved,
             "moe_combine": moved, "attention_finish": moved, "qk_row_scales": moved,
             "grouped_linear": grouped_linear, "low_rank": low_rank, "sum_norm": sum_norm, "token_shift_mix": token_shift_mix,
-            "embed_pairs": embed_pairs, "rmsnorm": moved}
+            "embed_pairs": embed_pairs, "rmsnorm": moved, "fixed_decay_scan": fixed_decay_scan, "streams_norm": streams_norm,
+            "embed_norm": embed_norm, "moe_router_share": moved, "scale_rows": moved}
 
 
 def per_op_times(runner, vocab: int, gen, batch: int, prompt_len: int, prefill_len: int):
@@ -587,7 +612,7 @@ def design_compare(args) -> int:
     from yalis_amd.models.presets import layer_runs, llama_like, mesolix_like, nutavik_like
 
     sizes = {"suranex": ("suranex-2k", "suranex-4k"), "nutavik": ("nutavik-2k", "nutavik-4k"), "mesolix": ("mesolix-2k", "mesolix-4k"),
-             "bekedra": ("bekedra-2k", "bekedra-4k"), "rafusun": ("rafusun-2k", "rafusun-4k")}[args.design]
+             "bekedra": ("bekedra-2k", "bekedra-4k"), "rafusun": ("rafusun-2k", "rafusun-4k"), "zimupel": ("zimupel-2k", "zimupel-4k")}[args.design]
     if args.design_shape:
         sizes = (args.design_shape,)
     for name in sizes:
@@ -597,7 +622,7 @@ def design_compare(args) -> int:
         beside = [("design", cfg)]
         if args.design in ("mesolix", "rafusun"):
             beside.append(("nutavik_of_equal_size", nutavik_like(cfg)))
-        if args.design == "bekedra":
+        if args.design in ("bekedra", "zimupel"):
             beside.append(("mesolix_of_equal_size", mesolix_like(cfg)))
         beside.append(("llama_of_equal_size", llama_like(cfg)))
         for who, c in beside:
@@ -622,9 +647,9 @@ def design_compare(args) -> int:
 
 def main() -> int:
     ap = argparse.ArgumentParser()
-    ap.add_argument("--design", choices=("suranex", "nutavik", "mesolix", "bekedra", "rafusun"), default=None,
+    ap.add_argument("--design", choices=("suranex", "nutavik", "mesolix", "bekedra", "rafusun", "zimupel"), default=None,
                     help="measure instead another design's prefill and decode at a few layer sizes, beside the Llama configuration of equal size, with the time and the bound of every kind of kernel")
-    ap.add_argument("--design-shape", default=None, help="with --design: one of its shapes only (suranex-2k, suranex-4k, nutavik-2k, nutavik-4k, mesolix-2k, mesolix-4k, bekedra-2k, bekedra-4k, rafusun-2k, rafusun-4k)")
+    ap.add_argument("--design-shape", default=None, help="with --design: one of its shapes only (suranex-2k, suranex-4k, nutavik-2k, nutavik-4k, mesolix-2k, mesolix-4k, bekedra-2k, bekedra-4k, rafusun-2k, rafusun-4k, zimupel-2k, zimupel-4k)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=32)
     ap.add_argument("--warmup", type=int, default=4)

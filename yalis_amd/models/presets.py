@@ -5,6 +5,7 @@ and needs the checkpoint; here a name stands for the layer sizes alone).
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, Tuple
 
 LLAMA3_8B = {
@@ -132,6 +133,33 @@ def rafusun_shape(width: int, vocab: int, heads: int, kv_heads: int, dim: int, c
             "embedding": {"scale": float(width) ** 0.5, "bigram": {"buckets": buckets, "mul_prev": 1009, "mul_cur": 31}}, "layers": layers}
 
 
+def zimupel_shape(width: int, vocab: int, heads: int, kv_heads: int, dim: int, vdim: int, lightning_heads: int, lightning_dim: int,
+                  retention_heads: int, retention_dim: int, retention_vdim: int, ff: int, experts: int, top: int, expert_ff: int, groups: int,
+                  keep: int, streams: int = 4, pattern=("attention", "lightning", "retention"), repeats: int = 2) -> dict:
+    """A Zimupel config.json of the given layer sizes: the mixers of ``pattern`` repeated ``repeats`` times, dense and routed
+    feed-forwards in turn; attention layers after the first read the first one's keys and values."""
+    att = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "diff": 0.5}
+    mixers = {"attention": att,
+              "lightning": {"heads": lightning_heads, "dim": lightning_dim, "vdim": lightning_dim,
+                            "decay": [math.exp(-2.0 ** (-8.0 * (h + 1) / lightning_heads)) for h in range(lightning_heads)]},
+              "retention": {"heads": retention_heads, "dim": retention_dim, "vdim": retention_vdim, "rot": {"base": 10000.0, "dims": retention_dim},
+                            "decay": [1.0 - 2.0 ** (-5.0 - h * 5.0 / retention_heads) for h in range(retention_heads)]}}
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "router": {"experts": experts, "top": top, "groups": {"count": groups, "keep": keep}}, "expert": {"ff": expert_ff}}
+    layers = []
+    first_attention = None
+    for i, kind in enumerate(pattern * repeats):
+        mixer = dict(mixers[kind])
+        if kind == "attention":
+            if first_attention is not None:
+                mixer["kv_from"] = first_attention
+            else:
+                first_attention = i
+        layers.append({"type": kind, "mixer": mixer, "mlp": dict(dense if i % 2 == 0 else moe)})
+    return {"architecture": "Zimupel", "vocab": vocab, "width": width, "streams": streams, "norm": {"eps": 1e-6}, "logit_scale": 0.5,
+            "logit_softcap": 20.0, "layers": layers}
+
+
 def layer_runs(design: dict) -> int:
     """How many layers a token passes through (a looped stretch counts every pass)."""
     loop = design.get("loop")
@@ -145,6 +173,14 @@ def llama_like(design: dict) -> dict:
     (its top experts and the shared one).  For Nutavik: the same width, layer count, vocabulary and
     attention heads (keys as wide as its unrotated and rotated parts together, a quarter as many key
     heads), a gated feed-forward with as many weights as its dense one (two thirds as wide)."""
+    if design.get("architecture") == "Zimupel":
+        # the same width, layer count, vocabulary and attention heads (both maps of a head together one head); a feed-forward with
+        # as many weights as the mean of what a token uses of the dense and the routed ones
+        att = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "attention")
+        used = [f["ff"] if f["kind"] == "dense" else f["router"]["top"] * f["expert"]["ff"] for f in (layer["mlp"] for layer in design["layers"]) if f]
+        inter = (sum(used) // max(len(used), 1) + 255) // 256 * 256
+        return dict(LLAMA3_8B, hidden_size=design["width"], num_hidden_layers=len(design["layers"]), num_attention_heads=att["heads"],
+                    num_key_value_heads=att["kv_heads"], head_dim=2 * att["dim"], intermediate_size=inter, vocab_size=design["vocab"])
     if design.get("architecture") == "Rafusun":
         # the same width, layer count, vocabulary, attention heads and feed-forward
         att = next(layer["mixer"]["left"] for layer in design["layers"] if layer["type"] == "parallel")
@@ -211,8 +247,22 @@ def nutavik_like(design: dict) -> dict:
 
 
 def mesolix_like(design: dict) -> dict:
-    """The Mesolix configuration of a Bekedra one's size: the same width, vocabulary, heads and experts (no shared
-    expert), as many layers as a token passes through (in threes), a window as long as the benchmark's prompts."""
+    """The Mesolix configuration of a Bekedra or Zimupel one's size: the same width, vocabulary, heads and experts (no shared
+    expert), as many layers as a token passes through (in threes), a window as long as the benchmark's prompts.  For Zimupel
+    also the same dense feed-forward, and state-space layers with as many heads, keys and values as its lightning layers."""
+    if design.get("architecture") == "Zimupel":
+        att = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "attention")
+        rec = next(layer["mixer"] for layer in design["layers"] if layer["type"] == "lightning")
+        dense = next(layer["mlp"]["ff"] for layer in design["layers"] if layer["mlp"] and layer["mlp"]["kind"] == "dense")
+        f = next(layer["mlp"] for layer in design["layers"] if layer["mlp"] and layer["mlp"]["kind"] == "moe")
+        width = design["width"]
+        cfg = mesolix_shape(width, design["vocab"], att["heads"], att["kv_heads"], 2 * att["dim"], 512, 768 * width // 2048, 2048, rec["heads"], rec["vdim"],
+                            rec["dim"], max(1, rec["heads"] // 8), dense, f["router"]["experts"], f["router"]["top"], f["expert"]["ff"],
+                            f["expert"]["ff"], repeats=max(1, len(design["layers"]) // 3))
+        for layer in cfg["layers"]:
+            if layer["mlp"]["kind"] == "moe":
+                layer["mlp"].pop("shared", None)
+        return cfg
     att = design["layers"][0]["mixer"]
     f = next(layer["mlp"] for layer in design["layers"] if layer["mlp"] is not None)
     width = design["width"]
@@ -243,6 +293,11 @@ RAFUSUN_2K = rafusun_shape(2048, 32768, 16, 4, 128, 2048, 16, 8, 128, 32, 64, 56
 RAFUSUN_4K = rafusun_shape(4096, 65536, 32, 8, 128, 2048, 32, 16, 128, 64, 64, 11264, 131071, repeats=1)
 RAFUSUN_TINY = rafusun_shape(64, 256, 4, 2, 16, 24, 4, 2, 16, 3, 16, 96, 101, repeats=1)
 
+ZIMUPEL_2K = zimupel_shape(2048, 32768, 16, 4, 64, 128, 16, 128, 8, 256, 256, 8192, 16, 2, 1024, 4, 2)
+ZIMUPEL_4K = zimupel_shape(4096, 65536, 32, 8, 64, 128, 32, 128, 16, 256, 256, 16384, 32, 4, 1024, 8, 4, repeats=1)
+ZIMUPEL_TINY = zimupel_shape(64, 256, 4, 2, 8, 16, 2, 16, 3, 16, 24, 96, 6, 2, 32, 3, 2, streams=3, pattern=("attention", "lightning", "retention", "attention"),
+                             repeats=1)
+
 # name -> (what to call it, config.json dictionary)
 SHAPES: Dict[str, Tuple[str, dict]] = {
     "8b": ("Llama-3-8B", LLAMA3_8B),
@@ -266,6 +321,9 @@ SHAPES: Dict[str, Tuple[str, dict]] = {
     "rafusun-2k": ("Rafusun, width 2,048", RAFUSUN_2K),
     "rafusun-4k": ("Rafusun, width 4,096", RAFUSUN_4K),
     "rafusun-tiny": ("tiny Rafusun", RAFUSUN_TINY),
+    "zimupel-2k": ("Zimupel, width 2,048", ZIMUPEL_2K),
+    "zimupel-4k": ("Zimupel, width 4,096", ZIMUPEL_4K),
+    "zimupel-tiny": ("tiny Zimupel", ZIMUPEL_TINY),
 }
 
 
