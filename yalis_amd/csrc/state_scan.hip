@@ -806,6 +806,67 @@ __global__ __launch_bounds__(256) void gated_head_norm_kernel(const float* __res
     out[item * vdim + c] = from_f32<TO>(row[c] * inv * weight(c) * head_gate_act(to_f32<TG>(g[c]), gate_act));
 }
 
+// The same in pieces of four elements, a thread holding up to four of them: everything is asked for before the sum.  A wave a
+// part (four parts a workgroup) or, for parts of more than 1,024 elements, a workgroup a part.
+template <typename T>
+__device__ __forceinline__ float4 hn_load4(const T* p);
+template <>
+__device__ __forceinline__ float4 hn_load4<float>(const float* p) { return *reinterpret_cast<const float4*>(p); }
+template <>
+__device__ __forceinline__ float4 hn_load4<bf16_t>(const bf16_t* p) {
+  const uint2 w = *reinterpret_cast<const uint2*>(p);
+  return make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16), __uint_as_float(w.y & 0xffff0000u));
+}
+__device__ __forceinline__ void hn_store4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+__device__ __forceinline__ void hn_store4(bf16_t* p, float4 v) { *reinterpret_cast<uint2*>(p) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w)); }
+
+template <typename TW, typename TG, typename TO, bool WAVE>
+__global__ __launch_bounds__(256) void gated_head_norm_vec_kernel(const float* __restrict__ o, const TW* __restrict__ w, float eps,
+                                                                  const TG* __restrict__ gate, int gate_stride, int gate_col, int n_heads,
+                                                                  int vdim, TO* __restrict__ out, size_t total, int w_stride, int gate_first,
+                                                                  int gate_act) {
+  __shared__ float scratch[17];
+  constexpr int T = WAVE ? kWave : 256, P = 4;
+  const size_t wanted = WAVE ? blockIdx.x * static_cast<size_t>(4) + threadIdx.x / kWave : blockIdx.x;
+  if (WAVE && wanted >= total) return;  // (a whole wave)
+  const size_t item = wanted;
+  const int t = threadIdx.x % T;
+  const size_t n = item / n_heads;
+  const int h = static_cast<int>(item % n_heads);
+  const float* row = o + item * vdim;
+  const TG* g = gate + n * gate_stride + gate_col + h * vdim;
+  float4 v[P], a[P], m[P];
+  float ss = 0.f;
+#pragma unroll
+  for (int p = 0; p < P; ++p) {
+    const int c = 4 * (t + p * T);
+    v[p] = a[p] = make_float4(0.f, 0.f, 0.f, 0.f);
+    m[p] = make_float4(1.f, 1.f, 1.f, 1.f);
+    if (c < vdim) {
+      v[p] = hn_load4<float>(row + c);
+      a[p] = hn_load4<TG>(g + c);
+      if (w != nullptr) m[p] = hn_load4<TW>(w + static_cast<size_t>(h) * w_stride + c);
+    }
+  }
+#pragma unroll
+  for (int p = 0; p < P; ++p) {
+    a[p] = make_float4(head_gate_act(a[p].x, gate_act), head_gate_act(a[p].y, gate_act), head_gate_act(a[p].z, gate_act), head_gate_act(a[p].w, gate_act));
+    if (gate_first) v[p] = make_float4(v[p].x * a[p].x, v[p].y * a[p].y, v[p].z * a[p].z, v[p].w * a[p].w);
+    ss = fmaf(v[p].x, v[p].x, fmaf(v[p].y, v[p].y, fmaf(v[p].z, v[p].z, fmaf(v[p].w, v[p].w, ss))));
+  }
+  ss = WAVE ? wave_sum(ss) : block_sum(ss, scratch);
+  const float inv = 1.f / sqrtf(ss / static_cast<float>(vdim) + eps);
+#pragma unroll
+  for (int p = 0; p < P; ++p) {
+    const int c = 4 * (t + p * T);
+    if (c < vdim) {
+      float4 y = make_float4(v[p].x * inv * m[p].x, v[p].y * inv * m[p].y, v[p].z * inv * m[p].z, v[p].w * inv * m[p].w);
+      if (!gate_first) y.x *= a[p].x, y.y *= a[p].y, y.z *= a[p].z, y.w *= a[p].w;
+      hn_store4(out + item * vdim + c, y);
+    }
+  }
+}
+
 extern "C" int yk_gated_head_norm(const float* o, const void* w, int w_dtype, float eps, const void* gate, int gate_dtype,
                                   int gate_stride, int gate_col, int n_heads, int vdim, void* out, int out_dtype, int n_tokens,
                                   int w_per_part, int gate_first, int gate_act, hipStream_t stream) {
@@ -816,8 +877,19 @@ extern "C" int yk_gated_head_norm(const float* o, const void* w, int w_dtype, fl
   const size_t total = static_cast<size_t>(n_tokens) * n_heads;
   const int grid = static_cast<int>((total + 3) / 4);
   const int w_stride = w_per_part ? vdim : 0;
+  auto al16 = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+  const bool vec = vdim % 4 == 0 && vdim <= 4096 && gate_stride % 4 == 0 && gate_col % 4 == 0 && al16(o) && al16(w) && al16(gate) && al16(out);
 #define YK_CASE(WD, TW, GD, TG, OD, TO)                                                                               \
   if (w_dtype == WD && gate_dtype == GD && out_dtype == OD) {                                                         \
+    if (vec && vdim > 1024)                                                                                           \
+      gated_head_norm_vec_kernel<TW, TG, TO, false><<<static_cast<unsigned>(total), 256, 0, stream>>>(                \
+          o, static_cast<const TW*>(w), eps, static_cast<const TG*>(gate), gate_stride, gate_col, n_heads, vdim,      \
+          static_cast<TO*>(out), total, w_stride, gate_first, gate_act);                                              \
+    else if (vec)                                                                                                     \
+      gated_head_norm_vec_kernel<TW, TG, TO, true><<<grid, 256, 0, stream>>>(                                         \
+          o, static_cast<const TW*>(w), eps, static_cast<const TG*>(gate), gate_stride, gate_col, n_heads, vdim,      \
+          static_cast<TO*>(out), total, w_stride, gate_first, gate_act);                                              \
+    else                                                                                                              \
     gated_head_norm_kernel<TW, TG, TO><<<grid, 256, 0, stream>>>(o, static_cast<const TW*>(w), eps,                   \
                                                                  static_cast<const TG*>(gate), gate_stride, gate_col, \
                                                                  n_heads, vdim, static_cast<TO*>(out), total, w_stride, \

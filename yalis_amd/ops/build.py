@@ -30,7 +30,7 @@ HOST_SOURCES = ["cache_manager.cpp"]
 KERNEL_LIBS = {
     "kernels": ["runtime.hip", "elementwise.hip", "gemm.hip", "gemm_tile.hip", "attention.hip", "library_gemm.hip",
                 "branch.hip", "attention_masked.hip", "recurrent.hip", "moe.hip", "sandwich_norm.hip", "latent_attention.hip",
-                "state_scan.hip", "time_mix.hip", "streams.hip"],
+                "state_scan.hip", "time_mix.hip", "streams.hip", "decay_scan.hip"],
     "sampling": ["runtime.hip", "sampling.hip"],
     "probe": ["runtime.hip", "probe.hip"],
 }

@@ -121,6 +121,17 @@ _SIGNATURES = {
         [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_float, _c_int, _vp, _c_int, _vp],
         _c_int,
     ),
+    "yk_decay_scan_chunks_ok": ([_c_int, _c_int, _c_int, _c_int], _c_int),
+    "yk_decay_scan_chunks_bytes": ([_c_int, _c_int, _c_int, _c_int, _c_int, _c_int], _c_size_t),
+    "yk_decay_scan_chunks": (
+        [_vp, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _c_int, _vp, _c_int, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_float, _c_int,
+         _vp, _vp, _c_size_t, _vp, _vp],
+        _c_int,
+    ),
+    "yk_decay_scan_step": (
+        [_vp, _c_int, _c_int, _c_int, _c_int, _c_int, _vp, _vp, _vp, _c_int, _vp, _vp, _vp, _c_int, _c_int, _c_int, _c_float, _c_int, _vp, _vp, _vp],
+        _c_int,
+    ),
     "yk_moe_router_share": ([_vp, _c_int, _c_int, _c_int, _vp, _vp, _c_int, _c_int, _vp, _vp, _c_int, _vp], _c_int),
     "yk_latent_prepare": (
         [_vp, _c_int, _c_int, _c_int, _vp, _c_int, _c_float, _vp, _c_int, _c_int, _c_int, _vp, _vp, _vp, _vp, _c_int, _c_int, _vp, _vp,
@@ -1855,12 +1866,61 @@ class HipOps:
             self._stream()))
         return out
 
-    def fixed_decay_scan(self, proj, n_heads, dim, vdim, state, ctx, decay, k_scale=1.0, rotation=None, act=None, chunks=None, seq_chunk0=None):
+    # scratch for the sums of a step's chunks (a few hundred chunks at these sizes; more are taken slab by slab)
+    DECAY_SLAB_BYTES = 256 << 20
+
+    def fixed_decay_scan(self, proj, n_heads, dim, vdim, state, ctx, decay, k_scale=1.0, rotation=None, act=None, chunks=None, seq_chunk0=None,
+                         form: Optional[str] = None):
         """The recurrence S <- a_h S + k v^T, o = S^T q with a constant decay per head (``decay`` float32 [heads]) over each
         request's span, S [slots, heads, dim, vdim] float32 updated in place.  ``proj`` [N, >= heads * (2 * dim + vdim)]: columns
-        [q | k | v | ...] as projected; see ``scan_inputs`` for what is made of them first.  Returns o float32 [N, heads * vdim]."""
-        rows = self.scan_inputs(proj, n_heads, dim, vdim, k_scale, rotation, ctx.arrays["positions"], act)
-        return self.linear_state_scan(rows, n_heads, n_heads, dim, vdim, state, ctx, decay=("fixed", decay))
+        [q | k | v | ...] as projected; see ``scan_inputs`` for what is made of them first.  Returns o float32 [N, heads * vdim].
+
+        Steps of single tokens take a kernel of their own; spans in bfloat16 the matrix cores, chunk by chunk (``chunks`` and
+        ``seq_chunk0``: ``span_chunks`` and ``chunk_starts`` of ``FIXED_DECAY_CHUNK`` tokens), where the sizes allow; what is left
+        is walked token by token.  ``form`` ("step", "chunks", "walk") forces one of them (tests, measurements)."""
+        self._rows(proj, "fixed_decay_scan input")
+        if act not in (None, "silu"):
+            raise KernelError(f"fixed_decay_scan: activation {act!r} is not offered")
+        n = proj.shape[0]
+        a = ctx.arrays
+        positions, n_seqs = a["positions"], a["seq_qstart"].numel()
+        if state.dtype != torch.float32 or not state.is_contiguous() or tuple(state.shape[1:]) != (n_heads, dim, vdim):
+            raise KernelError(f"fixed_decay_scan: state {tuple(state.shape)} does not hold {n_heads} matrices of {dim} x {vdim}")
+        if decay.dtype != torch.float32 or decay.numel() != n_heads or not decay.is_contiguous() or positions.numel() != n:
+            raise KernelError("fixed_decay_scan: the decays are contiguous float32 [heads], and every token has a position")
+        if proj.shape[1] < n_heads * (2 * dim + vdim):
+            raise KernelError(f"fixed_decay_scan: rows of {proj.shape[1]} elements, fewer than the heads need")
+        r = rotation
+        if r is not None and (r.cos.dtype != torch.float32 or r.cos.shape != r.sin.shape or r.cos.shape[1] != r.rotary_dim // 2):
+            raise KernelError("fixed_decay_scan: rotary tables are float32 [positions, rotary_dim/2]")
+        rot, inter, rows = (0, 0, 0) if r is None else (r.rotary_dim, int(bool(r.interleaved)), r.cos.shape[0])
+        inputs = (None if r is None else r.cos.data_ptr(), None if r is None else r.sin.data_ptr(), rot, inter, rows, float(k_scale), int(act == "silu"))
+        can_step = ctx.max_qlen == 1 and vdim % 4 == 0 and dim <= 4096
+        can_chunk = (proj.dtype == torch.bfloat16 and chunks is not None and proj.stride(0) % 8 == 0 and proj.data_ptr() % 16 == 0
+                     and self._ask("yk_decay_scan_chunks_ok", dim, vdim, rot, inter) == 1)
+        if form is None:
+            form = "step" if can_step else ("chunks" if can_chunk else "walk")
+        if (form == "step" and not can_step) or (form == "chunks" and not can_chunk):
+            raise KernelError(f"fixed_decay_scan: this step cannot take the form {form!r}")
+        if form == "walk":
+            x = self.scan_inputs(proj, n_heads, dim, vdim, k_scale, rotation, positions, act)
+            return self.linear_state_scan(x, n_heads, n_heads, dim, vdim, state, ctx, decay=("fixed", decay))
+        out = torch.empty((n, n_heads * vdim), dtype=torch.float32, device=proj.device)
+        if form == "step":
+            self._check(self.lib.yk_decay_scan_step(
+                proj.data_ptr(), proj.stride(0), _code(proj.dtype), n_heads, dim, vdim, state.data_ptr(), a["seq_qstart"].data_ptr(),
+                a["state_slots"].data_ptr(), n_seqs, positions.data_ptr(), *inputs, decay.data_ptr(), out.data_ptr(), self._stream()))
+            return out
+        n_chunks = chunks.shape[0]
+        if seq_chunk0 is None or seq_chunk0.numel() != n_seqs + 1 or chunks.shape[1] != 3:
+            raise KernelError("fixed_decay_scan: chunks are rows of (request, first token, count), with every request's first row")
+        slab = max(1, min(n_chunks, self.DECAY_SLAB_BYTES // (4 * n_heads * dim * vdim)))
+        need = int(self.lib.yk_decay_scan_chunks_bytes(n_chunks, slab, n_heads, dim, vdim, int(act == "silu")))
+        ws = torch.empty(need, dtype=torch.uint8, device=proj.device)
+        self._check(self.lib.yk_decay_scan_chunks(
+            proj.data_ptr(), proj.stride(0), n_heads, dim, vdim, state.data_ptr(), a["state_slots"].data_ptr(), n_seqs, chunks.data_ptr(), n_chunks,
+            seq_chunk0.data_ptr(), slab, positions.data_ptr(), *inputs, decay.data_ptr(), ws.data_ptr(), need, out.data_ptr(), self._stream()))
+        return out
 
     def gated_head_norm(self, o, weight, eps, gate, gate_col, n_heads, vdim, out_dtype, gate_first: bool = False,
                         gate_act: str = "silu") -> torch.Tensor:
