@@ -127,64 +127,62 @@ __device__ __forceinline__ void enter8(const bf16_t* row, int p, int pos, const 
 }  // namespace
 
 // ---------------------------------------------------------------------------------------- chunks: prepare
-// A workgroup a (chunk, head).  q_ws, k_ws [chunk][head][64][dim], kt_ws [chunk][head][dim][64], pairs of 8; vt_ws
-// [chunk][head][vdim][64], pairs of 8 or (VLO false) hi alone.  Places beyond the chunk's tokens are zeros.
+// A workgroup a (chunk, head, block of 64 channels of q, of k or of v).  q_ws, k_ws [chunk][head][64][dim], kt_ws
+// [chunk][head][dim][64], pairs of 8; vt_ws [chunk][head][vdim][64], pairs of 8 or (VLO false) hi alone.  Places beyond the
+// chunk's tokens are zeros.
+constexpr int kPrepare = 64;  // channels of a workgroup
 template <bool VLO>
 __global__ __launch_bounds__(256) void decay_prepare_kernel(const bf16_t* __restrict__ src, int src_stride, int n_heads, int dim, int vdim,
                                                             const float* __restrict__ decay, const int32_t* __restrict__ chunks, Inputs in,
                                                             bf16_t* __restrict__ q_ws, bf16_t* __restrict__ k_ws, bf16_t* __restrict__ kt_ws,
                                                             bf16_t* __restrict__ vt_ws) {
-  extern __shared__ float buf[];  // [64][max(dim, vdim) + 1], then the decay's powers [64]
+  __shared__ float buf[kChunk][kPrepare + 1];
+  __shared__ float power[kChunk];
   const int c = blockIdx.x, h = blockIdx.y;
   const int tok0 = chunks[3 * c + 1], n = chunks[3 * c + 2];
-  const int wide = max(dim, vdim) + 1;
-  float* power = buf + kChunk * wide;
-  if (threadIdx.x < kChunk) power[threadIdx.x] = powf(decay[h], static_cast<float>(threadIdx.x));
   const size_t slab = static_cast<size_t>(c) * n_heads + h;
-  const int pieces = dim / 8;
+  const int key_blocks = (dim + kPrepare - 1) / kPrepare;
+  const int what = min(static_cast<int>(blockIdx.z) / key_blocks, 2);  // 0: q, 1: k, 2: v
+  const int c0 = (blockIdx.z - what * key_blocks) * kPrepare;            // its first channel
+  const int width = what == 2 ? vdim : dim, here = min(kPrepare, width - c0), pieces = here / 8;
+  const bf16_t* col = src + (what == 2 ? 2 * n_heads * dim + h * vdim : what * n_heads * dim + h * dim);
+  if (what == 1 && threadIdx.x < kChunk) power[threadIdx.x] = powf(decay[h], static_cast<float>(threadIdx.x));
   for (int i = threadIdx.x; i < kChunk * pieces; i += 256) {
-    const int t = i / pieces, p = i % pieces;
-    float q[8], k[8];
-    if (t < n) {
-      const bf16_t* row = src + static_cast<size_t>(tok0 + t) * src_stride + h * dim;
-      const int pos = in.positions[tok0 + t];
-      enter8(row, p, pos, in, 1.f, q);
-      enter8(row + n_heads * dim, p, pos, in, in.k_scale, k);
-    } else {
-#pragma unroll
-      for (int e = 0; e < 8; ++e) q[e] = k[e] = 0.f;
-    }
-    const size_t at = ((slab * kChunk + t) * pieces + p) * 16;
-    store_pair(q_ws + at, q);
-    store_pair(k_ws + at, k);
-#pragma unroll
-    for (int e = 0; e < 8; ++e) buf[t * wide + 8 * p + e] = k[e];
-  }
-  __syncthreads();
-  for (int i = threadIdx.x; i < dim * (kChunk / 8); i += 256) {
-    const int d = i % dim, p = i / dim;
-    float v[8];
-#pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = 8 * p + e < n ? buf[(8 * p + e) * wide + d] * power[n - 1 - (8 * p + e)] : 0.f;
-    store_pair(kt_ws + ((slab * dim + d) * (kChunk / 8) + p) * 16, v);
-  }
-  __syncthreads();
-  const int v_pieces = vdim / 8;
-  for (int i = threadIdx.x; i < kChunk * v_pieces; i += 256) {
-    const int t = i / v_pieces, p = i % v_pieces;
+    const int t = i / pieces, p = c0 / 8 + i % pieces;
     float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (t < n) load8<bf16_t>(src + static_cast<size_t>(tok0 + t) * src_stride + 2 * n_heads * dim + h * vdim + 8 * p, v);
+    if (t < n) {
+      const bf16_t* row = col + static_cast<size_t>(tok0 + t) * src_stride;
+      if (what == 2) {
+        load8<bf16_t>(row + 8 * p, v);
+        if (VLO) {
 #pragma unroll
-    for (int e = 0; e < 8; ++e) buf[t * wide + 8 * p + e] = VLO ? act_silu(v[e]) : v[e];
+          for (int e = 0; e < 8; ++e) v[e] = act_silu(v[e]);
+        }
+      } else {
+        enter8(row, p, in.positions[tok0 + t], in, what == 1 ? in.k_scale : 1.f, v);
+      }
+    }
+    if (what != 2) store_pair((what == 0 ? q_ws : k_ws) + ((slab * kChunk + t) * (dim / 8) + p) * 16, v);
+    if (what != 0) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) buf[t][8 * p - c0 + e] = v[e];
+    }
   }
+  if (what == 0) return;
   __syncthreads();
-  for (int i = threadIdx.x; i < vdim * (kChunk / 8); i += 256) {
-    const int d = i % vdim, p = i / vdim;
+  // transposed: lanes side by side over a channel's pieces of eight tokens, so that a channel's row is written whole
+  for (int i = threadIdx.x; i < here * (kChunk / 8); i += 256) {
+    const int d = i / (kChunk / 8), p = i % (kChunk / 8);
     float v[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = buf[(8 * p + e) * wide + d];
-    const size_t at = (slab * vdim + d) * (kChunk / 8) + p;
-    if (VLO) {
+    for (int e = 0; e < 8; ++e) {
+      const int t = 8 * p + e;
+      v[e] = what == 2 ? buf[t][d] : (t < n ? buf[t][d] * power[n - 1 - t] : 0.f);
+    }
+    const size_t at = (slab * width + c0 + d) * (kChunk / 8) + p;
+    if (what == 1) {
+      store_pair(kt_ws + at * 16, v);
+    } else if (VLO) {
       store_pair(vt_ws + at * 16, v);
     } else {
       u32x4_t hi, lo;
@@ -290,7 +288,7 @@ __global__ __launch_bounds__(256) void decay_across_kernel(float* __restrict__ w
 }
 
 // ---------------------------------------------------------------------------------------- chunks: out
-// o of a (chunk, head).  A wave owns CT tiles of 16 tokens (the columns) and, with CT = 2, every other tile of 16 value
+// o of a (chunk, head), the tiles of value channels dealt out over gridDim.z workgroups.  A wave owns CT tiles of 16 tokens (the columns) and, with CT = 2, every other tile of 16 value
 // channels: out^T = (S^T q a^(i+1)) + v^T P^T with P^T[j][i] = a^(i-j) k_j . q_i.  The 16 rows of the two score products of a
 // group of 32 keys stand for keys 8 (row / 4) + row % 4 and 4 more, so that afterwards lane group g holds keys 8g .. 8g+7 in
 // order, as the second product's operand wants them.
@@ -304,7 +302,8 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
   const int tok0 = chunks[3 * (chunk0 + c) + 1], n = chunks[3 * (chunk0 + c) + 2];
   if (threadIdx.x <= kChunk) power[threadIdx.x] = powf(decay[h], static_cast<float>(threadIdx.x));
   __syncthreads();
-  const int col0 = 16 * CT * (wave / CT), e_first = wave % CT;  // first token of this wave; its first tile of value channels
+  const int col0 = 16 * CT * (wave / CT);  // first token of this wave
+  const int e_first = (wave % CT) * gridDim.z + blockIdx.z, e_step = CT * gridDim.z;  // its tiles of value channels
   if (col0 >= n) return;
   const size_t slab = static_cast<size_t>(chunk0 + c) * n_heads + h;
   const bf16_t* q = q_ws + slab * kChunk * dim * 2;
@@ -349,30 +348,43 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
   float before[CT];  // what the memory before the chunk has decayed to at the column's token
 #pragma unroll
   for (int t = 0; t < CT; ++t) before[t] = power[col0 + 16 * t + r + 1];
-  for (int et = e_first; et < vdim / 16; et += CT) {
+  // (a tile's memory and values are asked for while the tile before is worked on)
+  const int n_e = vdim / 16;
+  Pair sf[KS], vf[2];
+  auto ask = [&](int et) {
+    const bf16_t* srow = st + static_cast<size_t>(16 * et + r) * pieces * 16;
+#pragma unroll
+    for (int ks = 0; ks < KS; ++ks) sf[ks] = load_pair(srow + (4 * ks + g) * 16);
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      const bf16_t* p = vt + (static_cast<size_t>(16 * et + r) * (kChunk / 8) + 4 * u + g) * (VLO ? 16 : 8);
+      vf[u].hi.u = *reinterpret_cast<const u32x4_t*>(p);
+      if (VLO) vf[u].lo.u = *reinterpret_cast<const u32x4_t*>(p + 8);
+    }
+  };
+  if (e_first < n_e) ask(e_first);
+  for (int et = e_first; et < n_e; et += e_step) {
     f32x4_t acc[CT];
 #pragma unroll
     for (int t = 0; t < CT; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    const bf16_t* srow = st + static_cast<size_t>(16 * et + r) * pieces * 16;
+    Pair s_now[KS], v_now[2];
 #pragma unroll
-    for (int ks = 0; ks < KS; ++ks) {
-      const Pair a = load_pair(srow + (4 * ks + g) * 16);
+    for (int ks = 0; ks < KS; ++ks) s_now[ks] = sf[ks];
+    v_now[0] = vf[0], v_now[1] = vf[1];
+    if (et + e_step < n_e) ask(et + e_step);
 #pragma unroll
-      for (int t = 0; t < CT; ++t) acc[t] = mma_pairs(a, qf[t][ks], acc[t]);
-    }
+    for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+      for (int t = 0; t < CT; ++t) acc[t] = mma_pairs(s_now[ks], qf[t][ks], acc[t]);
 #pragma unroll
     for (int t = 0; t < CT; ++t) acc[t] *= before[t];
 #pragma unroll
     for (int u = 0; u < 2; ++u)
       if (u < groups) {
-        const bf16_t* p = vt + (static_cast<size_t>(16 * et + r) * (kChunk / 8) + 4 * u + g) * (VLO ? 16 : 8);
-        Pair a;
-        a.hi.u = *reinterpret_cast<const u32x4_t*>(p);
-        if (VLO) a.lo.u = *reinterpret_cast<const u32x4_t*>(p + 8);
 #pragma unroll
         for (int t = 0; t < CT; ++t) {
-          acc[t] = mma(a.hi, pf[t][u].lo, mma(a.hi, pf[t][u].hi, acc[t]));
-          if (VLO) acc[t] = mma(a.lo, pf[t][u].hi, acc[t]);
+          acc[t] = mma(v_now[u].hi, pf[t][u].lo, mma(v_now[u].hi, pf[t][u].hi, acc[t]));
+          if (VLO) acc[t] = mma(v_now[u].lo, pf[t][u].hi, acc[t]);
         }
       }
 #pragma unroll
@@ -383,6 +395,11 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
     }
   }
 }
+
+// How many workgroups share a (chunk, head)'s value channels in the last kernel (each makes the scores again): two where one
+// each leaves compute units without enough waves (8 heads of 256 x 256, 2,048 tokens: 135 us the whole scan with one, 126 with
+// two, 137 with four; 16 heads of 128 x 128: 81, 92, 113).
+static int decay_out_shares(int workgroups, int dim) { return dim == 256 && workgroups <= 512 ? 2 : 1; }
 
 // Whether the chunks' kernels take these sizes (bfloat16 rows; the rest of the spans go to the plain scan).
 extern "C" int yk_decay_scan_chunks_ok(int dim, int vdim, int rot, int interleaved) {
@@ -416,18 +433,15 @@ extern "C" int yk_decay_scan_chunks(const void* src, int src_stride, int n_heads
   bf16_t* kt_ws = k_ws + rows;
   bf16_t* vt_ws = kt_ws + rows;
   float* w_ws = reinterpret_cast<float*>(q_ws + decay_operand_elems(n_chunks, n_heads, dim, vdim, silu));
-  const size_t lds = (static_cast<size_t>(kChunk) * (std::max(dim, vdim) + 1) + kChunk) * sizeof(float);
-  const dim3 all(n_chunks, n_heads);
   {
+    const dim3 grid(n_chunks, n_heads, 2 * ((dim + kPrepare - 1) / kPrepare) + (vdim + kPrepare - 1) / kPrepare);
     auto kern = silu ? decay_prepare_kernel<true> : decay_prepare_kernel<false>;
-    if (lds > 64 * 1024 && hipFuncSetAttribute(reinterpret_cast<const void*>(kern), hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(lds)) != hipSuccess)
-      return yk_fail("decay_scan_chunks: a chunk's rows do not fit in LDS");
-    kern<<<all, 256, lds, stream>>>(static_cast<const bf16_t*>(src), src_stride, n_heads, dim, vdim, decay, chunks, in, q_ws, k_ws, kt_ws, vt_ws);
+    kern<<<grid, 256, 0, stream>>>(static_cast<const bf16_t*>(src), src_stride, n_heads, dim, vdim, decay, chunks, in, q_ws, k_ws, kt_ws, vt_ws);
     if (yk_check_launch("decay_prepare")) return -1;
   }
   for (int c0 = 0; c0 < n_chunks; c0 += slab_chunks) {
     const int nc = std::min(slab_chunks, n_chunks - c0);
-    const dim3 grid(nc, n_heads);
+    const dim3 grid(nc, n_heads), out_grid(nc, n_heads, decay_out_shares(nc * n_heads, dim));
     if (silu) decay_inside_kernel<true><<<grid, 256, 0, stream>>>(kt_ws, vt_ws, n_heads, dim, vdim, c0, w_ws);
     else decay_inside_kernel<false><<<grid, 256, 0, stream>>>(kt_ws, vt_ws, n_heads, dim, vdim, c0, w_ws);
     if (yk_check_launch("decay_inside")) return -1;
@@ -436,8 +450,8 @@ extern "C" int yk_decay_scan_chunks(const void* src, int src_stride, int n_heads
     if (yk_check_launch("decay_across")) return -1;
 #define YK_OUT(KS, CT)                                                                                                                \
   if (dim == 32 * KS) {                                                                                                               \
-    if (silu) decay_out_kernel<KS, CT, true><<<grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out); \
-    else decay_out_kernel<KS, CT, false><<<grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out);    \
+    if (silu) decay_out_kernel<KS, CT, true><<<out_grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out); \
+    else decay_out_kernel<KS, CT, false><<<out_grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out);    \
   }
     YK_OUT(1, 2)
     YK_OUT(2, 2)
