@@ -879,6 +879,7 @@ def moe_router_share(logits, top, experts=None, bias=None, correction=None, grou
 
 RefOps.embed_norm = staticmethod(embed_norm)
 RefOps.streams_norm = staticmethod(streams_norm)
+RefOps.fixed_decay_chunk = staticmethod(lambda: 64)
 RefOps.fixed_decay_scan = staticmethod(fixed_decay_scan)
 RefOps.moe_router_share = staticmethod(moe_router_share)
 RefOps.sum_norm = staticmethod(sum_norm)

@@ -288,7 +288,7 @@ __global__ __launch_bounds__(256) void decay_across_kernel(float* __restrict__ w
 }
 
 // ---------------------------------------------------------------------------------------- chunks: out
-// o of a (chunk, head), the tiles of value channels dealt out over gridDim.z workgroups.  A wave owns CT tiles of 16 tokens (the columns) and, with CT = 2, every other tile of 16 value
+// o of a (chunk, head).  A wave owns CT tiles of 16 tokens (the columns) and, with CT = 2, every other tile of 16 value
 // channels: out^T = (S^T q a^(i+1)) + v^T P^T with P^T[j][i] = a^(i-j) k_j . q_i.  The 16 rows of the two score products of a
 // group of 32 keys stand for keys 8 (row / 4) + row % 4 and 4 more, so that afterwards lane group g holds keys 8g .. 8g+7 in
 // order, as the second product's operand wants them.
@@ -302,8 +302,7 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
   const int tok0 = chunks[3 * (chunk0 + c) + 1], n = chunks[3 * (chunk0 + c) + 2];
   if (threadIdx.x <= kChunk) power[threadIdx.x] = powf(decay[h], static_cast<float>(threadIdx.x));
   __syncthreads();
-  const int col0 = 16 * CT * (wave / CT);  // first token of this wave
-  const int e_first = (wave % CT) * gridDim.z + blockIdx.z, e_step = CT * gridDim.z;  // its tiles of value channels
+  const int col0 = 16 * CT * (wave / CT), e_first = wave % CT;  // first token of this wave; its first tile of value channels
   if (col0 >= n) return;
   const size_t slab = static_cast<size_t>(chunk0 + c) * n_heads + h;
   const bf16_t* q = q_ws + slab * kChunk * dim * 2;
@@ -363,7 +362,7 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
     }
   };
   if (e_first < n_e) ask(e_first);
-  for (int et = e_first; et < n_e; et += e_step) {
+  for (int et = e_first; et < n_e; et += CT) {
     f32x4_t acc[CT];
 #pragma unroll
     for (int t = 0; t < CT; ++t) acc[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -371,7 +370,7 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks) s_now[ks] = sf[ks];
     v_now[0] = vf[0], v_now[1] = vf[1];
-    if (et + e_step < n_e) ask(et + e_step);
+    if (et + CT < n_e) ask(et + CT);
 #pragma unroll
     for (int ks = 0; ks < KS; ++ks)
 #pragma unroll
@@ -395,11 +394,6 @@ __global__ __launch_bounds__(256) void decay_out_kernel(const bf16_t* __restrict
     }
   }
 }
-
-// How many workgroups share a (chunk, head)'s value channels in the last kernel (each makes the scores again): two where one
-// each leaves compute units without enough waves (8 heads of 256 x 256, 2,048 tokens: 135 us the whole scan with one, 126 with
-// two, 137 with four; 16 heads of 128 x 128: 81, 92, 113).
-static int decay_out_shares(int workgroups, int dim) { return dim == 256 && workgroups <= 512 ? 2 : 1; }
 
 // Whether the chunks' kernels take these sizes (bfloat16 rows; the rest of the spans go to the plain scan).
 extern "C" int yk_decay_scan_chunks_ok(int dim, int vdim, int rot, int interleaved) {
@@ -441,7 +435,7 @@ extern "C" int yk_decay_scan_chunks(const void* src, int src_stride, int n_heads
   }
   for (int c0 = 0; c0 < n_chunks; c0 += slab_chunks) {
     const int nc = std::min(slab_chunks, n_chunks - c0);
-    const dim3 grid(nc, n_heads), out_grid(nc, n_heads, decay_out_shares(nc * n_heads, dim));
+    const dim3 grid(nc, n_heads);
     if (silu) decay_inside_kernel<true><<<grid, 256, 0, stream>>>(kt_ws, vt_ws, n_heads, dim, vdim, c0, w_ws);
     else decay_inside_kernel<false><<<grid, 256, 0, stream>>>(kt_ws, vt_ws, n_heads, dim, vdim, c0, w_ws);
     if (yk_check_launch("decay_inside")) return -1;
@@ -450,8 +444,8 @@ extern "C" int yk_decay_scan_chunks(const void* src, int src_stride, int n_heads
     if (yk_check_launch("decay_across")) return -1;
 #define YK_OUT(KS, CT)                                                                                                                \
   if (dim == 32 * KS) {                                                                                                               \
-    if (silu) decay_out_kernel<KS, CT, true><<<out_grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out); \
-    else decay_out_kernel<KS, CT, false><<<out_grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out);    \
+    if (silu) decay_out_kernel<KS, CT, true><<<grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out); \
+    else decay_out_kernel<KS, CT, false><<<grid, 256, 0, stream>>>(q_ws, k_ws, vt_ws, w_ws, chunks, c0, n_heads, vdim, decay, out);    \
   }
     YK_OUT(1, 2)
     YK_OUT(2, 2)

@@ -1844,7 +1844,10 @@ class HipOps:
             beta[0].data_ptr() if beta is not None and not beta_f32 else None, _ptr(bonus), _ptr(decays), self._stream()))
         return out
 
-    FIXED_DECAY_CHUNK = 64  # tokens of a span that meet in products
+    @staticmethod
+    def fixed_decay_chunk() -> int:
+        """Tokens of a span that meet in products in ``fixed_decay_scan``."""
+        return 64
 
     def scan_inputs(self, proj, n_heads, dim, vdim, k_scale=1.0, rotation=None, positions=None, act=None) -> torch.Tensor:
         """float32 rows [q | k | v] as they enter a recurrence, from a projection's rows [q | k | v | ...]: ``act`` ("silu") on all
@@ -1876,7 +1879,7 @@ class HipOps:
         [q | k | v | ...] as projected; see ``scan_inputs`` for what is made of them first.  Returns o float32 [N, heads * vdim].
 
         Steps of single tokens take a kernel of their own; spans in bfloat16 the matrix cores, chunk by chunk (``chunks`` and
-        ``seq_chunk0``: ``span_chunks`` and ``chunk_starts`` of ``FIXED_DECAY_CHUNK`` tokens), where the sizes allow; what is left
+        ``seq_chunk0``: ``span_chunks`` and ``chunk_starts`` of ``fixed_decay_chunk()`` tokens), where the sizes allow; what is left
         is walked token by token.  ``form`` ("step", "chunks", "walk") forces one of them (tests, measurements)."""
         self._rows(proj, "fixed_decay_scan input")
         if act not in (None, "silu"):

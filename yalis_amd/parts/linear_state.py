@@ -362,7 +362,7 @@ class _FixedDecayMixer(_MatrixStateMixer):
         self.decay = None
         self.qkv_cols = self.qk_cols + self.v_cols
         self.gate_col = self.qkv_cols + (-self.qkv_cols % 8)
-        self.chunk = int(getattr(rt.ops, "FIXED_DECAY_CHUNK", 64))  # tokens that meet in products
+        self.chunk = int(rt.ops.fixed_decay_chunk())  # tokens that meet in products
 
     def tensor_specs(self) -> Dict[str, TensorSpec]:
         specs = self._common_specs()
